@@ -1,4 +1,4 @@
-// Internal interface of the grouped/dense GEMM kernels (moe_gemm.hip).
+// Internal interface of the grouped (moe_gemm.hip) and dense (gemm_dense.cpp) GEMM kernels.
 #pragma once
 #include "common.hpp"
 
@@ -40,6 +40,8 @@ struct GemmParams {
 // (mat,row-tile) items.
 int run_gemm(const GemmParams &p, bool gather, int epi, int rows_per_tile, int max_tiles,
              hipStream_t s);
+// gemm_dense.cpp: bf16 weights, no gather (run_gemm comes here for that form)
+int run_gemm_dense(const GemmParams &p, int epi, int rows_per_tile, int max_tiles, hipStream_t s);
 // gemm_tall.hip: tiles of 256 x 256 with both operands through LDS, for launches of thousands of rows,
 // bound by the matrix cores (bf16 weights; gather + SwiGLU, plain fp32 output, or the row arg-max).  max_rows bounds
 // the rows of A that the launch can address.
@@ -49,7 +51,9 @@ bool gemm_tall_applies(const GemmParams &p, bool gather, int epi);
 inline bool gemm_tall_shape_ok(int N, int K, long long max_rows) {
   return K % 64 == 0 && K >= 256 && N % 32 == 0 && max_rows * K * 2 < (1ll << 32);
 }
-int run_gemm_tall(const GemmParams &p, bool gather, int epi, int max_tiles, long long max_rows, hipStream_t s);
+int check_gemm_tall(const GemmParams &p, bool gather, int epi, long long max_rows);
+int run_gemm_tall(const GemmParams &p, int epi, int max_tiles, long long max_rows, hipStream_t s);  // no gather
+int run_gemm_tall_gather(const GemmParams &p, int max_tiles, long long max_rows, hipStream_t s);    // gemm_tall_grouped.hip
 // norm_w / norm_out (optional, accumulate only): also write RMSNorm(out) * norm_w as bf16.  Returns
 // with only the combine done when the fused form does not apply (H > 4096 or misaligned); the
 // caller checks with combine_norm_applies().

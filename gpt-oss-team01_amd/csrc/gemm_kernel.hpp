@@ -695,38 +695,12 @@ int launch_gemm(const GemmParams &p, int max_tiles, hipStream_t s) {
   return GPTOSS_OK;
 }
 
-// the two operand/epilogue combinations in use, for every row-tile size
-#define GPTOSS_GEMM_INSTANTIATE(FP4V)                                                          \
-  template int launch_gemm<1, true, EPI_SWIGLU, FP4V>(const GemmParams &, int, hipStream_t);   \
-  template int launch_gemm<2, true, EPI_SWIGLU, FP4V>(const GemmParams &, int, hipStream_t);   \
-  template int launch_gemm<3, true, EPI_SWIGLU, FP4V>(const GemmParams &, int, hipStream_t);   \
-  template int launch_gemm<4, true, EPI_SWIGLU, FP4V>(const GemmParams &, int, hipStream_t);   \
-  template int launch_gemm<5, true, EPI_SWIGLU, FP4V>(const GemmParams &, int, hipStream_t);   \
-  template int launch_gemm<1, false, EPI_F32, FP4V>(const GemmParams &, int, hipStream_t);     \
-  template int launch_gemm<2, false, EPI_F32, FP4V>(const GemmParams &, int, hipStream_t);     \
-  template int launch_gemm<3, false, EPI_F32, FP4V>(const GemmParams &, int, hipStream_t);     \
-  template int launch_gemm<4, false, EPI_F32, FP4V>(const GemmParams &, int, hipStream_t);     \
-  template int launch_gemm<5, false, EPI_F32, FP4V>(const GemmParams &, int, hipStream_t);     \
-  template int launch_gemm<1, false, EPI_ARGMAX, FP4V>(const GemmParams &, int, hipStream_t);  \
-  template int launch_gemm<2, false, EPI_ARGMAX, FP4V>(const GemmParams &, int, hipStream_t);  \
-  template int launch_gemm<3, false, EPI_ARGMAX, FP4V>(const GemmParams &, int, hipStream_t);  \
-  template int launch_gemm<4, false, EPI_ARGMAX, FP4V>(const GemmParams &, int, hipStream_t);  \
-  template int launch_gemm<5, false, EPI_ARGMAX, FP4V>(const GemmParams &, int, hipStream_t);
-
-#define GPTOSS_GEMM_ATTR_ROW(M, FP4V)                                            \
-  if (err == hipSuccess) err = gemm_set_attr<M, true, EPI_SWIGLU, FP4V>();       \
-  if (err == hipSuccess) err = gemm_set_attr<M, false, EPI_F32, FP4V>();         \
-  if (err == hipSuccess) err = gemm_set_attr<M, false, EPI_ARGMAX, FP4V>();
-
-#define GPTOSS_GEMM_SET_ATTRS(NAME, FP4V) \
-  hipError_t NAME() {                     \
-    hipError_t err = hipSuccess;          \
-    GPTOSS_GEMM_ATTR_ROW(1, FP4V)         \
-    GPTOSS_GEMM_ATTR_ROW(2, FP4V)         \
-    GPTOSS_GEMM_ATTR_ROW(3, FP4V)         \
-    GPTOSS_GEMM_ATTR_ROW(4, FP4V)         \
-    GPTOSS_GEMM_ATTR_ROW(5, FP4V)         \
-    return err;                           \
-  }
+// the operand/epilogue combinations in use, for every row-tile size
+#define GPTOSS_GEMM_EACH_TILE(F, GATHER, EPI, FP4V) \
+  F(1, GATHER, EPI, FP4V) F(2, GATHER, EPI, FP4V) F(3, GATHER, EPI, FP4V) F(4, GATHER, EPI, FP4V) F(5, GATHER, EPI, FP4V)
+#define GPTOSS_GEMM_INSTANTIATE(M, GATHER, EPI, FP4V) \
+  template int launch_gemm<M, GATHER, EPI, FP4V>(const GemmParams &, int, hipStream_t);
+#define GPTOSS_GEMM_SET_ATTR(M, GATHER, EPI, FP4V) \
+  if (err == hipSuccess) err = gemm_set_attr<M, GATHER, EPI, FP4V>();
 
 }  // namespace gptoss

@@ -34,12 +34,14 @@ __global__ __launch_bounds__(256) void embedding_kernel(const bf16_t *__restrict
 // float products, eps added after the mean, 1/sqrtf in float, scale applied in double and
 // rounded once.  If residual != nullptr, x += residual first (in place), as
 // residual_rmsnorm_bf16_kernel does (layer_hip_batch.cpp:94-155).
-// Outputs: t_bf16 (always) and t_f32 (optional full-precision copy).
+// Outputs: t_bf16 (always) and t_f32 (optional full-precision copy).  n_mean: elements the mean is
+// taken over (rows padded with zeros have fewer than H).
 __global__ __launch_bounds__(256) void rmsnorm_kernel(float *__restrict__ x,
                                                       const float *__restrict__ residual,
                                                       const float *__restrict__ weight,
                                                       bf16_t *__restrict__ t_bf16,
-                                                      float *__restrict__ t_f32, int H) {
+                                                      float *__restrict__ t_f32, int H, float eps,
+                                                      int n_mean) {
   __shared__ double red[4];
   const int b = blockIdx.x;
   float *xr = x + (size_t)b * H;
@@ -56,8 +58,8 @@ __global__ __launch_bounds__(256) void rmsnorm_kernel(float *__restrict__ x,
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
   __syncthreads();
   ss = red[0] + red[1] + red[2] + red[3];
-  ss /= H;
-  ss += 1e-5f;
+  ss /= n_mean;
+  ss += eps;
   const double inv = (double)(1.0f / sqrtf((float)ss));
   for (int h = threadIdx.x; h < H; h += 256) {
     float o = (float)((double)weight[h] * (inv * (double)xr[h]));
@@ -73,7 +75,8 @@ __global__ __launch_bounds__(256) void rmsnorm_rows_kernel(float *__restrict__ x
                                                            const float *__restrict__ residual,
                                                            const float *__restrict__ weight,
                                                            bf16_t *__restrict__ t_bf16,
-                                                           float *__restrict__ t_f32, int H) {
+                                                           float *__restrict__ t_f32, int H, float eps,
+                                                           int n_mean) {
   __shared__ double red[4];
   const size_t row = (size_t)blockIdx.x * H;
   f32x4 v[VPT];
@@ -98,8 +101,8 @@ __global__ __launch_bounds__(256) void rmsnorm_rows_kernel(float *__restrict__ x
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
   __syncthreads();
   ss = red[0] + red[1] + red[2] + red[3];
-  ss /= H;
-  ss += 1e-5f;
+  ss /= n_mean;
+  ss += eps;
   const double inv = (double)(1.0f / sqrtf((float)ss));
 #pragma unroll
   for (int i = 0; i < VPT; i++) {
@@ -339,15 +342,16 @@ int run_embedding(const bf16_t *table, const int *tokens, float *x, int B, int H
 }
 
 int run_rmsnorm(float *x, const float *residual, const float *weight, bf16_t *t_bf16, float *t_f32,
-                int B, int H, hipStream_t s) {
+                int B, int H, hipStream_t s, float eps, int n_mean) {
+  if (n_mean == 0) n_mean = H;
   TraceScope ts(residual ? "residual_rmsnorm" : "rmsnorm", s);
   const bool vec = H % 4 == 0 && aligned(x, 16) && aligned(weight, 16) && aligned(t_bf16, 8) &&
                    (!residual || aligned(residual, 16)) && (!t_f32 || aligned(t_f32, 16));
-  if (vec && H <= 1024) rmsnorm_rows_kernel<1><<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H);
-  else if (vec && H <= 2048) rmsnorm_rows_kernel<2><<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H);
-  else if (vec && H <= 3072) rmsnorm_rows_kernel<3><<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H);
-  else if (vec && H <= 4096) rmsnorm_rows_kernel<4><<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H);
-  else rmsnorm_kernel<<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H);
+  if (vec && H <= 1024) rmsnorm_rows_kernel<1><<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H, eps, n_mean);
+  else if (vec && H <= 2048) rmsnorm_rows_kernel<2><<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H, eps, n_mean);
+  else if (vec && H <= 3072) rmsnorm_rows_kernel<3><<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H, eps, n_mean);
+  else if (vec && H <= 4096) rmsnorm_rows_kernel<4><<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H, eps, n_mean);
+  else rmsnorm_kernel<<<B, 256, 0, s>>>(x, residual, weight, t_bf16, t_f32, H, eps, n_mean);
   GPTOSS_LAUNCH_CHECK("rmsnorm_kernel");
   return GPTOSS_OK;
 }
@@ -499,6 +503,116 @@ int run_synth_bf16(bf16_t *dst, size_t n, uint64_t seed, float mean, float std, 
 int run_synth_f32(float *dst, size_t n, uint64_t seed, float mean, float std, hipStream_t s) {
   synth_normal_f32_kernel<<<grid_for(n), 256, 0, s>>>(dst, n, seed, mean, std);
   GPTOSS_LAUNCH_CHECK("synth_normal_f32_kernel");
+  return GPTOSS_OK;
+}
+
+// x[b,:] = table[token[b],:] + positions[p,:], p = lens[b] - 1 (a learned position vector), fp32 rows of
+// stride ld whose columns from H on are zero; also the first entry of the depth average's history.
+template <typename T>
+__global__ __launch_bounds__(256) void embedding_position_kernel(const T *__restrict__ table,
+                                                                 const T *__restrict__ positions,
+                                                                 const int *__restrict__ tokens,
+                                                                 const int *__restrict__ lens,
+                                                                 float *__restrict__ x, float *__restrict__ x0,
+                                                                 int H, int ld, int V, int n_pos) {
+  const int b = blockIdx.x;
+  const int tok = min(max(tokens[b], 0), V - 1), pos = min(max(lens[b] - 1, 0), n_pos - 1);
+  auto value = [](T v) {
+    if constexpr (sizeof(T) == 2) return bf16_to_f32(v);
+    else return v;
+  };
+  for (int h = threadIdx.x; h < ld; h += 256) {
+    const float v = h < H ? value(table[(size_t)tok * H + h]) + value(positions[(size_t)pos * H + h]) : 0.f;
+    x[(size_t)b * ld + h] = v;
+    x0[(size_t)b * ld + h] = v;
+  }
+}
+
+// The depth average behind layer i and the norm in front of layer i + 1: X = x + y (the layer's
+// result, kept in history[i + 1]), x = sum_j weights[j] * history[j] over j = 0 .. i + 1, and
+// t = weight * x / sqrt(mean(x^2) + eps).  history: [layers + 1][rows_cap, H]; norm_w nullptr: no norm.
+template <int VPT>
+__global__ __launch_bounds__(256) void depth_average_norm_kernel(float *__restrict__ x, const float *__restrict__ y,
+                                                                 float *__restrict__ history, size_t plane,
+                                                                 const float *__restrict__ weights, int layer,
+                                                                 const float *__restrict__ norm_w,
+                                                                 bf16_t *__restrict__ t_bf16,
+                                                                 float *__restrict__ t_f32, int H, float eps,
+                                                                 int n_mean) {
+  __shared__ double red[4];
+  const size_t row = (size_t)blockIdx.x * H;
+  f32x4 v[VPT];
+  double ss = 0.0;
+#pragma unroll
+  for (int i = 0; i < VPT; i++) {
+    const int h = (threadIdx.x + 256 * i) * 4;
+    v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (h < H) {
+      const f32x4 own = *reinterpret_cast<const f32x4 *>(x + row + h) + *reinterpret_cast<const f32x4 *>(y + row + h);
+      *reinterpret_cast<f32x4 *>(history + (size_t)(layer + 1) * plane + row + h) = own;
+      f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int j = 0; j <= layer; j++)
+        a += weights[j] * *reinterpret_cast<const f32x4 *>(history + (size_t)j * plane + row + h);
+      v[i] = a + weights[layer + 1] * own;
+      *reinterpret_cast<f32x4 *>(x + row + h) = v[i];
+#pragma unroll
+      for (int q = 0; q < 4; q++) ss += (double)__fmul_rn(v[i][q], v[i][q]);
+    }
+  }
+  if (!norm_w) return;
+  for (int m = 32; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, 64);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+  __syncthreads();
+  ss = red[0] + red[1] + red[2] + red[3];
+  ss /= n_mean;
+  ss += eps;
+  const double inv = (double)(1.0f / sqrtf((float)ss));
+#pragma unroll
+  for (int i = 0; i < VPT; i++) {
+    const int h = (threadIdx.x + 256 * i) * 4;
+    if (h < H) {
+      const f32x4 w = *reinterpret_cast<const f32x4 *>(norm_w + h);
+      f32x4 o;
+#pragma unroll
+      for (int q = 0; q < 4; q++) o[q] = (float)((double)w[q] * (inv * (double)v[i][q]));
+      *reinterpret_cast<u32x2 *>(t_bf16 + row + h) = u32x2{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
+      if (t_f32) *reinterpret_cast<f32x4 *>(t_f32 + row + h) = o;
+    }
+  }
+}
+
+template <typename T>
+static int launch_embedding_position(const T *table, const T *positions, const int *tokens, const int *lens, float *x,
+                                     float *x0, int rows, int H, int ld, int V, int n_pos, hipStream_t s) {
+  TraceScope ts("embedding", s);
+  embedding_position_kernel<T><<<rows, 256, 0, s>>>(table, positions, tokens, lens, x, x0, H, ld, V, n_pos);
+  GPTOSS_LAUNCH_CHECK("embedding_position_kernel");
+  return GPTOSS_OK;
+}
+
+int run_embedding_position(const bf16_t *table, const bf16_t *positions, const int *tokens, const int *lens, float *x,
+                           float *x0, int rows, int H, int ld, int V, int n_pos, hipStream_t s) {
+  return launch_embedding_position(table, positions, tokens, lens, x, x0, rows, H, ld, V, n_pos, s);
+}
+int run_embedding_position_f32(const float *table, const float *positions, const int *tokens, const int *lens,
+                               float *x, float *x0, int rows, int H, int ld, int V, int n_pos, hipStream_t s) {
+  return launch_embedding_position(table, positions, tokens, lens, x, x0, rows, H, ld, V, n_pos, s);
+}
+
+int run_depth_average_norm(float *x, const float *y, float *history, size_t plane, const float *weights, int layer,
+                           const float *norm_w, bf16_t *t_bf16, float *t_f32, int rows, int H, float eps, int n_mean,
+                           hipStream_t s) {
+  GPTOSS_REQUIRE(H % 4 == 0 && H <= 16384, GPTOSS_ERR_DIM, "depth_average: rows of %d elements (a multiple of 4, at most 16384)", H);
+  TraceScope ts("depth_average_norm", s);
+  auto go = [&](auto kern) {
+    kern<<<rows, 256, 0, s>>>(x, y, history, plane, weights, layer, norm_w, t_bf16, t_f32, H, eps, n_mean);
+  };
+  if (H <= 1024) go(depth_average_norm_kernel<1>);
+  else if (H <= 2048) go(depth_average_norm_kernel<2>);
+  else if (H <= 4096) go(depth_average_norm_kernel<4>);
+  else if (H <= 8192) go(depth_average_norm_kernel<8>);
+  else go(depth_average_norm_kernel<16>);
+  GPTOSS_LAUNCH_CHECK("depth_average_norm_kernel");
   return GPTOSS_OK;
 }
 

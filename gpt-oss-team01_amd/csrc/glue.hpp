@@ -5,9 +5,20 @@
 namespace gptoss {
 
 int run_embedding(const bf16_t *table, const int *tokens, float *x, int B, int H, int V, hipStream_t s);
-// x (+= residual) -> t_bf16 (and t_f32 when not null); residual may be null
+// x (+= residual) -> t_bf16 (and t_f32 when not null); residual may be null; n_mean: elements the mean
+// is taken over (0: H)
 int run_rmsnorm(float *x, const float *residual, const float *weight, bf16_t *t_bf16, float *t_f32,
-                int B, int H, hipStream_t s);
+                int B, int H, hipStream_t s, float eps = 1e-5f, int n_mean = 0);
+// x = x0 = table[token] + positions[lens - 1], rows of stride ld (zero from column H on)
+int run_embedding_position(const bf16_t *table, const bf16_t *positions, const int *tokens, const int *lens, float *x,
+                           float *x0, int rows, int H, int ld, int V, int n_pos, hipStream_t s);
+int run_embedding_position_f32(const float *table, const float *positions, const int *tokens, const int *lens,
+                               float *x, float *x0, int rows, int H, int ld, int V, int n_pos, hipStream_t s);
+// history[layer + 1] = x + y; x = sum over j <= layer + 1 of weights[j] * history[j] (planes of `plane`
+// elements); with norm_w also t = RMSNorm(x) * norm_w
+int run_depth_average_norm(float *x, const float *y, float *history, size_t plane, const float *weights, int layer,
+                           const float *norm_w, bf16_t *t_bf16, float *t_f32, int rows, int H, float eps, int n_mean,
+                           hipStream_t s);
 int run_rope_store(const float *qkv, float *q_out, bf16_t *kv, const float *cos_t,
                    const float *sin_t, int B, int n_q, int n_kv, int D, int cap, int pos,
                    hipStream_t s);

@@ -56,6 +56,11 @@ class Config(C.Structure):
         return cls(*[getattr(c, n) for n, _ in cls._fields_])
 
 
+class ModelInfo(C.Structure):
+    _fields_ = [(n, C.c_int) for n in ("vocab", "logits_stride", "hidden", "hidden_stride", "n_layers",
+                                       "max_batch", "max_seq", "max_rows")]
+
+
 _vp, _i, _sz, _f = C.c_void_p, C.c_int, C.c_size_t, C.c_float
 
 #: name -> (restype, argtypes); every symbol declared in include/gptoss_mi355.h
@@ -92,6 +97,12 @@ SIGNATURES = {
     "gptoss_rope_kv_store": (_i, [_vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp]),
     "gptoss_engine_create": (_i, [C.POINTER(Config), _vp, _i, _i, _i, C.c_uint64,
                                   C.POINTER(_vp)]),
+    "gptoss_engine_open": (_i, [C.c_char_p, _i, _i, _i, C.c_uint64, C.POINTER(_vp)]),
+    "gptoss_model_name": (C.c_char_p, [_i]),
+    "gptoss_engine_info": (_i, [_vp, C.POINTER(ModelInfo)]),
+    "gptoss_engine_step_logits": (_i, [_vp, _i, _vp, _vp, _vp, _i, _vp, _vp]),
+    "gptoss_engine_slot_acquire": (_i, [_vp, C.POINTER(_i)]),
+    "gptoss_engine_slot_release": (_i, [_vp, _i]),
     "gptoss_engine_step": (_i, [_vp, _vp, _i, _i, _vp]),
     "gptoss_engine_prefill": (_i, [_vp, _vp, _i, _i, _vp]),
     "gptoss_engine_step_ragged": (_i, [_vp, _vp, _vp, _i, _vp]),
@@ -109,15 +120,17 @@ SIGNATURES = {
 _lib = None
 
 
-def load(strict: bool = os.environ.get("GPTOSS_PARTIAL_LIB") != "1"):
-    """Load the shared library and bind every declared entry point."""
+def load(strict: bool = os.environ.get("GPTOSS_PARTIAL_LIB") != "1", path: str = None):
+    """Load the shared library and bind every declared entry point.  path: a library that serves
+    some model classes only (build.ensure_for); it lacks the other classes' entry points."""
     global _lib
     if _lib is not None:
         return _lib
-    if not os.path.exists(LIB_PATH):
-        raise ImportError(f"{LIB_PATH} is missing: build it with "
+    path, partial = path or LIB_PATH, path not in (None, LIB_PATH)
+    if not os.path.exists(path):
+        raise ImportError(f"{path} is missing: build it with "
                           f"`python {os.path.join(HERE, 'build.py')}` (hipcc, gfx950)")
-    L = C.CDLL(LIB_PATH)
+    L = C.CDLL(path)
     missing = []
     for name, (res, args) in SIGNATURES.items():
         try:
@@ -127,8 +140,8 @@ def load(strict: bool = os.environ.get("GPTOSS_PARTIAL_LIB") != "1"):
             continue
         fn.restype = res
         fn.argtypes = args
-    if missing and strict:
-        raise ImportError(f"{LIB_PATH} does not export: {', '.join(missing)}")
+    if missing and strict and not partial:
+        raise ImportError(f"{path} does not export: {', '.join(missing)}")
     _lib = L
     return L
 

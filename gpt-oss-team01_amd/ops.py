@@ -9,6 +9,7 @@ import ctypes as C
 
 import torch
 
+from . import engine as _e
 from . import lib as _l
 
 
@@ -335,91 +336,12 @@ class KernelTrace:
         return {k: (c, t / c) for k, (c, t) in agg.items()}
 
 
-class Engine:
-    """Single-GPU decode engine over a flat ``.bin`` payload (or synthetic on-device weights)."""
+class Engine(_e.Engine):
+    """The engine with what tests and benchmarks read through PyTorch."""
 
-    def __init__(self, cfg, weights_flat=None, max_batch=8, max_seq=64, synthetic=False,
-                 precise=False, seed=0, keep_logits=True, prefill=True, mxfp4_experts=False):
+    def __init__(self, *args, **kw):
         _need_gpu()
-        import numpy as np
-        self.L = _l.load()
-        self.cfg = cfg
-        self.max_batch, self.max_seq = max_batch, max_seq
-        flags = (_l.ENGINE_SYNTHETIC if synthetic else 0) | (_l.ENGINE_PRECISE if precise else 0) | \
-            (_l.ENGINE_LOGITS if keep_logits else 0) | (0 if prefill else _l.ENGINE_NO_PREFILL) | \
-            (_l.ENGINE_MXFP4_EXPERTS if mxfp4_experts else 0)
-        self._cc = _l.Config.from_config(cfg)
-        wp = None
-        if not synthetic:
-            self._w = np.ascontiguousarray(weights_flat, dtype=np.float32)
-            wp = self._w.ctypes.data_as(C.c_void_p)
-        h = C.c_void_p()
-        _l.check(self.L.gptoss_engine_create(C.byref(self._cc), wp, max_batch, max_seq, flags,
-                                             C.c_uint64(seed), C.byref(h)))
-        self._h = h
-
-    def step(self, tokens, pos):
-        import numpy as np
-        tok = np.ascontiguousarray(tokens, dtype=np.int32)
-        nxt = np.empty_like(tok)
-        _l.check(self.L.gptoss_engine_step(self._h, tok.ctypes.data_as(C.c_void_p), int(pos),
-                                           tok.size, nxt.ctypes.data_as(C.c_void_p)))
-        return nxt
-
-    def prefill(self, tokens):
-        """Positions 0..T-1 of every sequence (tokens int32 [B, T]) in one pass -> next ids [B]."""
-        import numpy as np
-        tok = np.ascontiguousarray(tokens, dtype=np.int32)
-        B, T = tok.shape
-        nxt = np.empty(B, np.int32)
-        _l.check(self.L.gptoss_engine_prefill(self._h, tok.ctypes.data_as(C.c_void_p), B, T,
-                                              nxt.ctypes.data_as(C.c_void_p)))
-        return nxt
-
-    def step_ragged(self, tokens, positions):
-        """One step with every sequence at its own position."""
-        import numpy as np
-        tok = np.ascontiguousarray(tokens, dtype=np.int32)
-        pos = np.ascontiguousarray(positions, dtype=np.int32)
-        nxt = np.empty_like(tok)
-        _l.check(self.L.gptoss_engine_step_ragged(self._h, tok.ctypes.data_as(C.c_void_p),
-                                                  pos.ctypes.data_as(C.c_void_p), tok.size,
-                                                  nxt.ctypes.data_as(C.c_void_p)))
-        return nxt
-
-    def step_rows(self, tokens, slots, positions, sample):
-        """One step over arbitrary rows (token, cache slot, position); -> next ids after the rows `sample`."""
-        import numpy as np
-        tok = np.ascontiguousarray(tokens, dtype=np.int32)
-        slot = np.ascontiguousarray(slots, dtype=np.int32)
-        pos = np.ascontiguousarray(positions, dtype=np.int32)
-        smp = np.ascontiguousarray(sample, dtype=np.int32)
-        nxt = np.empty(smp.size, np.int32)
-        p = lambda a: a.ctypes.data_as(C.c_void_p)
-        _l.check(self.L.gptoss_engine_step_rows(self._h, tok.size, p(tok), p(slot), p(pos), smp.size, p(smp), p(nxt)))
-        return nxt
-
-    def generate(self, prompts, max_seq_len, n_prompt=None, max_len=None):
-        """Greedy generation; max_len (optional, per request) limits a request's total length."""
-        import numpy as np
-        prompts = np.ascontiguousarray(prompts, dtype=np.int32)
-        n_req, stride = prompts.shape
-        npr = np.full(n_req, stride, np.int32) if n_prompt is None else \
-            np.ascontiguousarray(n_prompt, dtype=np.int32)
-        out = np.zeros((n_req, max_seq_len + 1), np.int32)
-        n = C.c_longlong(0)
-        if max_len is None:
-            _l.check(self.L.gptoss_engine_generate(self._h, prompts.ctypes.data_as(C.c_void_p),
-                                                   npr.ctypes.data_as(C.c_void_p), stride, n_req,
-                                                   max_seq_len, out.ctypes.data_as(C.c_void_p),
-                                                   C.byref(n)))
-        else:
-            ml = np.ascontiguousarray(max_len, dtype=np.int32)
-            _l.check(self.L.gptoss_engine_generate_ragged(self._h, prompts.ctypes.data_as(C.c_void_p),
-                                                          npr.ctypes.data_as(C.c_void_p), stride, n_req,
-                                                          max_seq_len, ml.ctypes.data_as(C.c_void_p),
-                                                          out.ctypes.data_as(C.c_void_p), C.byref(n)))
-        return out, int(n.value)
+        super().__init__(*args, **kw)
 
     def last_logits(self, B):
         """fp32 [B, vocab] logits of the last step (copied to the host)."""
@@ -427,7 +349,7 @@ class Engine:
         _l.check(self.L.gptoss_engine_debug_views(self._h, C.byref(lp), C.byref(xp), C.byref(nb)))
         if not lp.value:
             raise RuntimeError("the engine was created without keep_logits")
-        V = self.cfg.vocab_size
+        V = self.info.logits_stride
         host = torch.empty(B, V, dtype=torch.float32)
         torch.cuda.synchronize()
         # a plain device-to-host copy of memory the engine owns
@@ -435,7 +357,7 @@ class Engine:
         rc = rt.hipMemcpy(C.c_void_p(host.data_ptr()), lp, C.c_size_t(B * V * 4), 2)
         if rc != 0:
             raise RuntimeError(f"hipMemcpy failed: {rc}")
-        return host.numpy()
+        return host.numpy()[:, :self.info.vocab]
 
     def tensor(self, name, layer=0):
         """Copy of one weight tensor as the engine holds it on the device (uint8, flat);
@@ -449,19 +371,6 @@ class Engine:
         if rc != 0:
             raise RuntimeError(f"hipMemcpy failed: {rc}")
         return out
-
-    def device_bytes(self):
-        nb = C.c_size_t()
-        _l.check(self.L.gptoss_engine_debug_views(self._h, None, None, C.byref(nb)))
-        return nb.value
-
-    def close(self):
-        if getattr(self, "_h", None):
-            self.L.gptoss_engine_destroy(self._h)
-            self._h = None
-
-    def __del__(self):
-        self.close()
 
 
 def pack_mxfp4(blocks: torch.Tensor, scales: torch.Tensor, glu: bool = False) -> torch.Tensor:

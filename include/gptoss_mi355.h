@@ -323,6 +323,23 @@ enum {
 int gptoss_engine_create(const gptoss_config *cfg, const float *host_weights, int max_batch,
                          int max_seq, int flags, uint64_t seed, gptoss_engine **out);
 
+/* Open a checkpoint of any registered model: a folder with config.json (its "architecture" names the
+ * model class) and model.safetensors, or a flat .bin file (GPT-OSS).  max_seq <= 0: as many positions
+ * as the model has.  With GPTOSS_ENGINE_SYNTHETIC a folder needs config.json only.  Every function
+ * below that takes an engine works on the result; what a model does not offer returns
+ * GPTOSS_ERR_STATE.  The architectures, by index, until NULL: gptoss_model_name. */
+int gptoss_engine_open(const char *path, int max_batch, int max_seq, int flags, uint64_t seed,
+                       gptoss_engine **out);
+const char *gptoss_model_name(int i);
+
+typedef struct {
+  int vocab, logits_stride;     /* entries of a row of logits, and floats from one row to the next */
+  int hidden, hidden_stride;
+  int n_layers, max_batch, max_seq;
+  int max_rows;                 /* most rows of one step (0: the model has no step over rows) */
+} gptoss_model_info;
+int gptoss_engine_info(gptoss_engine *e, gptoss_model_info *info);
+
 /* One lock-step decode step: feed host_tokens[B] at position pos, return the arg-max next ids
  * (lowest id wins ties) in host_next[B].  Replaces forward_gpu_20b_batched
  * (getp-csrc/src/model.cpp:6-151).  Synchronises once, to hand the ids back. */
@@ -349,6 +366,18 @@ int gptoss_engine_step_ragged(gptoss_engine *e, const int *host_tokens, const in
  * available with GPTOSS_ENGINE_PRECISE or GPTOSS_ENGINE_NO_PREFILL. */
 int gptoss_engine_step_rows(gptoss_engine *e, int n_rows, const int *host_tokens, const int *host_slots,
                             const int *host_pos, int n_sample, const int *host_sample, int *host_next);
+
+/* The same rows, with the fp32 logits of the rows host_want (ascending) written to host_logits
+ * [n_want, vocab] instead of their arg-max.  Any number of rows: more than a step may hold are run as
+ * consecutive steps.  Needs GPTOSS_ENGINE_LOGITS. */
+int gptoss_engine_step_logits(gptoss_engine *e, int n_rows, const int *host_tokens, const int *host_slots,
+                              const int *host_pos, int n_want, const int *host_want, float *host_logits);
+
+/* Cache slots for callers that keep sequences of their own next to step_rows / step_logits: a free
+ * slot, and giving it back.  A sequence starts at position 0 whatever the slot held before.
+ * gptoss_engine_generate needs its slots (0 .. min(n_req, max_batch) - 1) free. */
+int gptoss_engine_slot_acquire(gptoss_engine *e, int *slot);
+int gptoss_engine_slot_release(gptoss_engine *e, int slot);
 
 /* Positions 0..T-1 of B sequences in one pass: host_tokens int32 [B, T]; fills the KV caches and
  * returns in host_next[B] the arg-max ids after position T-1, i.e. what T calls of
