@@ -38,8 +38,16 @@ def unit_vectors(x):
     return x / np.sqrt(np.sum(np.square(x), axis=-1, keepdims=True) + 1e-6)
 
 
+#: what forward(rounding=...) applies to the inputs of matrix products and to stored keys and values
+_rounding = None
+
+
+def rounded(x):
+    return f64(x) if _rounding is None else f64(_rounding(x)).reshape(np.shape(x))
+
+
 def linear(h, weight):
-    return f64(h) @ f64(weight).T
+    return rounded(h) @ f64(weight).T
 
 
 # ---- short convolution -------------------------------------------------------------------------
@@ -142,7 +150,7 @@ def mixer_window(h, w, p, mix, eps):
     q = over_rms(_heads(linear(h, w[f"{p}.q"]), H), eps) * f64(w[f"{p}.q.norm"])
     k = over_rms(_heads(linear(h, w[f"{p}.k"]), G), eps) * f64(w[f"{p}.k.norm"])
     v = _heads(linear(h, w[f"{p}.v"]), G)
-    o = window_attention(q, k, v, mix["scale"], mix["mask"]["size"])
+    o = window_attention(q, rounded(k), rounded(v), mix["scale"], mix["mask"]["size"])
     return linear(o.reshape(len(h), -1), w[f"{p}.o"])
 
 
@@ -173,8 +181,18 @@ def feed_forward(h, w, p):
     return linear(relu_squared(linear(h, w[f"{p}.up"])), w[f"{p}.down"])
 
 
-def forward(cfg, w, tokens, want_layers=False):
-    """Logits [T, vocab] of one sequence from position 0 (and the residual stream after every layer)."""
+def forward(cfg, w, tokens, want_layers=False, rounding=None):
+    """Logits [T, vocab] of one sequence from position 0 (and the residual stream after every layer).
+    rounding: applied where activations of lower precision enter matrix products or a cache."""
+    global _rounding
+    _rounding = rounding
+    try:
+        return _forward(cfg, w, tokens, want_layers)
+    finally:
+        _rounding = None
+
+
+def _forward(cfg, w, tokens, want_layers):
     eps = cfg["norm"]["eps"]
     tokens = np.asarray(tokens)
     x = f64(w["embed"])[tokens] + f64(w["pos"])[:len(tokens)]
