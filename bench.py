@@ -71,6 +71,10 @@ def parse():
     ap.add_argument("--mfma-rates", action="store_true",
                     help="only measure the register-fed issue rate of the bf16 and the scaled f8f6f4 MFMA "
                          "(gptoss_diag_mfma_rate) and print one JSON line of its own")
+    ap.add_argument("--model", choices=("gpt-oss", "nezavik"), default="gpt-oss",
+                    help="nezavik: only measure prefill and decode of the Nezavik model class at a few sizes, "
+                         "beside GPT-OSS engines of the same width, and print one JSON line of its own")
+    ap.add_argument("--only", default="", help="with --model nezavik: sizes to run, with commas between them")
     ap.add_argument("--no-sched", action="store_true", help="skip the scheduler leg of the end-to-end figure")
     return ap.parse_args()
 
@@ -528,6 +532,209 @@ def bench_loader(ops, torch):
             "what": "fp32 host payload (20B dimensions, 2 blocks) -> packed bf16 device weights, PCIe included"}
 
 
+VALU_FP32_PEAK_TFLOPS = 78.6   # MI355X fp32 vector units, packed instructions aside
+
+
+def nezavik_config(width, heads, ff, layers, attn_heads, kv_heads, window, positions, vocab=65536):
+    """Layers in the proportions of a real model: heads of 128 in the delta rules, 64 in the attention,
+    a state of 128 in the state-space half."""
+    delta = {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4}
+    par = {"left": {"heads": attn_heads, "kv_heads": kv_heads, "dim": 64, "vdim": 64, "scale": 0.125,
+                    "mask": {"size": window}},
+           "left_scale": 0.5,
+           "right": {"heads": width // 64, "groups": 8, "state": 128, "vdim": 64, "conv": 4, "norm_groups": 8},
+           "right_scale": 0.5}
+    kinds = [("delta", delta), ("parallel", par), ("channel_delta", delta), ("parallel", par)]
+    return {"architecture": "Nezavik", "vocab": vocab, "width": width, "max_positions": positions,
+            "norm": {"eps": 1e-5},
+            "layers": [{"type": t, "mixer": m, "mlp": {"kind": "dense", "ff": ff}}
+                       for t, m in (kinds[i % 4] for i in range(layers))]}
+
+
+def _nezavik_work(cfg, rows, seqs, context):
+    """Algorithmic (bytes, flop, peak TFLOP/s) of one step of `rows` rows over `seqs` sequences whose
+    window holds `context` positions per row, summed over the launches of each kernel label."""
+    W, up = cfg["width"], lambda n, m: (n + m - 1) // m * m
+    work = {}
+
+    def add(label, nbytes, flop=0.0, peak=MFMA_BF16_PEAK_TFLOPS):
+        b, f, _ = work.get(label, (0.0, 0.0, peak))
+        work[label] = (b + nbytes, f + flop, peak)
+
+    def gemm(n_out, n_in):
+        add("gemm_f32", n_out * n_in * 2 + rows * (n_in * 2 + n_out * 4), 2.0 * rows * n_out * n_in)
+
+    def conv(ch):
+        add("short_conv", rows * ch * 8)
+
+    def scan(label, heads, K, V, inputs):
+        # per state element and token: decay, prediction, update, read-out (2 flop each; no prediction
+        # in the state-space form)
+        per = 6 if label == "scan_state_space" else 7
+        add(label, seqs * heads * K * V * 8 + rows * (inputs + heads * V) * 4, float(per) * rows * heads * K * V,
+            VALU_FP32_PEAK_TFLOPS)
+
+    for i, layer in enumerate(cfg["layers"]):
+        m, ff = layer["mixer"], layer["mlp"]["ff"]
+        if layer["type"] == "parallel":
+            a, r = m["left"], m["right"]
+            qkv = a["heads"] * a["dim"] + a["kv_heads"] * (a["dim"] + a["vdim"])
+            inner, gn = r["heads"] * r["vdim"], r["groups"] * r["state"]
+            gemm(up(qkv + 2 * inner + 2 * gn + r["heads"] + ff, 32), W)
+            gemm(W, up(a["heads"] * a["vdim"] + inner + ff, 64))
+            add("window_store", rows * (qkv * 4 + a["heads"] * a["dim"] * 4 + a["kv_heads"] * (a["dim"] + a["vdim"]) * 2))
+            kv = context * a["kv_heads"] * (a["dim"] + a["vdim"]) * 2
+            add("window_decode" if rows == seqs else "window_tiles",
+                seqs * kv + rows * a["heads"] * (a["dim"] * 4 + a["vdim"] * 2),
+                2.0 * rows * context * a["heads"] * (a["dim"] + a["vdim"]))
+            conv(inner + 2 * gn)
+            scan("scan_state_space", r["heads"], r["state"], r["vdim"], inner + 2 * gn)
+            add("gated_norm", rows * inner * 10)
+        else:
+            H, nk, nv = m["heads"], m["kv_heads"] * m["dim"], m["heads"] * m["vdim"]
+            if layer["type"] == "delta":
+                gemm(up(2 * nk + 2 * nv + 2 * H + ff, 32), W)
+            else:
+                gemm(up(2 * nk + nv + H + 256 + ff, 32), W)
+                gemm(H * m["dim"] + nv, 256)
+                add("column_copy", rows * 256 * 6)
+            gemm(W, up(nv + ff, 64))
+            conv(2 * nk + nv)
+            extra = H * m["dim"] if layer["type"] == "channel_delta" else 0
+            scan("scan_" + layer["type"], H, m["dim"], m["vdim"], 2 * nk + nv + extra)
+            add("gated_norm", rows * nv * 10)
+        add("relu_squared", rows * ff * 6)
+        add("depth_average_norm", rows * W * 4 * (i + 1 + 4.5))
+    add("gemm_argmax", cfg["vocab"] * W * 2 + seqs * W * 2, 2.0 * seqs * cfg["vocab"] * W)
+    return work
+
+
+def _against_roofline(kern, work):
+    out = {}
+    for name, (calls, ms) in kern.items():
+        row = {"calls": calls, "us": round(ms * calls * 1e3, 1)}
+        if name in work:
+            nbytes, flop, peak = work[name]
+            roof = max(nbytes / (HBM_PEAK_GBS * 1e3), flop / (peak * 1e6))     # us
+            row["roofline"] = round(roof / (ms * calls * 1e3), 3)
+            row["bound"] = "hbm" if nbytes / (HBM_PEAK_GBS * 1e3) >= roof else "flop"
+        out[name] = row
+    return out
+
+
+def _gptoss_work(cfg, rows, seqs, contexts):
+    """The same for a GPT-OSS engine: contexts = positions a row of a full and of a window layer sees."""
+    H, I, E, k = cfg.hidden_dim, cfg.intermediate_dim, cfg.n_experts, cfg.experts_per_token
+    D, nq, nkv, L = cfg.head_dim, cfg.n_attn_heads, cfg.n_kv_heads, cfg.n_layers
+    qkv = (nq + 2 * nkv) * D
+    work = {"gemm_f32": [0.0, 0.0], "gemm1_gather_swiglu": [0.0, 0.0], "attn": [0.0, 0.0], "rope_store": [0.0, 0.0],
+            "combine_rmsnorm": [0.0, 0.0]}
+
+    def add(label, nbytes, flop=0.0):
+        work[label][0] += nbytes
+        work[label][1] += flop
+
+    for l in range(L):
+        for n_out, n_in in ((qkv, H), (H, nq * D)):
+            add("gemm_f32", n_out * n_in * 2 + rows * (n_in * 2 + n_out * 4), 2.0 * rows * n_out * n_in)
+        add("gemm_f32", E * H * I * 2 + rows * k * (I * 2 + H * 4), 2.0 * rows * k * H * I)
+        add("gemm1_gather_swiglu", E * 2 * I * H * 2 + rows * H * 2 + rows * k * I * 2, 4.0 * rows * k * H * I)
+        ctx = contexts[1 if l % 2 == 0 else 0]
+        add("attn", seqs * ctx * nkv * D * 4 + rows * nq * D * 6, 4.0 * rows * ctx * nq * D)
+        add("rope_store", rows * (qkv * 4 + nq * D * 4 + 2 * nkv * D * 2))
+        add("combine_rmsnorm", rows * H * (k * 4 + 8 + 2))
+    work = {n: (b, f, MFMA_BF16_PEAK_TFLOPS) for n, (b, f) in work.items()}
+    for n in ("attn_decode", "attn_prefill_tiles"):
+        work[n] = work["attn"]
+    work["gemm_argmax"] = (cfg.vocab_size * H * 2 + seqs * H * 2, 2.0 * seqs * cfg.vocab_size * H, MFMA_BF16_PEAK_TFLOPS)
+    return work
+
+
+#: name -> (configuration, (decoding sequences, their context), (prompts, positions))
+NEZAVIK_SIZES = {
+    "width2048": (dict(width=2048, heads=16, ff=8192, layers=8, attn_heads=32, kv_heads=8, window=512), (256, 1024), (8, 1024)),
+    "width4096": (dict(width=4096, heads=32, ff=14336, layers=8, attn_heads=64, kv_heads=8, window=1024), (256, 1024), (4, 2048)),
+    "width4096_small_batch": (dict(width=4096, heads=32, ff=14336, layers=8, attn_heads=64, kv_heads=8, window=1024), (16, 1024),
+                              (1, 2048)),
+}
+
+
+def _time_engine(ops, torch, eng, vocab, decode, prompt, steps):
+    """-> decode ms per step and prefill ms per pass with their kernels (the engine synchronises per step)."""
+    import numpy as np
+    rng = np.random.default_rng(7)
+    (B, ctx), (Bp, T) = decode, prompt
+    ids = rng.integers(0, vocab, size=(max(B, Bp), max(ctx, T)), dtype=np.int32)
+    res = {}
+    eng.prefill(np.ascontiguousarray(ids[:Bp, :T]))
+    times = []
+    for _ in range(max(3, steps // 10)):
+        t0 = time.perf_counter()
+        eng.prefill(np.ascontiguousarray(ids[:Bp, :T]))
+        times.append(time.perf_counter() - t0)
+    trace = ops.KernelTrace(capacity=4096)
+    with trace:
+        eng.prefill(np.ascontiguousarray(ids[:Bp, :T]))
+    res["prefill"] = (sorted(times)[len(times) // 2] * 1e3, trace.summary())
+    tok = eng.prefill(np.ascontiguousarray(ids[:B, :ctx]))
+    for i in range(3):
+        tok = eng.step(tok, ctx + i)
+    t0 = time.perf_counter()
+    for i in range(steps):
+        tok = eng.step(tok, ctx + 3 + i)
+    dt = (time.perf_counter() - t0) * 1e3 / steps
+    trace = ops.KernelTrace(capacity=4096)
+    with trace:
+        eng.step(tok, ctx + 3 + steps)
+    res["decode"] = (dt, trace.summary())
+    return res
+
+
+def bench_nezavik(ops, torch, steps, only):
+    import tempfile
+    binfmt = importlib.import_module("gpt-oss-team01_amd.binfmt")
+    out = {}
+    for name, (shape, decode, prompt) in NEZAVIK_SIZES.items():
+        if only and name not in only:
+            continue
+        (B, ctx), (Bp, T) = decode, prompt
+        positions = max(ctx + steps + 8, T)
+        cfg = nezavik_config(positions=positions, **shape)
+        W, L, window = shape["width"], shape["layers"], shape["window"]
+        # GPT-OSS of the same width and depth: 64-wide heads in the same numbers, its experts all active and
+        # together as wide as the feed-forward
+        other = binfmt.Config(vocab_size=cfg["vocab"], hidden_dim=W, n_experts=4, experts_per_token=4,
+                              intermediate_dim=shape["ff"] // 4, n_layers=L, head_dim=64,
+                              n_attn_heads=shape["attn_heads"], n_kv_heads=shape["kv_heads"], seq_len=positions,
+                              initial_context_length=4096, rope_theta=150000.0, rope_scaling_factor=32.0,
+                              sliding_window=window, swiglu_limit=7.0)
+        with tempfile.TemporaryDirectory() as d:
+            with open(os.path.join(d, "config.json"), "w") as f:
+                json.dump(cfg, f)
+            eng = ops.Engine.open(d, max_batch=max(B, Bp), max_seq=positions, synthetic=True, keep_logits=False)
+        mean_prompt = (window * (T - window) + window * (window + 1) / 2) / T if T > window else (T + 1) / 2
+        row = {}
+        for who, e, works in (
+                ("nezavik", eng, (_nezavik_work(cfg, B, B, min(window, ctx)),
+                                  _nezavik_work(cfg, Bp * T, Bp, mean_prompt))),
+                ("gpt_oss", None, (_gptoss_work(other, B, B, (ctx, min(window, ctx))),
+                                   _gptoss_work(other, Bp * T, Bp, ((T + 1) / 2, mean_prompt))))):
+            if e is None:
+                e = ops.Engine(other, None, max_batch=max(B, Bp), max_seq=positions, synthetic=True, keep_logits=False)
+            r = _time_engine(ops, torch, e, cfg["vocab"], decode, prompt, steps)
+            row[who] = {"decode_ms": round(r["decode"][0], 3), "decode_tok_s": round(B / r["decode"][0] * 1e3, 1),
+                        "prefill_ms": round(r["prefill"][0], 2), "prefill_tok_s": round(Bp * T / r["prefill"][0] * 1e3, 1),
+                        "device_gb": round(e.device_bytes() / 1e9, 2),
+                        "decode_kernels": _against_roofline(r["decode"][1], works[0]),
+                        "prefill_kernels": _against_roofline(r["prefill"][1], works[1])}
+            e.close()
+            del e
+        row["config"] = dict(shape, decode=f"{B} sequences at position {ctx}", prefill=f"{Bp} prompts of {T}")
+        out[name] = row
+        print(f"{name}: done", file=sys.stderr, flush=True)
+    return out
+
+
 def bench_mfma_rates(torch):
     """Register-fed rate of the matrix instructions (no loads, no LDS): 256 workgroups of 8 waves."""
     import ctypes as C
@@ -565,6 +772,13 @@ def main():
     if args.mfma_rates:
         print(json.dumps({"what": "register-fed MFMA issue rates, 256 workgroups x 8 waves x 4 accumulators",
                           "rates": bench_mfma_rates(torch)}))
+        return
+
+    if args.model == "nezavik":
+        only = [x for x in args.only.split(",") if x]
+        print(json.dumps({"what": "Nezavik beside GPT-OSS of the same width (random weights, bf16): ms per step, kernel "
+                                  "times and fraction of roofline (8 TB/s HBM, 2.5 PFLOP/s bf16, 78.6 TFLOP/s fp32)",
+                          "sizes": bench_nezavik(ops, torch, max(10, args.steps), only)}))
         return
 
     # a plain device copy of known size (2 x 1 GiB moved), so counter runs of this same command can

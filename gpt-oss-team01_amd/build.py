@@ -26,7 +26,7 @@ DEVICE = ["--offload-arch=gfx950", "-Xclang", "-target-feature", "-Xclang", "-pa
 
 #: sources every model class links
 CORE = ("common.cpp", "engine.cpp", "model_registry.cpp", "glue.hip", "precise.hip", "gemm_dense.cpp",
-        "gemm_bf16.hip", "gemm_tall.hip")
+        "gemm_bf16.hip", "gemm_mixed_bf16.hip", "gemm_tall.hip")
 #: architecture -> sources of its class beside CORE (None: all of them)
 MODELS = {"gpt-oss": None, "Nezavik": ("model_nezavik.cpp", "recurrent.hip", "window_attn.hip")}
 

@@ -4,7 +4,16 @@
 
 namespace gptoss {
 
-enum { EPI_F32 = 0, EPI_SWIGLU = 1, EPI_BF16 = 2, EPI_ARGMAX = 3 };
+enum { EPI_F32 = 0, EPI_SWIGLU = 1, EPI_BF16 = 2, EPI_ARGMAX = 3, EPI_MIXED = 4, EPI_PARTIAL = 5 };
+
+// EPI_MIXED (dense): the columns of one product leave in two ways.  fp32 rows of N as with EPI_F32, except
+// for up to two ranges of whole 32-column blocks that become bf16 rows of their own.
+struct GemmBf16Range {
+  int from = 0, to = 0;   // columns [from, to), multiples of 32; empty: none
+  bf16_t *out = nullptr;  // column `from` of row 0
+  int ld = 0;             // elements per row, a multiple of 4
+  int relu_squared = 0;   // the square of relu instead of the value itself
+};
 
 // Row tiles of ONE expert are grouped into blocks of up to MOE_TILE_BLOCK consecutive tiles by the
 // grouping kernel; a block never spans two experts, so every tile of a block multiplies the same
@@ -34,6 +43,9 @@ struct GemmParams {
   int N, K;
   int n_col_tiles;     // gemm_col_tiles(N)
   float limit;         // SwiGLU clamp
+  GemmBf16Range range[2];  // EPI_MIXED
+  int k_splits;        // EPI_PARTIAL (dense only): the sum over K is cut into k_splits parts of split_slabs
+  int split_slabs;     // 64-k slabs; part s is written to out + s * dense_rows * N (no bias)
 };
 
 // rows_per_tile in {32,64,96,128,160}, or 256 where gemm_tall_applies(); max_tiles bounds the number of
@@ -88,6 +100,14 @@ int moe_rows_per_tile(int B, int k, int E, bool mxfp4);
 // at most gemm_argmax_tiles(N), for run_argmax_tiles to finish
 int dense_gemm(const bf16_t *A, const bf16_t *W, const float *bias, void *out, int epi, int B, int N, int K,
                hipStream_t s, float *amax_val = nullptr, int *amax_idx = nullptr, int *amax_tiles = nullptr);
+// EPI_MIXED
+int dense_gemm_mixed(const bf16_t *A, const bf16_t *W, float *out, const GemmBf16Range *ranges, int n_ranges, int B,
+                     int N, int K, hipStream_t s);
+// C = A . W^T as *parts fp32 partial sums [*parts][B, N] (the caller adds them up) where that fills the chip
+// better; at most GEMM_MAX_PARTS, and at most max_elems / (B * N)
+constexpr int GEMM_MAX_PARTS = 16;
+int dense_gemm_partial(const bf16_t *A, const bf16_t *W, float *out, size_t max_elems, int *parts, int B, int N, int K,
+                       hipStream_t s);
 int gemm_col_tiles(int N);  // column tiles of one workgroup's width
 inline int gemm_argmax_tiles(int N) { return 2 * gemm_col_tiles(N); }  // pairs per row to allocate for EPI_ARGMAX
 // moe_route.hip

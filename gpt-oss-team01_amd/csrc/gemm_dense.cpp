@@ -44,7 +44,7 @@ __global__ __launch_bounds__(256) void pack_weight_kernel(const SRC *__restrict_
 
 // Host-side dispatcher of the form without gather.  rows_per_tile selects the kernel.
 template <int MBMAX, bool GATHER, int EPI, bool FP4>
-int launch_gemm(const GemmParams &p, int max_tiles, hipStream_t s);  // gemm_bf16.hip
+int launch_gemm(const GemmParams &p, int max_tiles, hipStream_t s);  // gemm_bf16.hip, gemm_mixed_bf16.hip
 
 template <int EPI>
 static int dispatch_rows(const GemmParams &p, int rows_per_tile, int max_tiles, hipStream_t s) {
@@ -58,7 +58,8 @@ static int dispatch_rows(const GemmParams &p, int rows_per_tile, int max_tiles, 
   return fail(GPTOSS_ERR_DIM, "run_gemm: unsupported rows_per_tile %d", rows_per_tile);
 }
 
-hipError_t gemm_set_attrs_bf16();  // gemm_bf16.hip
+hipError_t gemm_set_attrs_bf16();        // gemm_bf16.hip
+hipError_t gemm_set_attrs_mixed_bf16();  // gemm_mixed_bf16.hip
 
 // Raises the dynamic-LDS limit of every such kernel on the calling thread's current device, the
 // first time that device launches one.
@@ -72,6 +73,7 @@ static int gemm_prepare_device() {
   std::lock_guard<std::mutex> lock(mu);
   if (!done[dev]) {
     GPTOSS_HIP(gemm_set_attrs_bf16());
+    GPTOSS_HIP(gemm_set_attrs_mixed_bf16());
     done[dev] = true;
   }
   return GPTOSS_OK;
@@ -86,6 +88,8 @@ int run_gemm_dense(const GemmParams &p, int epi, int rows_per_tile, int max_tile
   int prc = gemm_prepare_device();
   if (prc != GPTOSS_OK) return prc;
   if (epi == EPI_F32) return dispatch_rows<EPI_F32>(p, rows_per_tile, max_tiles, s);
+  if (epi == EPI_MIXED && p.tiles == nullptr) return dispatch_rows<EPI_MIXED>(p, rows_per_tile, max_tiles, s);
+  if (epi == EPI_PARTIAL && p.tiles == nullptr) return dispatch_rows<EPI_PARTIAL>(p, rows_per_tile, max_tiles, s);
   if (epi == EPI_ARGMAX && p.tiles == nullptr && p.amax_val && p.amax_idx)
     return dispatch_rows<EPI_ARGMAX>(p, rows_per_tile, max_tiles, s);
   return fail(GPTOSS_ERR_DIM, "run_gemm: unsupported combination (dense, epi=%d)", epi);
@@ -112,13 +116,34 @@ static int argmax_tall_min_rows() {
   return v;
 }
 
-// C[B, N] = A[B, K] . W[N, K]^T (+ bias): the dense GEMMs of a step (QKV and output projections,
-// classifier), with the kernel and row tile chosen from the batch size.
-int dense_gemm(const bf16_t *A, const bf16_t *W, const float *bias, void *out, int epi, int B, int N,
-               int K, hipStream_t s, float *amax_val, int *amax_idx, int *amax_tiles) {
+// Row tile of a dense GEMM on the streaming kernels.  Up to 96 rows: the smallest size that holds every
+// row, so the weights are requested once.  A prompt pass (thousands of rows): 160 rows, every weight
+// fragment feeds five MFMAs.  In between the launch is a handful of rounds of work items on 256 CUs, and
+// an item of MB 32-row blocks takes (0.39 + 0.115 MB) us per 64-k slab (measured at 1024 rows: 0.50 /
+// 0.64 / 0.76 / 0.85 us for 32 / 64 / 96 / 128 rows), so the tile that needs the least rounds x slab time
+// wins: 96 rows for the QKV projection of 1024 rows (220 items, one round), 64 for the output
+// projection (192 items instead of 132: 48 -> 41 us).
+static double slab_us(int mb) { return 0.39 + 0.115 * mb; }
+
+static int dense_rows_per_tile(int B, int n_col_tiles) {
+  if (B <= 96) return align_up(B, 32);
+  if (B < 2048 && n_col_tiles >= 64) return 128;  // the unembedding: hundreds of column tiles, measured best at 1024 rows
+  if (B >= 2048) return 160;
+  double best = 0.0;
+  int rpt = 160;
+  for (int mb = 1; mb <= 5; mb++) {
+    const long long items = (long long)cdiv(B, 32 * mb) * n_col_tiles;
+    const double cost = (double)((items + 255) / 256) * slab_us(mb);
+    if (mb == 1 || cost <= best) {  // ties go to the larger tile: fewer re-reads of the weights
+      best = cost;
+      rpt = 32 * mb;
+    }
+  }
+  return rpt;
+}
+
+static GemmParams dense_params(const bf16_t *A, const bf16_t *W, const float *bias, void *out, int B, int N, int K) {
   GemmParams g{};
-  g.amax_val = amax_val;
-  g.amax_idx = amax_idx;
   g.A = A;
   g.W = W;
   g.bias = bias;
@@ -128,34 +153,17 @@ int dense_gemm(const bf16_t *A, const bf16_t *W, const float *bias, void *out, i
   g.N = N;
   g.K = K;
   g.n_col_tiles = gemm_col_tiles(N);
-  // Row tile.  Up to 96 rows: the smallest size that holds every row, so the weights are requested
-  // once.  A prompt pass (thousands of rows): 160 rows, every weight fragment feeds five MFMAs.  In
-  // between the launch is a handful of rounds of work items on 256 CUs, and an item of MB 32-row
-  // blocks takes (0.39 + 0.115 MB) us per 64-k slab (measured at 1024 rows: 0.50 / 0.64 / 0.76 /
-  // 0.85 us for 32 / 64 / 96 / 128 rows), so the tile that needs the least rounds x slab time wins:
-  // 96 rows for the QKV projection of 1024 rows (220 items, one round), 64 for the output
-  // projection (192 items instead of 132: 48 -> 41 us).
-  static const int sizes[5] = {32, 64, 96, 128, 160};
-  int rpt = 160;
-  if (B <= 96) {
-    for (int i = 0; i < 5; i++)
-      if (B <= sizes[i]) {
-        rpt = sizes[i];
-        break;
-      }
-  } else if (B < 2048 && g.n_col_tiles >= 64) {
-    rpt = 128;  // the unembedding: hundreds of column tiles, measured best at 1024 rows
-  } else if (B < 2048) {
-    double best = 0.0;
-    for (int mb = 1; mb <= 5; mb++) {
-      const long long items = (long long)cdiv(B, 32 * mb) * g.n_col_tiles;
-      const double cost = (double)((items + 255) / 256) * (0.39 + 0.115 * mb);
-      if (mb == 1 || cost <= best) {  // ties go to the larger tile: fewer re-reads of the weights
-        best = cost;
-        rpt = 32 * mb;
-      }
-    }
-  }
+  return g;
+}
+
+// C[B, N] = A[B, K] . W[N, K]^T (+ bias): the dense GEMMs of a step (QKV and output projections,
+// classifier), with the kernel and row tile chosen from the batch size.
+int dense_gemm(const bf16_t *A, const bf16_t *W, const float *bias, void *out, int epi, int B, int N,
+               int K, hipStream_t s, float *amax_val, int *amax_idx, int *amax_tiles) {
+  GemmParams g = dense_params(A, W, bias, out, B, N, K);
+  g.amax_val = amax_val;
+  g.amax_idx = amax_idx;
+  int rpt = dense_rows_per_tile(B, g.n_col_tiles);
   if (B >= (epi == EPI_ARGMAX ? argmax_tall_min_rows() : dense_tall_min_rows()) && gemm_tall_applies(g, false, epi) &&
       gemm_tall_shape_ok(N, K, B))
     rpt = 256;
@@ -164,6 +172,54 @@ int dense_gemm(const bf16_t *A, const bf16_t *W, const float *bias, void *out, i
     *amax_tiles = rpt == 256 ? 2 * g.n_col_tiles : g.n_col_tiles;
   }
   return run_gemm_dense(g, epi, rpt, cdiv(B, rpt), s);
+}
+
+int dense_gemm_mixed(const bf16_t *A, const bf16_t *W, float *out, const GemmBf16Range *ranges, int n_ranges, int B,
+                     int N, int K, hipStream_t s) {
+  GPTOSS_REQUIRE(n_ranges >= 0 && n_ranges <= 2, GPTOSS_ERR_DIM, "dense_gemm_mixed: %d ranges", n_ranges);
+  GemmParams g = dense_params(A, W, nullptr, out, B, N, K);
+  for (int i = 0; i < n_ranges; i++) {
+    g.range[i] = ranges[i];
+    GPTOSS_REQUIRE(ranges[i].from % 32 == 0 && ranges[i].to % 32 == 0 && ranges[i].ld % 4 == 0 && aligned(ranges[i].out, 8),
+                   GPTOSS_ERR_DIM, "dense_gemm_mixed: ranges are whole 32-column blocks of aligned rows");
+  }
+  int rpt = dense_rows_per_tile(B, g.n_col_tiles);
+  if (B >= dense_tall_min_rows() && gemm_tall_applies(g, false, EPI_MIXED) && gemm_tall_shape_ok(N, K, B)) rpt = 256;
+  return run_gemm_dense(g, EPI_MIXED, rpt, cdiv(B, rpt), s);
+}
+
+// Few rows and few columns leave most CUs without a work item while those that have one walk all of K.
+// Cutting K makes more items; what it costs is a fixed part per item and the partial sums' way to memory
+// and back.
+int dense_gemm_partial(const bf16_t *A, const bf16_t *W, float *out, size_t max_elems, int *parts, int B, int N, int K,
+                       hipStream_t s) {
+  *parts = 1;
+  GemmParams g = dense_params(A, W, nullptr, out, B, N, K);
+  if (B >= dense_tall_min_rows()) return dense_gemm(A, W, nullptr, out, EPI_F32, B, N, K, s);
+  const int nslab = K / 64;
+  double best = 0.0;
+  int rpt = 32, splits = 1, slabs = nslab;
+  for (int mb = 1; mb <= 5; mb++) {
+    if (mb > 1 && 32 * (mb - 1) >= B) break;
+    for (int want = 1; want <= GEMM_MAX_PARTS; want++) {
+      const int per = cdiv(nslab, want), n = cdiv(nslab, per);
+      // (an item prefetches two slabs of the next one, so no part may have fewer)
+      if (n != want || (n > 1 && (per < 4 || nslab - per * (n - 1) < 2 || (size_t)n * B * N > max_elems))) continue;
+      const long long items = (long long)cdiv(B, 32 * mb) * g.n_col_tiles * n;
+      const double cost = (double)((items + 255) / 256) * (per * slab_us(mb) + 5.0) + (n - 1) * (double)B * N * 8 / 5e6;
+      if ((mb == 1 && n == 1) || cost < best) {
+        best = cost;
+        rpt = 32 * mb;
+        splits = n;
+        slabs = per;
+      }
+    }
+  }
+  if (splits == 1) return run_gemm_dense(g, EPI_F32, rpt, cdiv(B, rpt), s);
+  g.k_splits = splits;
+  g.split_slabs = slabs;
+  *parts = splits;
+  return run_gemm_dense(g, EPI_PARTIAL, rpt, cdiv(B, rpt), s);
 }
 
 }  // namespace gptoss

@@ -23,7 +23,8 @@
 //     row and 16 channels: stores are 8/16 bytes wide, and since the packing order puts the gates
 //     of 16 (gate,up) pairs in channels 0-15 of a wave's block and their ups in channels 16-31,
 //     each pair sits in two registers of the same lane;
-//   * epilogues: +bias -> fp32, or +bias -> clamped SwiGLU -> bf16.
+//   * epilogues: +bias -> fp32, or +bias -> clamped SwiGLU -> bf16; for the dense form also the row arg-max,
+//     fp32 next to bf16 column ranges, and partial sums over parts of K.
 #pragma once
 
 #include <type_traits>
@@ -74,7 +75,7 @@ struct WStream {
 };
 
 template <bool FP4>
-__device__ __forceinline__ WStream w_stream(const GemmParams &p, int mat, int ct, int wave) {
+__device__ __forceinline__ WStream w_stream(const GemmParams &p, int mat, int ct, int wave, int slab0 = 0) {
   const int K = p.K, N = p.N;
   int n0 = ct * BN + wave * 32;
   if (n0 >= N) n0 = N - 32;  // idle waves of the last column tile stream a valid block again
@@ -86,7 +87,7 @@ __device__ __forceinline__ WStream w_stream(const GemmParams &p, int mat, int ct
     st.c = mb_ + (size_t)(n0 >> 5) * nslab * 1024;
     st.sc = mb_ + (size_t)N * K / 2 + (size_t)(n0 >> 5) * nslab * 64;
   } else {
-    st.w = p.W + (size_t)mat * N * K + (size_t)(n0 >> 5) * (K / 16) * 512;
+    st.w = p.W + (size_t)mat * N * K + ((size_t)(n0 >> 5) * (K / 16) + slab0 * 4) * 512;
   }
   return st;
 }
@@ -200,6 +201,34 @@ __device__ __forceinline__ void epilogue_store(const GemmParams &p, int mat, int
         const float lo = bp ? bp[g * 8 + q] : 0.f, hi_v = bp ? bp[g * 8 + 4 + q] : 0.f;
         bv[g * 4 + q] = hi ? hi_v : lo;
       }
+    if constexpr (EPI == EPI_MIXED) {
+#pragma unroll
+      for (int x = 0; x < 2; x++) {
+        const GemmBf16Range &rg = p.range[x];
+        if (n0 >= rg.from && n0 < rg.to) {   // wave-uniform: a wave's 32 columns lie in one range or in none
+          bf16_t *o = rg.out + (size_t)(row0 + tok) * rg.ld + (n0 - rg.from) + h4;
+#pragma unroll
+          for (int i = 0; i < MB; i++)
+            if (i * 32 < rows - tok) {
+#pragma unroll
+              for (int g = 0; g < 4; g++) {
+                float v[4];
+#pragma unroll
+                for (int q = 0; q < 4; q++) {
+                  v[q] = acc[i][g * 4 + q] + bv[g * 4 + q];
+                  if (rg.relu_squared) {
+                    v[q] = fmaxf(v[q], 0.f);
+                    v[q] *= v[q];
+                  }
+                }
+                *reinterpret_cast<u32x2 *>(o + (size_t)(i * 32) * rg.ld + g * 8) =
+                    u32x2{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
+              }
+            }
+          return;
+        }
+      }
+    }
     const uint32_t lane_off = (uint32_t)tok * (uint32_t)N + (uint32_t)h4;
     const int row_lim = rows - tok;
 #pragma unroll
@@ -211,7 +240,7 @@ __device__ __forceinline__ void epilogue_store(const GemmParams &p, int mat, int
           float v[4];
 #pragma unroll
           for (int q = 0; q < 4; q++) v[q] = acc[i][g * 4 + q] + bv[g * 4 + q];
-          if (EPI == EPI_F32)
+          if (EPI == EPI_F32 || EPI == EPI_MIXED)
             *reinterpret_cast<f32x4 *>(reinterpret_cast<float *>(p.out) + row_off + lane_off + g * 8) =
                 f32x4{v[0], v[1], v[2], v[3]};
           else
@@ -231,7 +260,8 @@ __device__ __forceinline__ void epilogue_store(const GemmParams &p, int mat, int
 template <int MB, int MBMAX, int NRING, bool GATHER, int EPI, bool FP4, bool ONCE>
 __device__ __forceinline__ void gemm_tile(const GemmParams &p, bf16_t *lds, int mat, int row0, int rows,
                                           int ct, WRing<NRING, FP4> &ring, const WStream &cur,
-                                          const WStream &next, bf16_t *hold = nullptr) {
+                                          const WStream &next, bf16_t *hold = nullptr, int slab0 = 0,
+                                          int part_slabs = 0, float *part_out = nullptr) {
   constexpr int LDS_STAGE = MBMAX * 32 * LDS_ROW;  // elements per A stage
   constexpr int D = NRING - 1;                     // slabs of W in flight
   constexpr int BQ = WRing<NRING, FP4>::BQ;
@@ -242,7 +272,7 @@ __device__ __forceinline__ void gemm_tile(const GemmParams &p, bf16_t *lds, int 
   const int K = p.K, N = p.N;
   const int n0 = ct * BN + wave * 32;
   const bool wave_active = n0 < N;
-  const int nslab = K / BK;
+  const int nslab = EPI == EPI_PARTIAL ? part_slabs : K / BK;
 
   // ---- A: the workgroup moves APASS rows x 8 chunks of 16 bytes per pass ----------------------
   const int a_row = tid >> 3, a_kc = tid & 7;
@@ -258,6 +288,7 @@ __device__ __forceinline__ void gemm_tile(const GemmParams &p, bf16_t *lds, int 
       else src = row0 + r;
     }
     a_off[i] = (uint32_t)src * (uint32_t)K + a_kc * 8;
+    if (EPI == EPI_PARTIAL) a_off[i] += (uint32_t)slab0 * BK;
   }
   // Register sets for A in flight.  With bf16 weights a slab's rows are requested one iteration
   // before they are stored to LDS; with MXFP4 weights the iterations are short (a quarter of the
@@ -478,7 +509,13 @@ __device__ __forceinline__ void gemm_tile(const GemmParams &p, bf16_t *lds, int 
   }
   if (!wave_active) return;
 
-  epilogue_store<MB, EPI>(p, mat, row0, rows, n0, lane, acc, hold, wave * 16);
+  if constexpr (EPI == EPI_PARTIAL) {
+    GemmParams q = p;
+    q.out = part_out;
+    epilogue_store<MB, EPI_F32>(q, mat, row0, rows, n0, lane, acc);
+  } else {
+    epilogue_store<MB, EPI>(p, mat, row0, rows, n0, lane, acc, hold, wave * 16);
+  }
 }
 
 // Kernels that keep two finished SwiGLU tiles in LDS until the workgroup's last item is done (see
@@ -518,7 +555,8 @@ __global__ __launch_bounds__(GEMM_THREADS, (gemm_two_per_cu(MBMAX, FP4) ? 4 : 2)
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
 
   const int n_tiles = p.tiles ? p.tiles[0] : (p.dense_rows + BM - 1) / BM;
-  const int total = n_tiles * p.n_col_tiles;
+  const int tile_items = n_tiles * p.n_col_tiles;
+  const int total = EPI == EPI_PARTIAL ? tile_items * p.k_splits : tile_items;
   const int per_xcd = gridDim.x >> 3;
   const int xcd = blockIdx.x & 7;
   int lo, hi;  // this XCD's part of the work list
@@ -537,11 +575,16 @@ __global__ __launch_bounds__(GEMM_THREADS, (gemm_two_per_cu(MBMAX, FP4) ? 4 : 2)
 
   struct Item {
     int mat, row0, rows, ct;
+    int part = 0;  // EPI_PARTIAL: which part of the sum over K
     int once;  // no other row tile multiplies this item's W (an int: the struct has no padding to copy)
   };
   auto decode = [&](int jj) {
-    const int work = lo + jj;
+    int work = lo + jj;
     Item it;
+    if (EPI == EPI_PARTIAL) {
+      it.part = work / tile_items;
+      work -= it.part * tile_items;
+    }
     int tile;
     if (p.tiles && p.tile_block > 1 && p.xcd_bounds) {
       // grouped, experts with several row tiles: the row tiles of one expert form blocks of up to
@@ -593,17 +636,22 @@ __global__ __launch_bounds__(GEMM_THREADS, (gemm_two_per_cu(MBMAX, FP4) ? 4 : 2)
   int it = 0;
   int held_row0_a = 0, held_rows_a = 0, held_ct_a = 0, held_row0_b = 0, held_rows_b = 0, held_ct_b = 0;
   Item cur = decode(j);
-  WStream cur_w = w_stream<FP4>(p, cur.mat, cur.ct, wave);
+  // EPI_PARTIAL: first slab and slabs of an item's part of K
+  auto part_slab0 = [&](const Item &i) { return EPI == EPI_PARTIAL ? i.part * p.split_slabs : 0; };
+  auto part_slabs = [&](const Item &i) { return EPI == EPI_PARTIAL ? min(p.split_slabs, p.K / BK - i.part * p.split_slabs) : 0; };
+  WStream cur_w = w_stream<FP4>(p, cur.mat, cur.ct, wave, part_slab0(cur));
   WRing<NRING, FP4> ring;
   static_for<0, NRING - 1>([&](auto r) {
-    w_load<NRING, FP4, false>(ring, cur_w, min((int)decltype(r)::value, p.K / BK - 1), lane, r);
+    const int last = EPI == EPI_PARTIAL ? part_slabs(cur) - 1 : p.K / BK - 1;
+    w_load<NRING, FP4, false>(ring, cur_w, min((int)decltype(r)::value, last), lane, r);
   });
   while (true) {
     const int jn = j + per_xcd;
     const bool more = valid(jn);
     const Item nxt = more ? decode(jn) : cur;
     // without a next item the refill re-reads this item's first slabs: harmless and unconditional
-    const WStream nxt_w = more ? w_stream<FP4>(p, nxt.mat, nxt.ct, wave) : cur_w;
+    const WStream nxt_w = more ? w_stream<FP4>(p, nxt.mat, nxt.ct, wave, part_slab0(nxt)) : cur_w;
+    float *part_out = EPI == EPI_PARTIAL ? (float *)p.out + (size_t)cur.part * p.dense_rows * p.N : nullptr;
     // one fully unrolled code path per number of 32-row blocks actually present in the tile
     const int mb = (cur.rows + 31) >> 5;
     bf16_t *hold_ptr = nullptr;
@@ -627,10 +675,12 @@ __global__ __launch_bounds__(GEMM_THREADS, (gemm_two_per_cu(MBMAX, FP4) ? 4 : 2)
         // the refill of the ring from the next item follows this item's choice
         if (!FP4 && cur.once)   // MXFP4 weights: a quarter of the bytes, not bound by their stream; one path keeps the 128-register kernels free of spills
           gemm_tile<M, MBMAX, NRING, GATHER, EPI, FP4, true>(p, lds, cur.mat, cur.row0, cur.rows, cur.ct, ring,
-                                                             cur_w, nxt_w, hold_ptr);
+                                                             cur_w, nxt_w, hold_ptr, part_slab0(cur), part_slabs(cur),
+                                                             part_out);
         else
           gemm_tile<M, MBMAX, NRING, GATHER, EPI, FP4, false>(p, lds, cur.mat, cur.row0, cur.rows, cur.ct, ring,
-                                                              cur_w, nxt_w, hold_ptr);
+                                                              cur_w, nxt_w, hold_ptr, part_slab0(cur), part_slabs(cur),
+                                                              part_out);
         done = true;
       }
     });
@@ -679,7 +729,7 @@ template <int MBMAX, bool GATHER, int EPI, bool FP4>
 int launch_gemm(const GemmParams &p, int max_tiles, hipStream_t s) {
   const size_t smem = gemm_smem_bytes<MBMAX, gemm_holds_output(GATHER, EPI, FP4)>();
   auto kern = grouped_gemm_kernel<MBMAX, GATHER, EPI, FP4>;
-  int total = max_tiles * p.n_col_tiles;
+  int total = max_tiles * p.n_col_tiles * (EPI == EPI_PARTIAL ? p.k_splits : 1);
   int grid = ((total + 7) / 8) * 8;
   // resident workgroups: one of 8 waves (2 per SIMD) per CU, or two where the registers allow
   const int resident = gemm_two_per_cu(MBMAX, FP4) ? 512 : 256;

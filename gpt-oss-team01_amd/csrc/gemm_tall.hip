@@ -4,7 +4,7 @@
 namespace gptoss {
 
 bool gemm_tall_applies(const GemmParams &p, bool gather, int epi) {
-  const bool kind = (gather && epi == EPI_SWIGLU) || (!gather && epi == EPI_F32) ||
+  const bool kind = (gather && epi == EPI_SWIGLU) || (!gather && (epi == EPI_F32 || epi == EPI_MIXED)) ||
                     (!gather && epi == EPI_ARGMAX && p.tiles == nullptr && p.amax_val && p.amax_idx);
   // whole A chunks of 64 k, and at least 8 stages: an item's first loads are requested during the
   // last four stages of the item before it
@@ -27,6 +27,7 @@ int run_gemm_tall(const GemmParams &p, int epi, int max_tiles, long long max_row
   if (rc != GPTOSS_OK) return rc;
   static_assert(Tall256::WC == 2, "dense_gemm reports two arg-max pairs per row and column tile");
   if (epi == EPI_ARGMAX) return launch_tall<Tall256, false, EPI_ARGMAX>(p, max_tiles, s);
+  if (epi == EPI_MIXED) return launch_tall<Tall256, false, EPI_MIXED>(p, max_tiles, s);
   return launch_tall<Tall256, false, EPI_F32>(p, max_tiles, s);
 }
 

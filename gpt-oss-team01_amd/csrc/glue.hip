@@ -529,11 +529,12 @@ __global__ __launch_bounds__(256) void embedding_position_kernel(const T *__rest
 }
 
 // The depth average behind layer i and the norm in front of layer i + 1: X = x + y (the layer's
-// result, kept in history[i + 1]), x = sum_j weights[j] * history[j] over j = 0 .. i + 1, and
+// result, kept in history[i + 1]; y in `parts` partial sums), x = sum_j weights[j] * history[j] over j = 0 .. i + 1, and
 // t = weight * x / sqrt(mean(x^2) + eps).  history: [layers + 1][rows_cap, H]; norm_w nullptr: no norm.
 template <int VPT>
 __global__ __launch_bounds__(256) void depth_average_norm_kernel(float *__restrict__ x, const float *__restrict__ y,
                                                                  float *__restrict__ history, size_t plane,
+                                                                 int parts, size_t part_stride,
                                                                  const float *__restrict__ weights, int layer,
                                                                  const float *__restrict__ norm_w,
                                                                  bf16_t *__restrict__ t_bf16,
@@ -548,7 +549,9 @@ __global__ __launch_bounds__(256) void depth_average_norm_kernel(float *__restri
     const int h = (threadIdx.x + 256 * i) * 4;
     v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (h < H) {
-      const f32x4 own = *reinterpret_cast<const f32x4 *>(x + row + h) + *reinterpret_cast<const f32x4 *>(y + row + h);
+      f32x4 own = *reinterpret_cast<const f32x4 *>(y + row + h);
+      for (int j = 1; j < parts; j++) own += *reinterpret_cast<const f32x4 *>(y + j * part_stride + row + h);
+      own += *reinterpret_cast<const f32x4 *>(x + row + h);
       *reinterpret_cast<f32x4 *>(history + (size_t)(layer + 1) * plane + row + h) = own;
       f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
       for (int j = 0; j <= layer; j++)
@@ -599,13 +602,13 @@ int run_embedding_position_f32(const float *table, const float *positions, const
   return launch_embedding_position(table, positions, tokens, lens, x, x0, rows, H, ld, V, n_pos, s);
 }
 
-int run_depth_average_norm(float *x, const float *y, float *history, size_t plane, const float *weights, int layer,
-                           const float *norm_w, bf16_t *t_bf16, float *t_f32, int rows, int H, float eps, int n_mean,
+int run_depth_average_norm(float *x, const float *y, int parts, float *history, size_t plane, const float *weights,
+                           int layer, const float *norm_w, bf16_t *t_bf16, float *t_f32, int rows, int H, float eps, int n_mean,
                            hipStream_t s) {
   GPTOSS_REQUIRE(H % 4 == 0 && H <= 16384, GPTOSS_ERR_DIM, "depth_average: rows of %d elements (a multiple of 4, at most 16384)", H);
   TraceScope ts("depth_average_norm", s);
   auto go = [&](auto kern) {
-    kern<<<rows, 256, 0, s>>>(x, y, history, plane, weights, layer, norm_w, t_bf16, t_f32, H, eps, n_mean);
+    kern<<<rows, 256, 0, s>>>(x, y, history, plane, parts, (size_t)rows * H, weights, layer, norm_w, t_bf16, t_f32, H, eps, n_mean);
   };
   if (H <= 1024) go(depth_average_norm_kernel<1>);
   else if (H <= 2048) go(depth_average_norm_kernel<2>);

@@ -14,10 +14,10 @@ int run_embedding_position(const bf16_t *table, const bf16_t *positions, const i
                            float *x0, int rows, int H, int ld, int V, int n_pos, hipStream_t s);
 int run_embedding_position_f32(const float *table, const float *positions, const int *tokens, const int *lens,
                                float *x, float *x0, int rows, int H, int ld, int V, int n_pos, hipStream_t s);
-// history[layer + 1] = x + y; x = sum over j <= layer + 1 of weights[j] * history[j] (planes of `plane`
+// history[layer + 1] = x + y (y: `parts` partial sums [rows, H]); x = sum over j <= layer + 1 of weights[j] * history[j] (planes of `plane`
 // elements); with norm_w also t = RMSNorm(x) * norm_w
-int run_depth_average_norm(float *x, const float *y, float *history, size_t plane, const float *weights, int layer,
-                           const float *norm_w, bf16_t *t_bf16, float *t_f32, int rows, int H, float eps, int n_mean,
+int run_depth_average_norm(float *x, const float *y, int parts, float *history, size_t plane, const float *weights,
+                           int layer, const float *norm_w, bf16_t *t_bf16, float *t_f32, int rows, int H, float eps, int n_mean,
                            hipStream_t s);
 int run_rope_store(const float *qkv, float *q_out, bf16_t *kv, const float *cos_t,
                    const float *sin_t, int B, int n_q, int n_kv, int D, int cap, int pos,

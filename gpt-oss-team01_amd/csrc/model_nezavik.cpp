@@ -59,7 +59,8 @@ struct Nezavik final : gptoss_engine {
   // activations of a pass
   Shapes wide;
   float *in_rows = nullptr, *conv_rows = nullptr, *y_rows = nullptr, *low_out_rows = nullptr, *q_rows = nullptr;
-  float *branch = nullptr, *history = nullptr;   // [rows, hidden], [layers + 1][rows, hidden]
+  float *branch = nullptr, *history = nullptr;   // partial sums of [rows, hidden], [layers + 1][rows, hidden]
+  size_t branch_elems = 0;
   bf16_t *t_rows = nullptr;
   float *t_rows_f32 = nullptr;
   void *act_rows = nullptr, *low_rows = nullptr;
@@ -68,11 +69,30 @@ struct Nezavik final : gptoss_engine {
   int check_segments(const std::vector<RowSeg> &segs) override;
   int forward_rows(const StepRows &r) override;
 
+  int project_in(const NezavikLayer &w, int n);
   int gemm(const Matrix &m, const bf16_t *a, const float *a_f32, float *out, int n) {
     if (precise()) return precise_matmul(out, a_f32, m.f32, nullptr, nullptr, n, m.n_in, m.n_out, 1, stream);
     return dense_gemm(a, m.packed, nullptr, out, EPI_F32, n, m.n_out, m.n_in, stream);
   }
 };
+
+// Everything that reads the norm's output: mixer projections in fp32; the feed-forward's activations and
+// the inner ends of the low-rank pairs go where the next products read them.
+int Nezavik::project_in(const NezavikLayer &w, int n) {
+  const int ld_in = w.in.n_out, ld_act = w.out.n_in, ld_low = w.low_rank.n_in;
+  if (precise()) {
+    GPTOSS_STEP(gemm(w.in, nullptr, t_rows_f32, in_rows, n));
+    if (w.ff) GPTOSS_STEP(run_column_map(in_rows, ld_in, w.up_col, w.ff, true, (float *)act_rows, ld_act, n, stream));
+    if (w.low_width)
+      GPTOSS_STEP(run_column_map(in_rows, ld_in, w.low_col, w.low_width, false, (float *)low_rows, ld_low, n, stream));
+    return GPTOSS_OK;
+  }
+  GemmBf16Range ranges[2];
+  int k = 0;
+  if (w.ff) ranges[k++] = {w.up_col, ld_in, (bf16_t *)act_rows, ld_act, 1};   // the last columns
+  if (w.low_width) ranges[k++] = {w.low_col, w.low_col + (w.low_width + 31) / 32 * 32, (bf16_t *)low_rows, ld_low, 0};
+  return dense_gemm_mixed(t_rows, w.in.packed, in_rows, ranges, k, n, ld_in, w.in.n_in, stream);
+}
 
 // A recurrent state knows only its own position: a sequence goes on where it stopped, or starts over.
 int Nezavik::check_segments(const std::vector<RowSeg> &segs) {
@@ -97,8 +117,7 @@ int Nezavik::forward_rows(const StepRows &r) {
   for (int l = 0; l < n_layers; l++) {
     NezavikLayer &w = layers[l];
     const int ld_in = w.in.n_out, ld_act = w.out.n_in;
-    GPTOSS_STEP(gemm(w.in, t_rows, t_rows_f32, in_rows, n));
-    if (w.ff) GPTOSS_STEP(run_column_map(in_rows, ld_in, w.up_col, w.ff, true, act_rows, ld_act, 0, f32, n, s));
+    GPTOSS_STEP(project_in(w, n));
     if (w.type == NezavikLayer::PARALLEL) {
       WindowAttn a = w.attn;
       a.in = in_rows;
@@ -109,7 +128,6 @@ int Nezavik::forward_rows(const StepRows &r) {
       GPTOSS_STEP(run_window_attn(a, r, s));
     }
     if (w.type == NezavikLayer::CHANNEL_DELTA) {
-      GPTOSS_STEP(run_column_map(in_rows, ld_in, w.low_col, w.low_width, false, low_rows, w.low_rank.n_in, 0, f32, n, s));
       GPTOSS_STEP(gemm(w.low_rank, (const bf16_t *)low_rows, (const float *)low_rows, low_out_rows, n));
     }
     GPTOSS_STEP(run_short_conv(w.conv, r, in_rows, ld_in, w.scan.conv_state, conv_rows, w.conv.channels, s));
@@ -133,9 +151,13 @@ int Nezavik::forward_rows(const StepRows &r) {
     g.ld_out = ld_act;
     g.out_f32 = f32;
     GPTOSS_STEP(run_gated_norm(g, n, s));
-    GPTOSS_STEP(gemm(w.out, (const bf16_t *)act_rows, (const float *)act_rows, branch, n));
+    int parts = 1;
+    if (f32) GPTOSS_STEP(gemm(w.out, nullptr, (const float *)act_rows, branch, n));
+    else
+      GPTOSS_STEP(dense_gemm_partial((const bf16_t *)act_rows, w.out.packed, branch, branch_elems, &parts, n, w.out.n_out,
+                                     w.out.n_in, s));
     const float *next_norm = l + 1 < n_layers ? layers[l + 1].norm : nullptr;   // the sampled rows are normed later
-    GPTOSS_STEP(run_depth_average_norm(rows_x, branch, history, plane, w.average, l, next_norm, t_rows, t_rows_f32, n,
+    GPTOSS_STEP(run_depth_average_norm(rows_x, branch, parts, history, plane, w.average, l, next_norm, t_rows, t_rows_f32, n,
                                        hidden, norm_eps, hidden_real, s));
   }
   return GPTOSS_OK;
@@ -574,7 +596,9 @@ int open_nezavik(const ModelSource &src, const OpenOptions &o, gptoss_engine **o
     e->y_rows = b.alloc<float>((size_t)R * e->wide.y);
     e->low_out_rows = b.alloc<float>((size_t)R * e->wide.low_out);
     e->q_rows = b.alloc<float>((size_t)R * e->wide.q);
-    e->branch = b.alloc<float>((size_t)R * e->hidden);
+    // room for every part of the output projection's sum while the rows are few
+    e->branch_elems = std::max((size_t)R * e->hidden, std::min<size_t>((size_t)R * e->hidden * GEMM_MAX_PARTS, (size_t)32 << 20));
+    e->branch = b.alloc<float>(e->branch_elems);
     e->history = b.alloc<float>((size_t)R * e->hidden * (e->n_layers + 1));
     e->t_rows = b.alloc<bf16_t>((size_t)R * e->hidden);
     if (e->precise()) e->t_rows_f32 = b.alloc<float>((size_t)R * e->hidden);

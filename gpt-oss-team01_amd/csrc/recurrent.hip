@@ -45,42 +45,91 @@ __device__ __forceinline__ float conv_input(const ShortConv &c, const float *in,
   return state[((size_t)slot * (c.taps - 1) + (c.taps - 1 + off - j)) * c.channels + ch];
 }
 
-// One wave per (row, head): heads of unit_dim channels that become unit vectors first, then the
-// remaining channels in pieces of 64.
+// One wave per (rows, head): heads of unit_dim channels that become unit vectors first, then the remaining
+// channels in pieces of 64.  A wave takes RT consecutive rows, whose inputs it requests together and
+// slides the taps over (TAPS 0: any number of taps, inputs read tap by tap).
+template <int TAPS, int RT>
 __global__ __launch_bounds__(256) void short_conv_kernel(ShortConv c, const int *__restrict__ slots,
                                                          const int *__restrict__ lens,
                                                          const int *__restrict__ offset,
                                                          const float *__restrict__ in, int ld_in,
                                                          const float *__restrict__ state, float *__restrict__ out,
-                                                         int ld_out, int units) {
-  const int row = blockIdx.y, lane = threadIdx.x & 63;
+                                                         int ld_out, int units, int n) {
+  constexpr int PIECES = SCAN_MAX_KEY / 64;
+  const int row0 = blockIdx.y * RT, lane = threadIdx.x & 63;
   const int unit = blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   if (unit >= units) return;
-  const int off = offset[row], pos = lens[row] - 1, slot = slots[row];
   const bool norm = unit < 2 * c.n_unit;
   const int unit_ch = 2 * c.n_unit * c.unit_dim;
   const int ch0 = norm ? unit * c.unit_dim : unit_ch + (unit - 2 * c.n_unit) * 64;
   const int width = norm ? c.unit_dim : min(64, c.channels - ch0);
-  float v[SCAN_MAX_KEY / 64], ss = 0.f;
+  const int live = min(RT, n - row0);
+  int off[RT], pos[RT], slot[RT];
 #pragma unroll
-  for (int i = 0; i < SCAN_MAX_KEY / 64; i++) {
-    v[i] = 0.f;
-    const int d = lane + 64 * i;
-    if (d < width) {
-      const int ch = ch0 + d;
-      float a = c.bias ? c.bias[ch] : 0.f;
-      for (int j = c.taps - 1; j >= 0; j--)
-        a += c.weight[(size_t)ch * c.taps + (c.taps - 1 - j)] * conv_input(c, in, ld_in, state, row, off, pos, slot, ch, j);
-      v[i] = silu_f(a);
-      ss += v[i] * v[i];
+  for (int r = 0; r < RT; r++) {
+    const int row = row0 + min(r, live - 1);
+    off[r] = offset[row];
+    pos[r] = lens[row] - 1;
+    slot[r] = slots[row];
+  }
+  float v[PIECES][RT], ss[RT];
+#pragma unroll
+  for (int r = 0; r < RT; r++) ss[r] = 0.f;
+#pragma unroll
+  for (int i = 0; i < PIECES; i++) {
+    if (64 * i >= width) break;
+    const int d = lane + 64 * i, ch = ch0 + min(d, width - 1);
+    const float bias = c.bias ? c.bias[ch] : 0.f;
+    if constexpr (TAPS > 0) {
+      float w[TAPS], x[RT], past[TAPS];   // past[j]: the input j + 1 tokens back
+#pragma unroll
+      for (int j = 0; j < TAPS; j++) w[j] = c.weight[(size_t)ch * TAPS + (TAPS - 1 - j)];
+#pragma unroll
+      for (int r = 0; r < RT; r++) x[r] = in[(size_t)(row0 + min(r, live - 1)) * ld_in + c.col + ch];
+#pragma unroll
+      for (int r = 0; r < RT; r++) {
+        if (r == 0 || off[r] == 0) {   // wave-uniform: the first row here, or of its sequence in this step
+#pragma unroll
+          for (int j = 0; j + 1 < TAPS; j++)
+            past[j] = conv_input(c, in, ld_in, state, row0 + min(r, live - 1), off[r], pos[r], slot[r], ch, j + 1);
+        }
+        float a = bias;
+#pragma unroll
+        for (int j = TAPS - 1; j >= 1; j--) a = fmaf(w[j], past[j - 1], a);
+        a = fmaf(w[0], x[r], a);
+#pragma unroll
+        for (int j = TAPS - 2; j >= 1; j--) past[j] = past[j - 1];
+        if (TAPS > 1) past[0] = x[r];
+        v[i][r] = d < width ? silu_f(a) : 0.f;
+        ss[r] = fmaf(v[i][r], v[i][r], ss[r]);
+      }
+    } else {
+#pragma unroll
+      for (int r = 0; r < RT; r++) {
+        float a = bias;
+        for (int j = c.taps - 1; j >= 0; j--)
+          a = fmaf(c.weight[(size_t)ch * c.taps + (c.taps - 1 - j)],
+                   conv_input(c, in, ld_in, state, row0 + min(r, live - 1), off[r], pos[r], slot[r], ch, j), a);
+        v[i][r] = d < width ? silu_f(a) : 0.f;
+        ss[r] = fmaf(v[i][r], v[i][r], ss[r]);
+      }
     }
   }
-  float scale = 1.f;
-  if (norm) scale = (unit < c.n_unit ? c.unit_scale : 1.f) / sqrtf(wave_sum_f(ss) + 1e-6f);
+  float scale[RT];
 #pragma unroll
-  for (int i = 0; i < SCAN_MAX_KEY / 64; i++) {
+  for (int r = 0; r < RT; r++) scale[r] = 1.f;
+  if (norm) {
+#pragma unroll
+    for (int r = 0; r < RT; r++)
+      scale[r] = (unit < c.n_unit ? c.unit_scale : 1.f) / sqrtf(wave_sum_f(ss[r]) + 1e-6f);
+  }
+#pragma unroll
+  for (int i = 0; i < PIECES; i++) {
+    if (64 * i >= width) break;
     const int d = lane + 64 * i;
-    if (d < width) out[(size_t)row * ld_out + ch0 + d] = v[i] * scale;
+#pragma unroll
+    for (int r = 0; r < RT; r++)
+      if (r < live && d < width) out[(size_t)(row0 + r) * ld_out + ch0 + d] = v[i][r] * scale[r];
   }
 }
 
@@ -104,21 +153,33 @@ __device__ __forceinline__ void advance_conv_state(const Scan &p, const RowSeg &
   }
 }
 
-template <int NI, int KIND>
+// What a lane needs of one token.
+template <int NI, bool CHANNEL>
+struct ScanToken {
+  f32x4 k[NI], q[NI], g[CHANNEL ? NI : 1];
+  float v[2], decay, beta;
+};
+
+// ONE: every sequence has one row (decoding); the launch is then a stream of states through the chip.
+template <int NI, int KIND, bool ONE>
 __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restrict__ segs) {
-  constexpr int KP = 32 * NI, TC = SCAN_TOKENS;
+  constexpr int KP = 32 * NI, TC = ONE ? 1 : SCAN_TOKENS;
   constexpr bool CHANNEL = KIND == SCAN_CHANNEL_DELTA, SSM = KIND == SCAN_STATE_SPACE;
-  __shared__ __attribute__((aligned(16))) float sk[TC][KP], sq[TC][KP], sg[CHANNEL ? TC : 1][KP];
-  __shared__ float sv[TC][SCAN_COLS], s_decay[TC], s_beta[TC];
+  constexpr int PIECES = (TC * KP + 255) / 256, VPIECES = (TC * SCAN_COLS + 255) / 256;
+  // one token more than is staged: the loop reads a token ahead
+  __shared__ __attribute__((aligned(16))) float sk[TC + 1][KP], sq[TC + 1][KP], sg[CHANNEL ? TC + 1 : 1][KP];
+  __shared__ __attribute__((aligned(8))) float sv[TC + 1][SCAN_COLS];
+  __shared__ float s_decay[TC + 1], s_beta[TC + 1];
   const RowSeg seg = segs[blockIdx.x];
   const int h = blockIdx.y;
   if (h == p.heads) {
     advance_conv_state(p, seg);
     return;
   }
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int j = lane & 7;
   const int c0 = blockIdx.z * SCAN_COLS, cw = wave * 16 + (lane >> 3) * 2;   // this lane's columns c0 + cw, + 1
+  const bool busy = c0 + wave * 16 < p.V;                                    // wave-uniform
   const int kh = h / (p.heads / p.key_heads);
   const float rate = expf(p.a_log[h]);
   const float bias = CHANNEL ? 0.f : p.dt_bias[h];
@@ -131,103 +192,129 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
 #pragma unroll
     for (int i = 0; i < NI; i++) {
       S[c][i] = f32x4{0.f, 0.f, 0.f, 0.f};
-      if (seg.pos0 > 0 && c0 + cw + c < p.V) S[c][i] = *reinterpret_cast<const f32x4 *>(st + c * KP + 32 * i);
+      if (seg.pos0 > 0 && c0 + cw + c < p.V)
+        S[c][i] = __builtin_nontemporal_load(reinterpret_cast<const f32x4 *>(st + c * KP + 32 * i));
     }
 
-  for (int t0 = 0; t0 < seg.n; t0 += TC) {
+  // the next tokens' inputs travel through registers while the current ones are worked on
+  float rk[PIECES], rq[PIECES], rg[CHANNEL ? PIECES : 1], rv[VPIECES], r_beta = 0.f, r_decay = 0.f;
+  auto fetch = [&](int t0) {
     const int T = min(TC, seg.n - t0);
-    if (t0 > 0) __syncthreads();
-    for (int idx = tid; idx < T * KP; idx += 256) {
-      const int t = idx / KP, d = idx - t * KP;
-      const size_t row = seg.row0 + t0 + t;
-      float k = 0.f, q = 0.f, g = 0.f;
-      if (d < p.K) {
+#pragma unroll
+    for (int x = 0; x < PIECES; x++) {
+      const int idx = tid + 256 * x, t = idx / KP, d = idx - t * KP;
+      rk[x] = rq[x] = 0.f;
+      if (CHANNEL) rg[x] = 0.f;
+      if (t < T && d < p.K) {
+        const size_t row = seg.row0 + t0 + t;
         const float *cr = p.conv + row * p.ld_conv + kh * p.K + d;
-        k = cr[p.k_col];
-        q = cr[p.q_col];
-        if (CHANNEL)
-          g = expf(-rate * softplus_f(p.channel_decay[row * p.ld_decay + h * p.K + d] + p.dt_bias[h * p.K + d]));
+        rk[x] = cr[p.k_col];
+        rq[x] = cr[p.q_col];
+        if (CHANNEL) rg[x] = p.channel_decay[row * p.ld_decay + h * p.K + d];
       }
-      sk[t][d] = k;
-      sq[t][d] = q;
-      if (CHANNEL) sg[t][d] = g;
     }
-    for (int idx = tid; idx < T * SCAN_COLS; idx += 256) {
-      const int t = idx / SCAN_COLS, c = idx - t * SCAN_COLS;
-      sv[t][c] = c0 + c < p.V ? p.conv[(size_t)(seg.row0 + t0 + t) * p.ld_conv + p.v_col + h * p.V + c0 + c] : 0.f;
+#pragma unroll
+    for (int x = 0; x < VPIECES; x++) {
+      const int idx = tid + 256 * x, t = idx / SCAN_COLS, c = idx - t * SCAN_COLS;
+      rv[x] = t < T && c0 + c < p.V ? p.conv[(size_t)(seg.row0 + t0 + t) * p.ld_conv + p.v_col + h * p.V + c0 + c] : 0.f;
     }
     if (tid < T) {
       const float *ir = p.in + (size_t)(seg.row0 + t0 + tid) * p.ld_in;
+      if (!SSM) r_beta = ir[p.beta_col + h];
+      if (!CHANNEL) r_decay = ir[p.decay_col + h];
+    }
+  };
+  auto put = [&](int t0) {
+    const int T = min(TC, seg.n - t0);
+#pragma unroll
+    for (int x = 0; x < PIECES; x++) {
+      const int idx = tid + 256 * x, t = idx / KP, d = idx - t * KP;
+      if (t < T) {
+        sk[t][d] = rk[x];
+        sq[t][d] = rq[x];
+        if (CHANNEL) sg[t][d] = d < p.K ? expf(-rate * softplus_f(rg[x] + p.dt_bias[h * p.K + d])) : 0.f;
+      }
+    }
+#pragma unroll
+    for (int x = 0; x < VPIECES; x++) {
+      const int idx = tid + 256 * x;
+      if (idx < TC * SCAN_COLS) (&sv[0][0])[idx] = rv[x];
+    }
+    if (tid < T) {
       if (SSM) {
-        const float dt = softplus_f(ir[p.decay_col + h] + bias);
+        const float dt = softplus_f(r_decay + bias);
         s_decay[tid] = expf(-rate * dt);
         s_beta[tid] = dt;
       } else {
-        s_beta[tid] = sigmoid_f(ir[p.beta_col + h]);
-        if (!CHANNEL) s_decay[tid] = expf(-rate * softplus_f(ir[p.decay_col + h] + bias));
+        s_beta[tid] = sigmoid_f(r_beta);
+        if (!CHANNEL) s_decay[tid] = expf(-rate * softplus_f(r_decay + bias));
       }
     }
-    __syncthreads();
-    float keep[2] = {0.f, 0.f};
-    for (int t = 0; t < T; t++) {
-      f32x4 k[NI], q[NI];
+  };
+  using Token = ScanToken<NI, CHANNEL>;
+  auto read = [&](Token &x, int t) {
 #pragma unroll
-      for (int i = 0; i < NI; i++) {
-        k[i] = *reinterpret_cast<const f32x4 *>(&sk[t][32 * i + 4 * j]);
-        q[i] = *reinterpret_cast<const f32x4 *>(&sq[t][32 * i + 4 * j]);
-      }
-      const float beta = s_beta[t];
-      float v[2] = {sv[t][cw], sv[t][cw + 1]}, u[2], o[2];
-      if constexpr (CHANNEL) {
+    for (int i = 0; i < NI; i++) {
+      x.k[i] = *reinterpret_cast<const f32x4 *>(&sk[t][32 * i + 4 * j]);
+      x.q[i] = *reinterpret_cast<const f32x4 *>(&sq[t][32 * i + 4 * j]);
+      if (CHANNEL) x.g[i] = *reinterpret_cast<const f32x4 *>(&sg[t][32 * i + 4 * j]);
+    }
+    x.v[0] = sv[t][cw];
+    x.v[1] = sv[t][cw + 1];
+    x.beta = s_beta[t];
+    if (!CHANNEL) x.decay = s_decay[t];
+  };
+  auto advance = [&](const Token &x, float (&o)[2]) {
 #pragma unroll
-        for (int i = 0; i < NI; i++) {
-          const f32x4 g = *reinterpret_cast<const f32x4 *>(&sg[t][32 * i + 4 * j]);
+    for (int c = 0; c < 2; c++)
 #pragma unroll
-          for (int c = 0; c < 2; c++)
+      for (int i = 0; i < NI; i++)
 #pragma unroll
-            for (int e = 0; e < 4; e++) S[c][i][e] *= g[e];
-        }
+        for (int e = 0; e < 4; e++) S[c][i][e] *= CHANNEL ? x.g[CHANNEL ? i : 0][e] : x.decay;
+    float u[2];
+#pragma unroll
+    for (int c = 0; c < 2; c++) {
+      if constexpr (SSM) {
+        u[c] = x.beta * x.v[c];
       } else {
-        const float g = s_decay[t];
-#pragma unroll
-        for (int c = 0; c < 2; c++)
-#pragma unroll
-          for (int i = 0; i < NI; i++)
-#pragma unroll
-            for (int e = 0; e < 4; e++) S[c][i][e] *= g;
-      }
-#pragma unroll
-      for (int c = 0; c < 2; c++) {
-        if constexpr (SSM) {
-          u[c] = beta * v[c];
-        } else {
-          float d0 = 0.f, d1 = 0.f;
-#pragma unroll
-          for (int i = 0; i < NI; i++) {
-            d0 = fmaf(S[c][i][0], k[i][0], d0);
-            d1 = fmaf(S[c][i][1], k[i][1], d1);
-            d0 = fmaf(S[c][i][2], k[i][2], d0);
-            d1 = fmaf(S[c][i][3], k[i][3], d1);
-          }
-          u[c] = beta * (v[c] - sum8(d0 + d1));
-        }
-      }
-#pragma unroll
-      for (int c = 0; c < 2; c++) {
         float d0 = 0.f, d1 = 0.f;
 #pragma unroll
         for (int i = 0; i < NI; i++) {
-#pragma unroll
-          for (int e = 0; e < 4; e++) S[c][i][e] = fmaf(k[i][e], u[c], S[c][i][e]);
-          d0 = fmaf(S[c][i][0], q[i][0], d0);
-          d1 = fmaf(S[c][i][1], q[i][1], d1);
-          d0 = fmaf(S[c][i][2], q[i][2], d0);
-          d1 = fmaf(S[c][i][3], q[i][3], d1);
+          d0 = fmaf(S[c][i][0], x.k[i][0], d0);
+          d1 = fmaf(S[c][i][1], x.k[i][1], d1);
+          d0 = fmaf(S[c][i][2], x.k[i][2], d0);
+          d1 = fmaf(S[c][i][3], x.k[i][3], d1);
         }
-        o[c] = sum8(d0 + d1);
-        if (SSM) o[c] = fmaf(skip, v[c], o[c]);
+        u[c] = x.beta * (x.v[c] - sum8(d0 + d1));
       }
-      // lane j of a group keeps the results of tokens t with t % 8 == j and stores them together
+    }
+#pragma unroll
+    for (int c = 0; c < 2; c++) {
+      float d0 = 0.f, d1 = 0.f;
+#pragma unroll
+      for (int i = 0; i < NI; i++) {
+#pragma unroll
+        for (int e = 0; e < 4; e++) S[c][i][e] = fmaf(x.k[i][e], u[c], S[c][i][e]);
+        d0 = fmaf(S[c][i][0], x.q[i][0], d0);
+        d1 = fmaf(S[c][i][1], x.q[i][1], d1);
+        d0 = fmaf(S[c][i][2], x.q[i][2], d0);
+        d1 = fmaf(S[c][i][3], x.q[i][3], d1);
+      }
+      o[c] = sum8(d0 + d1);
+      if (SSM) o[c] = fmaf(skip, x.v[c], o[c]);
+    }
+  };
+  fetch(0);
+  for (int t0 = 0; t0 < seg.n; t0 += TC) {
+    const int T = min(TC, seg.n - t0);
+    if (t0 > 0) __syncthreads();
+    put(t0);
+    __syncthreads();
+    if (!ONE && t0 + TC < seg.n) fetch(t0 + TC);
+    if (!busy) continue;
+    float keep[2] = {0.f, 0.f};
+    // lane j of a group keeps the results of tokens t with t % 8 == j and stores them together
+    auto emit = [&](int t, const float (&o)[2]) {
       if ((t & 7) == j) {
         keep[0] = o[0];
         keep[1] = o[1];
@@ -240,17 +327,49 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
           if (c0 + cw + 1 < p.V) dst[1] = keep[1];
         }
       }
+    };
+    Token a;
+    read(a, 0);
+    if constexpr (ONE) {
+      float o[2];
+      advance(a, o);
+      emit(0, o);
+    } else if constexpr (NI <= 4) {
+      // two tokens in registers: the next one's inputs are requested before the current one is worked on
+      Token b;
+      for (int t = 0; t < T; t += 2) {
+        float o[2];
+        read(b, t + 1);
+        advance(a, o);
+        emit(t, o);
+        if (t + 1 >= T) break;
+        read(a, t + 2);
+        advance(b, o);
+        emit(t + 1, o);
+      }
+    } else {
+      for (int t = 0; t < T; t++) {
+        float o[2];
+        advance(a, o);
+        emit(t, o);
+        if (t + 1 < T) read(a, t + 1);
+      }
     }
   }
 #pragma unroll
   for (int c = 0; c < 2; c++)
 #pragma unroll
     for (int i = 0; i < NI; i++)
-      if (c0 + cw + c < p.V) *reinterpret_cast<f32x4 *>(st + c * KP + 32 * i) = S[c][i];
+      if (c0 + cw + c < p.V)
+        __builtin_nontemporal_store(S[c][i], reinterpret_cast<f32x4 *>(st + c * KP + 32 * i));
 }
 
 // ---- gated output norm ---------------------------------------------------------------------------
-// One wave per (row, group).
+__device__ __forceinline__ float gated_value(const GatedNorm &g, float y, float gate) {
+  return g.gate_first ? y * silu_f(gate) : y;
+}
+
+// One wave per (row, group), any size and alignment.
 template <typename OUT>
 __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNorm g) {
   const int row = blockIdx.y, lane = threadIdx.x & 63;
@@ -261,14 +380,13 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNorm g) {
   const float *w = g.weight + (g.weight_per_group ? group * g.size : 0);
   float ss = 0.f;
   for (int d = lane; d < g.size; d += 64) {
-    const float v = g.gate_first ? y[d] * silu_f(gate[d]) : y[d];
+    const float v = gated_value(g, y[d], gate[d]);
     ss += v * v;
   }
   const float inv = 1.f / sqrtf(wave_sum_f(ss) / g.size + g.eps);
   OUT *out = (OUT *)g.out + (size_t)row * g.ld_out + g.out_col + group * g.size;
   for (int d = lane; d < g.size; d += 64) {
-    float v = g.gate_first ? y[d] * silu_f(gate[d]) : y[d];
-    v = v * inv * w[d];
+    float v = gated_value(g, y[d], gate[d]) * inv * w[d];
     if (!g.gate_first) v *= g.sigmoid_gate ? sigmoid_f(gate[d]) : silu_f(gate[d]);
     v *= g.scale;
     if constexpr (sizeof(OUT) == 2) out[d] = f32_to_bf16(v);
@@ -276,10 +394,60 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNorm g) {
   }
 }
 
-template <typename OUT>
+// Groups of at most 4 * LANES * VPT values whose rows are 16-byte aligned: LANES lanes hold a group in
+// registers, a wave 64 / LANES groups.
+template <typename OUT, int LANES, int VPT>
+__global__ __launch_bounds__(256) void gated_norm_vec_kernel(GatedNorm g) {
+  const int row = blockIdx.y, l = threadIdx.x % LANES;
+  const int group = blockIdx.x * (256 / LANES) + threadIdx.x / LANES;
+  const bool live = group < g.groups;
+  const int at = (live ? group : 0) * g.size;
+  const float *y = g.y + (size_t)row * g.ld_y + at, *gate = g.gate + (size_t)row * g.ld_gate + at;
+  const float *w = g.weight + (g.weight_per_group ? at : 0);
+  f32x4 v[VPT], z[VPT];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < VPT; i++) {
+    const int d = (l + LANES * i) * 4;
+    v[i] = z[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (d < g.size) {
+      v[i] = *reinterpret_cast<const f32x4 *>(y + d);
+      z[i] = *reinterpret_cast<const f32x4 *>(gate + d);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < VPT; i++)
+#pragma unroll
+    for (int e = 0; e < 4; e++) {
+      v[i][e] = gated_value(g, v[i][e], z[i][e]);
+      ss = fmaf(v[i][e], v[i][e], ss);
+    }
+#pragma unroll
+  for (int m = LANES / 2; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, 64);
+  const float inv = 1.f / sqrtf(ss / g.size + g.eps);
+  if (!live) return;
+  OUT *out = (OUT *)g.out + (size_t)row * g.ld_out + g.out_col + at;
+#pragma unroll
+  for (int i = 0; i < VPT; i++) {
+    const int d = (l + LANES * i) * 4;
+    if (d < g.size) {
+      const f32x4 wv = *reinterpret_cast<const f32x4 *>(w + d);
+      f32x4 o;
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        o[e] = v[i][e] * inv * wv[e];
+        if (!g.gate_first) o[e] *= g.sigmoid_gate ? sigmoid_f(z[i][e]) : silu_f(z[i][e]);
+        o[e] *= g.scale;
+      }
+      if constexpr (sizeof(OUT) == 2)
+        *reinterpret_cast<u32x2 *>(out + d) = u32x2{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
+      else *reinterpret_cast<f32x4 *>(out + d) = o;
+    }
+  }
+}
+
 __global__ __launch_bounds__(256) void column_map_kernel(const float *__restrict__ in, int ld_in, int col, int width,
-                                                         int relu_squared, OUT *__restrict__ out, int ld_out,
-                                                         int out_col) {
+                                                         int relu_squared, float *__restrict__ out, int ld_out) {
   const int d = blockIdx.x * 256 + threadIdx.x;
   const size_t row = blockIdx.y;
   if (d >= width) return;
@@ -288,8 +456,7 @@ __global__ __launch_bounds__(256) void column_map_kernel(const float *__restrict
     v = fmaxf(v, 0.f);
     v *= v;
   }
-  if constexpr (sizeof(OUT) == 2) out[row * ld_out + out_col + d] = f32_to_bf16(v);
-  else out[row * ld_out + out_col + d] = v;
+  out[row * ld_out + d] = v;
 }
 
 // ---- launches ------------------------------------------------------------------------------------
@@ -300,18 +467,31 @@ int run_short_conv(const ShortConv &c, const StepRows &r, const float *in, int l
   const int plain = c.channels - 2 * c.n_unit * c.unit_dim;
   const int units = 2 * c.n_unit + cdiv(plain, 64);
   TraceScope ts("short_conv", s);
-  short_conv_kernel<<<dim3(cdiv(units, 4), r.n), 256, 0, s>>>(c, r.slots, r.lens, r.offset, in, ld_in, state, out,
-                                                              ld_out, units);
+  auto go = [&](auto kern, int rt) {
+    kern<<<dim3(cdiv(units, 4), cdiv(r.n, rt)), 256, 0, s>>>(c, r.slots, r.lens, r.offset, in, ld_in, state, out, ld_out,
+                                                             units, r.n);
+  };
+  const bool many = r.longest > 1 && r.n >= 256;
+  if (c.taps == 4) many ? go(short_conv_kernel<4, 8>, 8) : go(short_conv_kernel<4, 1>, 1);
+  else if (c.taps == 3) many ? go(short_conv_kernel<3, 8>, 8) : go(short_conv_kernel<3, 1>, 1);
+  else if (c.taps == 2) many ? go(short_conv_kernel<2, 8>, 8) : go(short_conv_kernel<2, 1>, 1);
+  else go(short_conv_kernel<0, 1>, 1);
   GPTOSS_LAUNCH_CHECK("short_conv_kernel");
   return GPTOSS_OK;
+}
+
+template <int NI, int KIND>
+static void launch_scan_kind(const Scan &p, const StepRows &r, dim3 grid, hipStream_t s) {
+  if (r.longest == 1) scan_kernel<NI, KIND, true><<<grid, 256, 0, s>>>(p, r.segs);
+  else scan_kernel<NI, KIND, false><<<grid, 256, 0, s>>>(p, r.segs);
 }
 
 template <int NI>
 static void launch_scan(const Scan &p, const StepRows &r, dim3 grid, hipStream_t s) {
   switch (p.kind) {
-    case SCAN_DELTA: scan_kernel<NI, SCAN_DELTA><<<grid, 256, 0, s>>>(p, r.segs); break;
-    case SCAN_CHANNEL_DELTA: scan_kernel<NI, SCAN_CHANNEL_DELTA><<<grid, 256, 0, s>>>(p, r.segs); break;
-    case SCAN_STATE_SPACE: scan_kernel<NI, SCAN_STATE_SPACE><<<grid, 256, 0, s>>>(p, r.segs); break;
+    case SCAN_DELTA: launch_scan_kind<NI, SCAN_DELTA>(p, r, grid, s); break;
+    case SCAN_CHANNEL_DELTA: launch_scan_kind<NI, SCAN_CHANNEL_DELTA>(p, r, grid, s); break;
+    case SCAN_STATE_SPACE: launch_scan_kind<NI, SCAN_STATE_SPACE>(p, r, grid, s); break;
   }
 }
 
@@ -336,21 +516,30 @@ int run_scan(const Scan &p, const StepRows &r, hipStream_t s) {
   return GPTOSS_OK;
 }
 
+template <typename OUT>
+static void launch_gated_norm(const GatedNorm &g, int n, hipStream_t s) {
+  const bool vec = g.size % 4 == 0 && g.ld_y % 4 == 0 && g.ld_gate % 4 == 0 && g.ld_out % 4 == 0 && g.out_col % 4 == 0 &&
+                   aligned(g.y, 16) && aligned(g.gate, 16) && aligned(g.weight, 16) && aligned(g.out, 16);
+  if (vec && g.size <= 64) gated_norm_vec_kernel<OUT, 16, 1><<<dim3(cdiv(g.groups, 16), n), 256, 0, s>>>(g);
+  else if (vec && g.size <= 128) gated_norm_vec_kernel<OUT, 32, 1><<<dim3(cdiv(g.groups, 8), n), 256, 0, s>>>(g);
+  else if (vec && g.size <= 256) gated_norm_vec_kernel<OUT, 64, 1><<<dim3(cdiv(g.groups, 4), n), 256, 0, s>>>(g);
+  else if (vec && g.size <= 512) gated_norm_vec_kernel<OUT, 64, 2><<<dim3(cdiv(g.groups, 4), n), 256, 0, s>>>(g);
+  else if (vec && g.size <= 1024) gated_norm_vec_kernel<OUT, 64, 4><<<dim3(cdiv(g.groups, 4), n), 256, 0, s>>>(g);
+  else gated_norm_kernel<OUT><<<dim3(cdiv(g.groups, 4), n), 256, 0, s>>>(g);
+}
+
 int run_gated_norm(const GatedNorm &g, int n, hipStream_t s) {
   TraceScope ts("gated_norm", s);
-  const dim3 grid(cdiv(g.groups, 4), n);
-  if (g.out_f32) gated_norm_kernel<float><<<grid, 256, 0, s>>>(g);
-  else gated_norm_kernel<bf16_t><<<grid, 256, 0, s>>>(g);
+  if (g.out_f32) launch_gated_norm<float>(g, n, s);
+  else launch_gated_norm<bf16_t>(g, n, s);
   GPTOSS_LAUNCH_CHECK("gated_norm_kernel");
   return GPTOSS_OK;
 }
 
-int run_column_map(const float *in, int ld_in, int col, int width, bool relu_squared, void *out, int ld_out,
-                   int out_col, bool out_f32, int n, hipStream_t s) {
+int run_column_map(const float *in, int ld_in, int col, int width, bool relu_squared, float *out, int ld_out, int n,
+                   hipStream_t s) {
   TraceScope ts(relu_squared ? "relu_squared" : "column_copy", s);
-  const dim3 grid(cdiv(width, 256), n);
-  if (out_f32) column_map_kernel<float><<<grid, 256, 0, s>>>(in, ld_in, col, width, relu_squared, (float *)out, ld_out, out_col);
-  else column_map_kernel<bf16_t><<<grid, 256, 0, s>>>(in, ld_in, col, width, relu_squared, (bf16_t *)out, ld_out, out_col);
+  column_map_kernel<<<dim3(cdiv(width, 256), n), 256, 0, s>>>(in, ld_in, col, width, relu_squared, out, ld_out);
   GPTOSS_LAUNCH_CHECK("column_map_kernel");
   return GPTOSS_OK;
 }

@@ -64,8 +64,9 @@ struct GatedNorm {
 };
 int run_gated_norm(const GatedNorm &g, int n, hipStream_t s);
 
-// out[:, out_col + i] = f(in[:, col + i]), i < width; f: the square of relu, or the identity
-int run_column_map(const float *in, int ld_in, int col, int width, bool relu_squared, void *out, int ld_out,
-                   int out_col, bool out_f32, int n, hipStream_t s);
+// out[:, i] = f(in[:, col + i]), i < width; f: the square of relu, or the identity (what EPI_MIXED does in
+// the bf16 GEMM, for fp32 rows)
+int run_column_map(const float *in, int ld_in, int col, int width, bool relu_squared, float *out, int ld_out, int n,
+                   hipStream_t s);
 
 }  // namespace gptoss

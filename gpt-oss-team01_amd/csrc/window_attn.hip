@@ -16,65 +16,83 @@ namespace gptoss {
 constexpr float WNEG = -1.0e30f;
 
 // ---- norms and K/V store -------------------------------------------------------------------------
-// One wave per (row, head): query heads, key heads, value heads.
-template <bool F32>
+// One wave per (RT rows, head): query heads, key heads, value heads.
+template <bool F32, int RT>
 __global__ __launch_bounds__(256) void window_store_kernel(WindowAttn a, const int *__restrict__ slots,
-                                                           const int *__restrict__ lens) {
-  const int row = blockIdx.y, lane = threadIdx.x & 63;
+                                                           const int *__restrict__ lens, int n) {
+  constexpr int PIECES = WINDOW_ATTN_MAX_DIM / 64;
+  const int row0 = blockIdx.y * RT, lane = threadIdx.x & 63, live = min(RT, n - row0);
   const int unit = blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int H = a.heads, G = a.kv_heads;
   if (unit >= H + 2 * G) return;
-  const int DK = F32 ? a.dim : a.dim_pad();
+  const int DK = F32 ? a.dim : a.dim_pad(), DV = a.vdim_pad();
   const bool is_q = unit < H, is_v = unit >= H + G;
   const int head = is_q ? unit : is_v ? unit - H - G : unit - H;
-  const int width = is_v ? a.vdim : a.dim;
-  const float *src = a.in + (size_t)row * a.ld_in + (is_q ? a.q_col : is_v ? a.v_col : a.k_col) + head * width;
-  const int slot_seq = slots[row], cslot = (lens[row] - 1) % a.cap;
-  float v[WINDOW_ATTN_MAX_DIM / 64], ss = 0.f;
+  const int width = is_v ? a.vdim : a.dim, padded = F32 ? width : is_v ? DV : DK;
+  const float *src = a.in + (is_q ? a.q_col : is_v ? a.v_col : a.k_col) + head * width;
+  float v[PIECES][RT], ss[RT];
 #pragma unroll
-  for (int i = 0; i < WINDOW_ATTN_MAX_DIM / 64; i++) {
+  for (int r = 0; r < RT; r++) ss[r] = 0.f;
+#pragma unroll
+  for (int i = 0; i < PIECES; i++) {
+    if (64 * i >= padded) break;
     const int d = lane + 64 * i;
-    v[i] = d < width ? src[d] : 0.f;
-    ss += v[i] * v[i];
+#pragma unroll
+    for (int r = 0; r < RT; r++) v[i][r] = d < width ? src[(size_t)(row0 + min(r, live - 1)) * a.ld_in + d] : 0.f;
+#pragma unroll
+    for (int r = 0; r < RT; r++) ss[r] = fmaf(v[i][r], v[i][r], ss[r]);
   }
   if (!is_v) {
-#pragma unroll
-    for (int m = 32; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, 64);
-    const float inv = 1.f / sqrtf(ss / a.dim + a.eps);
     const float *w = is_q ? a.q_norm : a.k_norm;
+    float inv[RT];
 #pragma unroll
-    for (int i = 0; i < WINDOW_ATTN_MAX_DIM / 64; i++) {
+    for (int r = 0; r < RT; r++) {
+#pragma unroll
+      for (int m = 32; m >= 1; m >>= 1) ss[r] += __shfl_xor(ss[r], m, 64);
+      inv[r] = 1.f / sqrtf(ss[r] / a.dim + a.eps);
+    }
+#pragma unroll
+    for (int i = 0; i < PIECES; i++) {
+      if (64 * i >= padded) break;
       const int d = lane + 64 * i;
-      if (d < width) v[i] = v[i] * inv * w[d];
+      const float wd = d < width ? w[d] : 0.f;
+#pragma unroll
+      for (int r = 0; r < RT; r++) v[i][r] = v[i][r] * inv[r] * wd;
     }
   }
-  if (is_q) {
-    float *dst = a.q + ((size_t)row * H + head) * DK;
 #pragma unroll
-    for (int i = 0; i < WINDOW_ATTN_MAX_DIM / 64; i++)
-      if (lane + 64 * i < DK) dst[lane + 64 * i] = v[i];
-    return;
-  }
-  if constexpr (F32) {
-    float *dst = (is_v ? a.v32 : a.k32) + (((size_t)slot_seq * a.cap + cslot) * G + head) * width;
+  for (int r = 0; r < RT; r++) {
+    if (r >= live) break;
+    const int row = row0 + r;
+    if (is_q) {
+      float *dst = a.q + ((size_t)row * H + head) * DK;
 #pragma unroll
-    for (int i = 0; i < WINDOW_ATTN_MAX_DIM / 64; i++)
-      if (lane + 64 * i < width) dst[lane + 64 * i] = v[i];
-  } else {
-    bf16_t *blk = a.kv + ((size_t)(slot_seq * G + head) * (a.cap >> 6) + (cslot >> 6)) * a.block_elems();
+      for (int i = 0; i < PIECES; i++)
+        if (lane + 64 * i < DK) dst[lane + 64 * i] = v[i][r];
+      continue;
+    }
+    const int seq = slots[row], cslot = (lens[row] - 1) % a.cap;
+    if constexpr (F32) {
+      float *dst = (is_v ? a.v32 : a.k32) + (((size_t)seq * a.cap + cslot) * G + head) * width;
 #pragma unroll
-    for (int i = 0; i < WINDOW_ATTN_MAX_DIM / 64; i++) {
-      const int d = lane + 64 * i;
-      if (is_v) {
-        // operand order of V^T behind the block's 64 key rows (kv_v_elem, value rows of vdim_pad)
-        if (d < a.vdim_pad()) {
-          const int tt = cslot & 31, within = tt & 15;
-          const int e = (((cslot & 63) >> 5) * (a.vdim_pad() >> 4) + (d >> 4)) * 512 +
-                        ((within >> 2) * 16 + (d & 15)) * 8 + (tt >> 4) * 4 + (within & 3);
-          blk[KV_BLOCK * DK + e] = f32_to_bf16(v[i]);
+      for (int i = 0; i < PIECES; i++)
+        if (lane + 64 * i < width) dst[lane + 64 * i] = v[i][r];
+    } else {
+      bf16_t *blk = a.kv + ((size_t)(seq * G + head) * (a.cap >> 6) + (cslot >> 6)) * a.block_elems();
+#pragma unroll
+      for (int i = 0; i < PIECES; i++) {
+        const int d = lane + 64 * i;
+        if (is_v) {
+          // operand order of V^T behind the block's 64 key rows (kv_v_elem, value rows of vdim_pad)
+          if (d < DV) {
+            const int tt = cslot & 31, within = tt & 15;
+            const int e = (((cslot & 63) >> 5) * (DV >> 4) + (d >> 4)) * 512 + ((within >> 2) * 16 + (d & 15)) * 8 +
+                          (tt >> 4) * 4 + (within & 3);
+            blk[KV_BLOCK * DK + e] = f32_to_bf16(v[i][r]);
+          }
+        } else if (d < DK) {
+          blk[(cslot & 63) * DK + d] = f32_to_bf16(v[i][r]);
         }
-      } else if (d < DK) {
-        blk[(cslot & 63) * DK + d] = f32_to_bf16(v[i]);
       }
     }
   }
@@ -119,13 +137,11 @@ __device__ __forceinline__ void load_q(QFrag<KS> &f, const float *q, int ks_n, i
   }
 }
 
-// One 64-slot block for 16 query columns: scores, online softmax, output.  kf(tb, ks) and vf(kg, db)
-// return operands; key slot i of the block is position pos0 + i; the column sees positions lo..hi.
-template <int KS, int DB, typename KF, typename VF>
-__device__ __forceinline__ void attend_block(const QFrag<KS> &q, int ks_n, int db_n, int pos0, int lo, int hi, int c,
-                                             float &m, float &l, f32x4 (&o)[DB], KF &&kf, VF &&vf) {
-  f32x4 s[4];
-  float mx = WNEG;
+// One 64-slot block for 16 query columns, in two halves so that a caller can request the next block's K
+// between them.  kf(tb, ks) and vf(kg, db) return operands; key slot i of the block is position
+// pos0 + i; the column sees positions lo..hi.
+template <int KS, typename KF>
+__device__ __forceinline__ void block_scores(const QFrag<KS> &q, int ks_n, f32x4 (&s)[4], KF &&kf) {
 #pragma unroll
   for (int tb = 0; tb < 4; tb++) {
     s[tb] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -136,13 +152,21 @@ __device__ __forceinline__ void attend_block(const QFrag<KS> &q, int ks_n, int d
         s[tb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, q.lo[ks], s[tb], 0, 0, 0);
         s[tb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, q.hi[ks], s[tb], 0, 0, 0);
       }
+  }
+}
+
+template <int DB, typename VF>
+__device__ __forceinline__ void block_output(f32x4 (&s)[4], int db_n, int pos0, int lo, int hi, int c, float &m, float &l,
+                                             f32x4 (&o)[DB], VF &&vf) {
+  float mx = WNEG;
+#pragma unroll
+  for (int tb = 0; tb < 4; tb++)
 #pragma unroll
     for (int e = 0; e < 4; e++) {
       const int pos = pos0 + tb * 16 + c * 4 + e;
       s[tb][e] = (pos >= lo && pos <= hi) ? s[tb][e] : WNEG;
       mx = fmaxf(mx, s[tb][e]);
     }
-  }
   mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
   mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
   const float m_new = fmaxf(m, mx);
@@ -182,6 +206,14 @@ __device__ __forceinline__ void attend_block(const QFrag<KS> &q, int ks_n, int d
   }
 }
 
+template <int KS, int DB, typename KF, typename VF>
+__device__ __forceinline__ void attend_block(const QFrag<KS> &q, int ks_n, int db_n, int pos0, int lo, int hi, int c,
+                                             float &m, float &l, f32x4 (&o)[DB], KF &&kf, VF &&vf) {
+  f32x4 s[4];
+  block_scores<KS>(q, ks_n, s, kf);
+  block_output<DB>(s, db_n, pos0, lo, hi, c, m, l, o, vf);
+}
+
 // Row sums over the four lane groups of a column (each lane has summed its own key rows).
 __device__ __forceinline__ float column_sum(float l) {
   l += __shfl_xor(l, 16, 64);
@@ -209,7 +241,9 @@ __device__ __forceinline__ void store_column(bf16_t *dst, int vdim, int db_n, in
 }
 
 // ---- decoding rows -------------------------------------------------------------------------------
-template <int DMAX>
+// EXACT: both head sizes are DMAX, so every operand has its place in registers: a wave's K and V of the next
+// block are requested as soon as those of the current one have been used.
+template <int DMAX, bool EXACT>
 __global__ __launch_bounds__(256) void window_decode_kernel(WindowAttn a, const RowSeg *__restrict__ singles) {
   constexpr int KS = DMAX / 32, DB = DMAX / 16;
   __shared__ float so[3][DMAX][16], sm[3][16], sl[3][16];
@@ -217,26 +251,63 @@ __global__ __launch_bounds__(256) void window_decode_kernel(WindowAttn a, const 
   const int g = blockIdx.y, per = a.heads / a.kv_heads;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int n = lane & 15, c = lane >> 4;
-  const int ks_n = a.dim_pad() / 32, db_n = a.vdim_pad() / 16, DK = a.dim_pad();
+  const int ks_n = EXACT ? KS : a.dim_pad() / 32, db_n = EXACT ? DB : a.vdim_pad() / 16, DK = EXACT ? DMAX : a.dim_pad();
+  const size_t block = EXACT ? (size_t)KV_BLOCK * 2 * DMAX : a.block_elems();
   const int hh = blockIdx.z * 16 + n;             // head within the group
   const bool live = hh < per;
   const int head = g * per + min(hh, per - 1);
-  QFrag<KS> q;
-  load_q<KS>(q, a.q + ((size_t)seg.row0 * a.heads + head) * DK, ks_n, c, a.scale * 1.4426950408889634f);
   const int hi = seg.pos0, lo = max(0, hi - a.window + 1);
   float m = WNEG, l = 0.f;
   f32x4 o[DB];
 #pragma unroll
   for (int db = 0; db < DB; db++) o[db] = f32x4{0.f, 0.f, 0.f, 0.f};
-  const bf16_t *plane = a.kv + (size_t)(seg.slot * a.kv_heads + g) * (a.cap >> 6) * a.block_elems();
   const int ring = a.cap >> 6;
-  for (int b = (lo >> 6) + wave; b <= (hi >> 6); b += 4) {
-    const bf16_t *blk = plane + (size_t)(b % ring) * a.block_elems();
-    const bf16_t *kl = blk + n * DK + c * ks_n * 8, *vl = blk + KV_BLOCK * DK + lane * 8;
-    attend_block<KS, DB>(
-        q, ks_n, db_n, b << 6, lo, hi, c, m, l, o,
-        [&](int tb, int ks) { return as_bf16x8(__builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(kl + tb * 16 * DK + ks * 8))); },
-        [&](int kg, int db) { return as_bf16x8(__builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(vl + (kg * db_n + db) * 512))); });
+  const bf16_t *plane = a.kv + (size_t)(seg.slot * a.kv_heads + g) * ring * block;
+  const size_t k_lane = n * DK + c * ks_n * 8, v_lane = KV_BLOCK * DK + lane * 8;
+  const int b_last = hi >> 6;
+  int b = (lo >> 6) + wave, rb = b % ring;   // block and its place in the ring
+  auto fetch = [](const bf16_t *x) { return __builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(x)); };
+  if constexpr (EXACT) {
+    u32x4 kr[4][KS], vr[2][DB];
+    auto load_k = [&](int at) {
+      const bf16_t *x = plane + (size_t)at * block + k_lane;
+#pragma unroll
+      for (int tb = 0; tb < 4; tb++)
+#pragma unroll
+        for (int ks = 0; ks < KS; ks++) kr[tb][ks] = fetch(x + tb * 16 * DMAX + ks * 8);
+    };
+    auto load_v = [&](int at) {
+      const bf16_t *x = plane + (size_t)at * block + v_lane;
+#pragma unroll
+      for (int kg = 0; kg < 2; kg++)
+#pragma unroll
+        for (int db = 0; db < DB; db++) vr[kg][db] = fetch(x + (kg * DB + db) * 512);
+    };
+    if (b <= b_last) {
+      load_k(rb);
+      load_v(rb);
+    }
+    QFrag<KS> q;
+    load_q<KS>(q, a.q + ((size_t)seg.row0 * a.heads + head) * DK, ks_n, c, a.scale * 1.4426950408889634f);
+    while (b <= b_last) {
+      const int next = b + 4 <= b_last ? (rb + 4) % ring : rb;   // past the end: this block again, unused
+      f32x4 s[4];
+      block_scores<KS>(q, KS, s, [&](int tb, int ks) { return as_bf16x8(kr[tb][ks]); });
+      load_k(next);
+      block_output<DB>(s, DB, b << 6, lo, hi, c, m, l, o, [&](int kg, int db) { return as_bf16x8(vr[kg][db]); });
+      load_v(next);
+      b += 4;
+      rb = next;
+    }
+  } else {
+    QFrag<KS> q;
+    load_q<KS>(q, a.q + ((size_t)seg.row0 * a.heads + head) * DK, ks_n, c, a.scale * 1.4426950408889634f);
+    for (; b <= b_last; b += 4) {
+      const bf16_t *blk = plane + (size_t)(b % ring) * block;
+      attend_block<KS, DB>(q, ks_n, db_n, b << 6, lo, hi, c, m, l, o,
+                           [&](int tb, int ks) { return as_bf16x8(fetch(blk + k_lane + tb * 16 * DK + ks * 8)); },
+                           [&](int kg, int db) { return as_bf16x8(fetch(blk + v_lane + (kg * db_n + db) * 512)); });
+    }
   }
   l = column_sum(l);
   if (wave > 0) {
@@ -399,11 +470,11 @@ int run_window_attn(const WindowAttn &a, const StepRows &r, hipStream_t s) {
                  WINDOW_ATTN_MAX_DIM, a.dim, a.vdim, a.heads, a.kv_heads, a.window);
   GPTOSS_REQUIRE(r.max_len <= a.cap || a.window - 1 + r.longest <= a.cap, GPTOSS_ERR_DIM,
                  "window_attn: a ring of %d slots cannot hold a window of %d and %d rows", a.cap, a.window, r.longest);
-  const dim3 store(cdiv(a.heads + 2 * a.kv_heads, 4), r.n);
+  const int units = a.heads + 2 * a.kv_heads;
   if (a.k32) {
     {
       TraceScope ts("window_store", s);
-      window_store_kernel<true><<<store, 256, 0, s>>>(a, r.slots, r.lens);
+      window_store_kernel<true, 1><<<dim3(cdiv(units, 4), r.n), 256, 0, s>>>(a, r.slots, r.lens, r.n);
     }
     GPTOSS_LAUNCH_CHECK("window_store_kernel");
     TraceScope ts("window_attn_f32", s);
@@ -413,16 +484,22 @@ int run_window_attn(const WindowAttn &a, const StepRows &r, hipStream_t s) {
   }
   {
     TraceScope ts("window_store", s);
-    window_store_kernel<false><<<store, 256, 0, s>>>(a, r.slots, r.lens);
+    if (r.n >= 1024) window_store_kernel<false, 4><<<dim3(cdiv(units, 4), cdiv(r.n, 4)), 256, 0, s>>>(a, r.slots, r.lens, r.n);
+    else window_store_kernel<false, 1><<<dim3(cdiv(units, 4), r.n), 256, 0, s>>>(a, r.slots, r.lens, r.n);
   }
   GPTOSS_LAUNCH_CHECK("window_store_kernel");
   const int widest = std::max(a.dim, a.vdim);
   if (r.n_singles) {
     TraceScope ts("window_decode", s);
     const dim3 grid(r.n_singles, a.kv_heads, cdiv(a.heads / a.kv_heads, 16));
-    if (widest <= 64) window_decode_kernel<64><<<grid, 256, 0, s>>>(a, r.singles);
-    else if (widest <= 128) window_decode_kernel<128><<<grid, 256, 0, s>>>(a, r.singles);
-    else window_decode_kernel<256><<<grid, 256, 0, s>>>(a, r.singles);
+    const bool both = a.dim_pad() == a.vdim_pad();
+    if (widest <= 64)
+      both && a.dim_pad() == 64 ? window_decode_kernel<64, true><<<grid, 256, 0, s>>>(a, r.singles)
+                                : window_decode_kernel<64, false><<<grid, 256, 0, s>>>(a, r.singles);
+    else if (widest <= 128)
+      both && a.dim_pad() == 128 ? window_decode_kernel<128, true><<<grid, 256, 0, s>>>(a, r.singles)
+                                 : window_decode_kernel<128, false><<<grid, 256, 0, s>>>(a, r.singles);
+    else window_decode_kernel<256, false><<<grid, 256, 0, s>>>(a, r.singles);
     GPTOSS_LAUNCH_CHECK("window_decode_kernel");
   }
   const StepRows::Tiles &t = r.tiles[a.tiles];

@@ -311,6 +311,31 @@ def test_other_sizes(open_model, name, precise):
     check_model(e, 1, cfg, w, tok, precise, [70, 1, 2, 13, 1], factor)
 
 
+@BOTH
+def test_wide_rows_and_passes_of_thousands_of_rows(open_model, precise):
+    """Sizes at which the products cut their sum over K into parts (few rows, many inputs) and run on the
+    256-row tiles (2048 rows and more in a pass, several sequences)."""
+    cfg = nm.config([nm.channel_delta(heads=2, kv=1, dim=32, vdim=128, ff=1400),
+                     nm.parallel(heads=2, kv=1, dim=64, vdim=64, window=100, s_heads=1, groups=1, state=64, s_vdim=64,
+                                 norm_groups=1, ff=900)], vocab=96, width=320, max_positions=900)
+    w = nm.weights(cfg, 73, 40, 60)
+    lens = (800, 790, 810)
+    toks = [nm.tokens(cfg, n, n) for n in lens]
+    rounding = None if precise else nm.bf16
+    want = [nz.forward(cfg, w, t, rounding=rounding) for t in toks]
+    e = open_model(cfg, w, precise, max_batch=3)
+    tok, slot, pos = (np.concatenate(x) for x in zip(*[(t[:-5], [i] * (len(t) - 5), np.arange(len(t) - 5))
+                                                       for i, t in enumerate(toks)]))
+    got = np.split(e.step_logits(tok, slot, pos, np.arange(len(tok))), np.cumsum([n - 5 for n in lens])[:-1])
+    for i in range(3):
+        check(got[i], want[i][:-5], precise, 1.0 if precise else STAGED_TOL / TOL[False])
+    for k in range(5):      # decoding: three rows at a time
+        at = [n - 5 + k for n in lens]
+        lg = e.step_logits([t[p] for t, p in zip(toks, at)], [0, 1, 2], at, [0, 1, 2])
+        for i in range(3):
+            check(lg[i:i + 1], want[i][at[i]:at[i] + 1], precise, 1.0 if precise else STAGED_TOL / TOL[False])
+
+
 def test_fp32_checkpoints_load(open_model, tmp_path):
     cfg = nm.config([nm.delta()])
     w = nm.weights(cfg, 3)
