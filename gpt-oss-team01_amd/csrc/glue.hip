@@ -549,13 +549,30 @@ __global__ __launch_bounds__(256) void depth_average_norm_kernel(float *__restri
     const int h = (threadIdx.x + 256 * i) * 4;
     v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (h < H) {
+      // sums in order of their index, four loads in flight at a time
       f32x4 own = *reinterpret_cast<const f32x4 *>(y + row + h);
-      for (int j = 1; j < parts; j++) own += *reinterpret_cast<const f32x4 *>(y + j * part_stride + row + h);
-      own += *reinterpret_cast<const f32x4 *>(x + row + h);
+      const f32x4 before = *reinterpret_cast<const f32x4 *>(x + row + h);
+      int k = 1;
+      for (; k + 4 <= parts; k += 4) {
+        f32x4 part[4];
+#pragma unroll
+        for (int q = 0; q < 4; q++) part[q] = *reinterpret_cast<const f32x4 *>(y + (k + q) * part_stride + row + h);
+#pragma unroll
+        for (int q = 0; q < 4; q++) own += part[q];
+      }
+      for (; k < parts; k++) own += *reinterpret_cast<const f32x4 *>(y + k * part_stride + row + h);
+      own += before;
       *reinterpret_cast<f32x4 *>(history + (size_t)(layer + 1) * plane + row + h) = own;
       f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
-      for (int j = 0; j <= layer; j++)
-        a += weights[j] * *reinterpret_cast<const f32x4 *>(history + (size_t)j * plane + row + h);
+      int j = 0;
+      for (; j + 4 <= layer + 1; j += 4) {
+        f32x4 old[4];
+#pragma unroll
+        for (int q = 0; q < 4; q++) old[q] = *reinterpret_cast<const f32x4 *>(history + (size_t)(j + q) * plane + row + h);
+#pragma unroll
+        for (int q = 0; q < 4; q++) a += weights[j + q] * old[q];
+      }
+      for (; j <= layer; j++) a += weights[j] * *reinterpret_cast<const f32x4 *>(history + (size_t)j * plane + row + h);
       v[i] = a + weights[layer + 1] * own;
       *reinterpret_cast<f32x4 *>(x + row + h) = v[i];
 #pragma unroll

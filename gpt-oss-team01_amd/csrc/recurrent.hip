@@ -14,9 +14,18 @@
 
 namespace gptoss {
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
-__device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// On the hardware's exp2, log2 and reciprocal (about one unit in the last place each), which keeps these
+// within a few units: the argument of an exponential that matters is small.
+__device__ __forceinline__ float exp_f(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
+__device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.f + exp_f(-z)); }
+__device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }
+// max(z, 0) + log(1 + e), e = exp(-|z|).  With u = 1 + e rounded, log(u) e / (u - 1) is log(1 + e) to a few
+// units in the last place however small e is (W. Kahan's form of log1p).
+__device__ __forceinline__ float softplus_f(float z) {
+  const float e = exp_f(-fabsf(z)), u = 1.f + e, d = u - 1.f;
+  const float l = __builtin_amdgcn_logf(u) * 0.6931471805599453f * e * __builtin_amdgcn_rcpf(d);
+  return fmaxf(z, 0.f) + (d == 0.f ? e : l);
+}
 
 __device__ __forceinline__ float wave_sum_f(float v) {
 #pragma unroll
@@ -138,10 +147,10 @@ constexpr int SCAN_TOKENS = 16;   // tokens staged at a time
 constexpr int SCAN_COLS = 64;     // state columns of a workgroup: 4 waves x 8 lane groups x 2
 
 // The convolution's last taps - 1 inputs after the stretch; one thread owns a channel.
-__device__ __forceinline__ void advance_conv_state(const Scan &p, const RowSeg &seg) {
+__device__ __forceinline__ void advance_conv_state(const Scan &p, const RowSeg &seg, int part, int parts) {
   const ShortConv &c = p.conv_desc;
   const int keep = c.taps - 1;
-  for (int ch = blockIdx.z * 256 + threadIdx.x; ch < c.channels; ch += gridDim.z * 256) {
+  for (int ch = part * 256 + threadIdx.x; ch < c.channels; ch += parts * 256) {
     float *st = p.conv_state + (size_t)seg.slot * keep * c.channels + ch;
     for (int i = 0; i < keep; i++) {
       const int t = seg.n - keep + i;   // row of the stretch whose input belongs here; negative: an older one
@@ -162,23 +171,26 @@ struct ScanToken {
 
 // ONE: every sequence has one row (decoding); the launch is then a stream of states through the chip.
 template <int NI, int KIND, bool ONE>
-__global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restrict__ segs) {
+__global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restrict__ segs, int n_seg) {
   constexpr int KP = 32 * NI, TC = ONE ? 1 : SCAN_TOKENS;
   constexpr bool CHANNEL = KIND == SCAN_CHANNEL_DELTA, SSM = KIND == SCAN_STATE_SPACE;
-  constexpr int PIECES = (TC * KP + 255) / 256, VPIECES = (TC * SCAN_COLS + 255) / 256;
+  constexpr int PIECES = (TC * KP / 4 + 255) / 256, VPIECES = (TC * SCAN_COLS / 4 + 255) / 256;
   // one token more than is staged: the loop reads a token ahead
   __shared__ __attribute__((aligned(16))) float sk[TC + 1][KP], sq[TC + 1][KP], sg[CHANNEL ? TC + 1 : 1][KP];
-  __shared__ __attribute__((aligned(8))) float sv[TC + 1][SCAN_COLS];
+  __shared__ __attribute__((aligned(16))) float sv[TC + 1][SCAN_COLS];
   __shared__ float s_decay[TC + 1], s_beta[TC + 1];
-  const RowSeg seg = segs[blockIdx.x];
-  const int h = blockIdx.y;
-  if (h == p.heads) {
-    advance_conv_state(p, seg);
+  // workgroups in order of (head, column block, sequence); those of the convolutions' states come last
+  const int blocks = (p.V + SCAN_COLS - 1) / SCAN_COLS;
+  const int seg_id = blockIdx.x % n_seg, unit = blockIdx.x / n_seg;
+  const RowSeg seg = segs[seg_id];
+  if (unit >= p.heads * blocks) {
+    advance_conv_state(p, seg, unit - p.heads * blocks, blocks);
     return;
   }
+  const int h = unit / blocks;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int j = lane & 7;
-  const int c0 = blockIdx.z * SCAN_COLS, cw = wave * 16 + (lane >> 3) * 2;   // this lane's columns c0 + cw, + 1
+  const int c0 = (unit - h * blocks) * SCAN_COLS, cw = wave * 16 + (lane >> 3) * 2;   // this lane's columns c0 + cw, + 1
   const bool busy = c0 + wave * 16 < p.V;                                    // wave-uniform
   const int kh = h / (p.heads / p.key_heads);
   const float rate = expf(p.a_log[h]);
@@ -196,58 +208,73 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
         S[c][i] = __builtin_nontemporal_load(reinterpret_cast<const f32x4 *>(st + c * KP + 32 * i));
     }
 
-  // the next tokens' inputs travel through registers while the current ones are worked on
-  float rk[PIECES], rq[PIECES], rg[CHANNEL ? PIECES : 1], rv[VPIECES], r_beta = 0.f, r_decay = 0.f;
+  // the next tokens' inputs travel through registers, four values at a time, while the current ones are
+  // worked on; rows and columns outside the problem are read from inside it and replaced by zero
+  f32x4 rk[PIECES], rq[PIECES], rg[CHANNEL ? PIECES : 1], rv[VPIECES];
+  float r_beta = 0.f, r_decay = 0.f;
+  const float *k_src = p.conv + p.k_col + kh * p.K, *q_src = p.conv + p.q_col + kh * p.K;
+  const float *v_src = p.conv + p.v_col + h * p.V, *g_src = p.channel_decay + h * p.K;
+  auto load4 = [&](const float *row, int d, int limit) {
+    f32x4 x;
+    if (p.vec) {
+      x = *reinterpret_cast<const f32x4 *>(row + min(d, limit - 4));
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; e++) x[e] = row[min(d + e, limit - 1)];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; e++) x[e] = d + e < limit ? x[e] : 0.f;
+    return x;
+  };
   auto fetch = [&](int t0) {
     const int T = min(TC, seg.n - t0);
+    const size_t first = seg.row0 + t0;
 #pragma unroll
     for (int x = 0; x < PIECES; x++) {
-      const int idx = tid + 256 * x, t = idx / KP, d = idx - t * KP;
-      rk[x] = rq[x] = 0.f;
-      if (CHANNEL) rg[x] = 0.f;
-      if (t < T && d < p.K) {
-        const size_t row = seg.row0 + t0 + t;
-        const float *cr = p.conv + row * p.ld_conv + kh * p.K + d;
-        rk[x] = cr[p.k_col];
-        rq[x] = cr[p.q_col];
-        if (CHANNEL) rg[x] = p.channel_decay[row * p.ld_decay + h * p.K + d];
-      }
+      const int idx = tid + 256 * x, t = min(idx / (KP / 4), T - 1), d = idx % (KP / 4) * 4;
+      rk[x] = load4(k_src + (first + t) * p.ld_conv, d, p.K);
+      rq[x] = load4(q_src + (first + t) * p.ld_conv, d, p.K);
+      if (CHANNEL) rg[x] = load4(g_src + (first + t) * p.ld_decay, d, p.K);
     }
 #pragma unroll
     for (int x = 0; x < VPIECES; x++) {
-      const int idx = tid + 256 * x, t = idx / SCAN_COLS, c = idx - t * SCAN_COLS;
-      rv[x] = t < T && c0 + c < p.V ? p.conv[(size_t)(seg.row0 + t0 + t) * p.ld_conv + p.v_col + h * p.V + c0 + c] : 0.f;
+      const int idx = tid + 256 * x, t = min(idx / (SCAN_COLS / 4), T - 1), c = c0 + idx % (SCAN_COLS / 4) * 4;
+      rv[x] = load4(v_src + (first + t) * p.ld_conv, c, p.V);
     }
-    if (tid < T) {
-      const float *ir = p.in + (size_t)(seg.row0 + t0 + tid) * p.ld_in;
-      if (!SSM) r_beta = ir[p.beta_col + h];
-      if (!CHANNEL) r_decay = ir[p.decay_col + h];
-    }
+    const float *ir = p.in + (first + min(tid, T - 1)) * p.ld_in + h;
+    if (!SSM) r_beta = ir[p.beta_col];
+    if (!CHANNEL) r_decay = ir[p.decay_col];
   };
-  auto put = [&](int t0) {
-    const int T = min(TC, seg.n - t0);
+  auto put = [&]() {
 #pragma unroll
     for (int x = 0; x < PIECES; x++) {
-      const int idx = tid + 256 * x, t = idx / KP, d = idx - t * KP;
-      if (t < T) {
-        sk[t][d] = rk[x];
-        sq[t][d] = rq[x];
-        if (CHANNEL) sg[t][d] = d < p.K ? expf(-rate * softplus_f(rg[x] + p.dt_bias[h * p.K + d])) : 0.f;
+      const int idx = tid + 256 * x, t = idx / (KP / 4), d = idx % (KP / 4) * 4;
+      if (TC * KP / 4 % 256 == 0 || t < TC) {
+        *reinterpret_cast<f32x4 *>(&sk[t][d]) = rk[x];
+        *reinterpret_cast<f32x4 *>(&sq[t][d]) = rq[x];
+        if (CHANNEL) {
+          f32x4 g;
+#pragma unroll
+          for (int e = 0; e < 4; e++)
+            g[e] = exp_f(-rate * softplus_f(rg[x][e] + p.dt_bias[h * p.K + min(d + e, p.K - 1)]));
+          *reinterpret_cast<f32x4 *>(&sg[t][d]) = g;
+        }
       }
     }
 #pragma unroll
     for (int x = 0; x < VPIECES; x++) {
       const int idx = tid + 256 * x;
-      if (idx < TC * SCAN_COLS) (&sv[0][0])[idx] = rv[x];
+      if (TC * SCAN_COLS / 4 % 256 == 0 || idx < TC * SCAN_COLS / 4)
+        *reinterpret_cast<f32x4 *>(&sv[0][0] + idx * 4) = rv[x];
     }
-    if (tid < T) {
+    if (tid < TC) {
       if (SSM) {
         const float dt = softplus_f(r_decay + bias);
-        s_decay[tid] = expf(-rate * dt);
+        s_decay[tid] = exp_f(-rate * dt);
         s_beta[tid] = dt;
       } else {
         s_beta[tid] = sigmoid_f(r_beta);
-        if (!CHANNEL) s_decay[tid] = expf(-rate * softplus_f(r_decay + bias));
+        if (!CHANNEL) s_decay[tid] = exp_f(-rate * softplus_f(r_decay + bias));
       }
     }
   };
@@ -304,29 +331,35 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
       if (SSM) o[c] = fmaf(skip, x.v[c], o[c]);
     }
   };
+  // lane j of a group keeps the results of tokens t with t % 8 == j; they are stored eight at a time, those
+  // of a piece's last tokens after the next piece has been staged (the wait for its loads would otherwise
+  // be one for these stores)
+  float keep[2] = {0.f, 0.f};
+  int kept = -1;   // first row of the tokens in keep; -1: stored
+  auto flush = [&](int rows) {
+    if (j < rows) {
+      float *dst = p.out + (size_t)(kept + j) * p.ld_out + h * p.V + c0 + cw;
+      if (c0 + cw < p.V) dst[0] = keep[0];
+      if (c0 + cw + 1 < p.V) dst[1] = keep[1];
+    }
+    kept = -1;
+  };
   fetch(0);
   for (int t0 = 0; t0 < seg.n; t0 += TC) {
     const int T = min(TC, seg.n - t0);
     if (t0 > 0) __syncthreads();
-    put(t0);
+    put();
     __syncthreads();
     if (!ONE && t0 + TC < seg.n) fetch(t0 + TC);
     if (!busy) continue;
-    float keep[2] = {0.f, 0.f};
-    // lane j of a group keeps the results of tokens t with t % 8 == j and stores them together
+    if (!ONE && kept >= 0) flush(8);   // a full piece came before
     auto emit = [&](int t, const float (&o)[2]) {
       if ((t & 7) == j) {
         keep[0] = o[0];
         keep[1] = o[1];
       }
-      if ((t & 7) == 7 || t == T - 1) {
-        const int tj = (t & ~7) + j;
-        if (tj <= t) {
-          float *dst = p.out + (size_t)(seg.row0 + t0 + tj) * p.ld_out + h * p.V + c0 + cw;
-          if (c0 + cw < p.V) dst[0] = keep[0];
-          if (c0 + cw + 1 < p.V) dst[1] = keep[1];
-        }
-      }
+      if ((t & 7) == 0) kept = seg.row0 + t0 + t;
+      if ((t & 7) == 7 && t + 1 < TC) flush(8);
     };
     Token a;
     read(a, 0);
@@ -356,6 +389,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
       }
     }
   }
+  if (busy && kept >= 0) flush(seg.row0 + seg.n - kept);
 #pragma unroll
   for (int c = 0; c < 2; c++)
 #pragma unroll
@@ -482,8 +516,8 @@ int run_short_conv(const ShortConv &c, const StepRows &r, const float *in, int l
 
 template <int NI, int KIND>
 static void launch_scan_kind(const Scan &p, const StepRows &r, dim3 grid, hipStream_t s) {
-  if (r.longest == 1) scan_kernel<NI, KIND, true><<<grid, 256, 0, s>>>(p, r.segs);
-  else scan_kernel<NI, KIND, false><<<grid, 256, 0, s>>>(p, r.segs);
+  if (r.longest == 1) scan_kernel<NI, KIND, true><<<grid, 256, 0, s>>>(p, r.segs, r.n_seg);
+  else scan_kernel<NI, KIND, false><<<grid, 256, 0, s>>>(p, r.segs, r.n_seg);
 }
 
 template <int NI>
@@ -495,13 +529,19 @@ static void launch_scan(const Scan &p, const StepRows &r, dim3 grid, hipStream_t
   }
 }
 
-int run_scan(const Scan &p, const StepRows &r, hipStream_t s) {
+int run_scan(const Scan &scan, const StepRows &r, hipStream_t s) {
+  Scan p = scan;
+  p.vec = p.K % 4 == 0 && p.V % 4 == 0 && p.ld_conv % 4 == 0 && p.k_col % 4 == 0 && p.q_col % 4 == 0 && p.v_col % 4 == 0 &&
+          aligned(p.conv, 16) &&
+          (p.kind != SCAN_CHANNEL_DELTA || (p.ld_decay % 4 == 0 && aligned(p.channel_decay, 16)));
   GPTOSS_REQUIRE(p.K >= 1 && p.K <= SCAN_MAX_KEY && p.V >= 1 && p.key_heads >= 1 && p.heads % p.key_heads == 0,
                  GPTOSS_ERR_DIM, "scan: key dimension %d (at most %d), %d heads over %d", p.K, SCAN_MAX_KEY, p.heads,
                  p.key_heads);
+  GPTOSS_REQUIRE((long long)r.n_seg * (p.heads + 1) * cdiv(p.V, SCAN_COLS) < (1ll << 31), GPTOSS_ERR_DIM,
+                 "scan: too many workgroups");
   static const char *names[] = {"scan_delta", "scan_channel_delta", "scan_state_space"};
   TraceScope ts(names[p.kind], s);
-  const dim3 grid(r.n_seg, p.heads + 1, cdiv(p.V, SCAN_COLS));   // y == heads: the convolution's state
+  const dim3 grid((unsigned)(r.n_seg * (p.heads + 1) * cdiv(p.V, SCAN_COLS)));
   switch (scan_key_pad(p.K) / 32) {
     case 1: launch_scan<1>(p, r, grid, s); break;
     case 2: launch_scan<2>(p, r, grid, s); break;

@@ -43,6 +43,7 @@ struct Scan {
   // the convolution's state is brought up to date by the same launch
   ShortConv conv_desc;
   float *conv_state = nullptr;
+  int vec = 0;            // rows may be read 16 bytes at a time (run_scan sets it)
 };
 inline int scan_key_pad(int K) { return (K + 31) / 32 * 32; }
 inline size_t scan_state_elems(int heads, int K, int V) { return (size_t)heads * V * scan_key_pad(K); }
