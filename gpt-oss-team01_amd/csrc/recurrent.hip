@@ -2,10 +2,10 @@
 // state-space recurrence, with the short convolutions in front of them and the gated norms behind.
 //
 // The recurrence of a head acts on a K x V state whose V columns are independent of each other, so a
-// column lives in 8 lanes of a wave (K / 8 rows each, in registers) and a wave owns 16 columns: for a
-// step of one token the launch streams every state once through the chip, 16 bytes per lane and
+// column lives in 8 lanes of a wave (K / 8 rows each, in registers) and a wave owns 16 columns (8 where
+// there is little to share out): for a step of one token the launch streams every state once through the chip, 16 bytes per lane and
 // request; for a stretch of a prompt the state stays in registers while the tokens go by, their keys,
-// queries and gates staged in LDS and shared by the workgroup's 64 columns.  Everything is fp32, and
+// queries and gates staged in LDS and shared by the workgroup's columns.  Everything is fp32, and
 // the tokens are taken one after the other, so a sequence's results are bit for bit the same however
 // it is cut into steps.
 #include <type_traits>
@@ -144,7 +144,6 @@ __global__ __launch_bounds__(256) void short_conv_kernel(ShortConv c, const int 
 
 // ---- recurrence ----------------------------------------------------------------------------------
 constexpr int SCAN_TOKENS = 16;   // tokens staged at a time
-constexpr int SCAN_COLS = 64;     // state columns of a workgroup: 4 waves x 8 lane groups x 2
 
 // The convolution's last taps - 1 inputs after the stretch; one thread owns a channel.
 __device__ __forceinline__ void advance_conv_state(const Scan &p, const RowSeg &seg, int part, int parts) {
@@ -163,24 +162,27 @@ __device__ __forceinline__ void advance_conv_state(const Scan &p, const RowSeg &
 }
 
 // What a lane needs of one token.
-template <int NI, bool CHANNEL>
+template <int NI, bool CHANNEL, int CPL>
 struct ScanToken {
   f32x4 k[NI], q[NI], g[CHANNEL ? NI : 1];
-  float v[2], decay, beta;
+  float v[CPL], decay, beta;
 };
 
+// CPL: columns per lane; a workgroup has 4 waves x 8 lane groups x CPL columns.  Two share the reads of a
+// token's keys and queries; one gives twice the workgroups, where there are few heads and sequences.
 // ONE: every sequence has one row (decoding); the launch is then a stream of states through the chip.
-template <int NI, int KIND, bool ONE>
+template <int NI, int KIND, bool ONE, int CPL>
 __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restrict__ segs, int n_seg) {
   constexpr int KP = 32 * NI, TC = ONE ? 1 : SCAN_TOKENS;
   constexpr bool CHANNEL = KIND == SCAN_CHANNEL_DELTA, SSM = KIND == SCAN_STATE_SPACE;
-  constexpr int PIECES = (TC * KP / 4 + 255) / 256, VPIECES = (TC * SCAN_COLS / 4 + 255) / 256;
+  constexpr int COLS = 32 * CPL;
+  constexpr int PIECES = (TC * KP / 4 + 255) / 256, VPIECES = (TC * COLS / 4 + 255) / 256;
   // one token more than is staged: the loop reads a token ahead
   __shared__ __attribute__((aligned(16))) float sk[TC + 1][KP], sq[TC + 1][KP], sg[CHANNEL ? TC + 1 : 1][KP];
-  __shared__ __attribute__((aligned(16))) float sv[TC + 1][SCAN_COLS];
+  __shared__ __attribute__((aligned(16))) float sv[TC + 1][COLS];
   __shared__ float s_decay[TC + 1], s_beta[TC + 1];
   // workgroups in order of (head, column block, sequence); those of the convolutions' states come last
-  const int blocks = (p.V + SCAN_COLS - 1) / SCAN_COLS;
+  const int blocks = (p.V + COLS - 1) / COLS;
   const int seg_id = blockIdx.x % n_seg, unit = blockIdx.x / n_seg;
   const RowSeg seg = segs[seg_id];
   if (unit >= p.heads * blocks) {
@@ -190,17 +192,17 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
   const int h = unit / blocks;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int j = lane & 7;
-  const int c0 = (unit - h * blocks) * SCAN_COLS, cw = wave * 16 + (lane >> 3) * 2;   // this lane's columns c0 + cw, + 1
-  const bool busy = c0 + wave * 16 < p.V;                                    // wave-uniform
+  const int c0 = (unit - h * blocks) * COLS, cw = (wave * 8 + (lane >> 3)) * CPL;   // this lane's first column is c0 + cw
+  const bool busy = c0 + wave * 8 * CPL < p.V;   // wave-uniform
   const int kh = h / (p.heads / p.key_heads);
   const float rate = expf(p.a_log[h]);
   const float bias = CHANNEL ? 0.f : p.dt_bias[h];
   const float skip = SSM ? p.d_skip[h] : 0.f;
 
-  f32x4 S[2][NI];
+  f32x4 S[CPL][NI];
   float *st = p.state + (((size_t)seg.slot * p.heads + h) * p.V + c0 + cw) * KP + 4 * j;
 #pragma unroll
-  for (int c = 0; c < 2; c++)
+  for (int c = 0; c < CPL; c++)
 #pragma unroll
     for (int i = 0; i < NI; i++) {
       S[c][i] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -238,7 +240,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
     }
 #pragma unroll
     for (int x = 0; x < VPIECES; x++) {
-      const int idx = tid + 256 * x, t = min(idx / (SCAN_COLS / 4), T - 1), c = c0 + idx % (SCAN_COLS / 4) * 4;
+      const int idx = tid + 256 * x, t = min(idx / (COLS / 4), T - 1), c = c0 + idx % (COLS / 4) * 4;
       rv[x] = load4(v_src + (first + t) * p.ld_conv, c, p.V);
     }
     const float *ir = p.in + (first + min(tid, T - 1)) * p.ld_in + h;
@@ -264,7 +266,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
 #pragma unroll
     for (int x = 0; x < VPIECES; x++) {
       const int idx = tid + 256 * x;
-      if (TC * SCAN_COLS / 4 % 256 == 0 || idx < TC * SCAN_COLS / 4)
+      if (TC * COLS / 4 % 256 == 0 || idx < TC * COLS / 4)
         *reinterpret_cast<f32x4 *>(&sv[0][0] + idx * 4) = rv[x];
     }
     if (tid < TC) {
@@ -278,7 +280,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
       }
     }
   };
-  using Token = ScanToken<NI, CHANNEL>;
+  using Token = ScanToken<NI, CHANNEL, CPL>;
   auto read = [&](Token &x, int t) {
 #pragma unroll
     for (int i = 0; i < NI; i++) {
@@ -286,21 +288,21 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
       x.q[i] = *reinterpret_cast<const f32x4 *>(&sq[t][32 * i + 4 * j]);
       if (CHANNEL) x.g[i] = *reinterpret_cast<const f32x4 *>(&sg[t][32 * i + 4 * j]);
     }
-    x.v[0] = sv[t][cw];
-    x.v[1] = sv[t][cw + 1];
+#pragma unroll
+    for (int c = 0; c < CPL; c++) x.v[c] = sv[t][cw + c];
     x.beta = s_beta[t];
     if (!CHANNEL) x.decay = s_decay[t];
   };
-  auto advance = [&](const Token &x, float (&o)[2]) {
+  auto advance = [&](const Token &x, float (&o)[CPL]) {
 #pragma unroll
-    for (int c = 0; c < 2; c++)
+    for (int c = 0; c < CPL; c++)
 #pragma unroll
       for (int i = 0; i < NI; i++)
 #pragma unroll
         for (int e = 0; e < 4; e++) S[c][i][e] *= CHANNEL ? x.g[CHANNEL ? i : 0][e] : x.decay;
-    float u[2];
+    float u[CPL];
 #pragma unroll
-    for (int c = 0; c < 2; c++) {
+    for (int c = 0; c < CPL; c++) {
       if constexpr (SSM) {
         u[c] = x.beta * x.v[c];
       } else {
@@ -316,7 +318,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
       }
     }
 #pragma unroll
-    for (int c = 0; c < 2; c++) {
+    for (int c = 0; c < CPL; c++) {
       float d0 = 0.f, d1 = 0.f;
 #pragma unroll
       for (int i = 0; i < NI; i++) {
@@ -334,13 +336,14 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
   // lane j of a group keeps the results of tokens t with t % 8 == j; they are stored eight at a time, those
   // of a piece's last tokens after the next piece has been staged (the wait for its loads would otherwise
   // be one for these stores)
-  float keep[2] = {0.f, 0.f};
+  float keep[CPL];
   int kept = -1;   // first row of the tokens in keep; -1: stored
   auto flush = [&](int rows) {
     if (j < rows) {
       float *dst = p.out + (size_t)(kept + j) * p.ld_out + h * p.V + c0 + cw;
-      if (c0 + cw < p.V) dst[0] = keep[0];
-      if (c0 + cw + 1 < p.V) dst[1] = keep[1];
+#pragma unroll
+      for (int c = 0; c < CPL; c++)
+        if (c0 + cw + c < p.V) dst[c] = keep[c];
     }
     kept = -1;
   };
@@ -353,25 +356,23 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
     if (!ONE && t0 + TC < seg.n) fetch(t0 + TC);
     if (!busy) continue;
     if (!ONE && kept >= 0) flush(8);   // a full piece came before
-    auto emit = [&](int t, const float (&o)[2]) {
-      if ((t & 7) == j) {
-        keep[0] = o[0];
-        keep[1] = o[1];
-      }
+    auto emit = [&](int t, const float (&o)[CPL]) {
+#pragma unroll
+      for (int c = 0; c < CPL; c++) keep[c] = (t & 7) == j ? o[c] : keep[c];
       if ((t & 7) == 0) kept = seg.row0 + t0 + t;
       if ((t & 7) == 7 && t + 1 < TC) flush(8);
     };
     Token a;
     read(a, 0);
     if constexpr (ONE) {
-      float o[2];
+      float o[CPL];
       advance(a, o);
       emit(0, o);
     } else if constexpr (NI <= 4) {
       // two tokens in registers: the next one's inputs are requested before the current one is worked on
       Token b;
       for (int t = 0; t < T; t += 2) {
-        float o[2];
+        float o[CPL];
         read(b, t + 1);
         advance(a, o);
         emit(t, o);
@@ -382,7 +383,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
       }
     } else {
       for (int t = 0; t < T; t++) {
-        float o[2];
+        float o[CPL];
         advance(a, o);
         emit(t, o);
         if (t + 1 < T) read(a, t + 1);
@@ -391,7 +392,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
   }
   if (busy && kept >= 0) flush(seg.row0 + seg.n - kept);
 #pragma unroll
-  for (int c = 0; c < 2; c++)
+  for (int c = 0; c < CPL; c++)
 #pragma unroll
     for (int i = 0; i < NI; i++)
       if (c0 + cw + c < p.V)
@@ -515,17 +516,21 @@ int run_short_conv(const ShortConv &c, const StepRows &r, const float *in, int l
 }
 
 template <int NI, int KIND>
-static void launch_scan_kind(const Scan &p, const StepRows &r, dim3 grid, hipStream_t s) {
-  if (r.longest == 1) scan_kernel<NI, KIND, true><<<grid, 256, 0, s>>>(p, r.segs, r.n_seg);
-  else scan_kernel<NI, KIND, false><<<grid, 256, 0, s>>>(p, r.segs, r.n_seg);
+static void launch_scan_kind(const Scan &p, const StepRows &r, hipStream_t s) {
+  auto grid = [&](int cols) { return dim3((unsigned)(r.n_seg * (p.heads + 1) * cdiv(p.V, cols))); };
+  // stretches of few heads and sequences: with two columns per lane half of the chip would be idle
+  const bool few = (long long)r.n_seg * p.heads * cdiv(p.V, 64) <= 128;
+  if (r.longest == 1) scan_kernel<NI, KIND, true, 2><<<grid(64), 256, 0, s>>>(p, r.segs, r.n_seg);
+  else if (few) scan_kernel<NI, KIND, false, 1><<<grid(32), 256, 0, s>>>(p, r.segs, r.n_seg);
+  else scan_kernel<NI, KIND, false, 2><<<grid(64), 256, 0, s>>>(p, r.segs, r.n_seg);
 }
 
 template <int NI>
-static void launch_scan(const Scan &p, const StepRows &r, dim3 grid, hipStream_t s) {
+static void launch_scan(const Scan &p, const StepRows &r, hipStream_t s) {
   switch (p.kind) {
-    case SCAN_DELTA: launch_scan_kind<NI, SCAN_DELTA>(p, r, grid, s); break;
-    case SCAN_CHANNEL_DELTA: launch_scan_kind<NI, SCAN_CHANNEL_DELTA>(p, r, grid, s); break;
-    case SCAN_STATE_SPACE: launch_scan_kind<NI, SCAN_STATE_SPACE>(p, r, grid, s); break;
+    case SCAN_DELTA: launch_scan_kind<NI, SCAN_DELTA>(p, r, s); break;
+    case SCAN_CHANNEL_DELTA: launch_scan_kind<NI, SCAN_CHANNEL_DELTA>(p, r, s); break;
+    case SCAN_STATE_SPACE: launch_scan_kind<NI, SCAN_STATE_SPACE>(p, r, s); break;
   }
 }
 
@@ -537,20 +542,19 @@ int run_scan(const Scan &scan, const StepRows &r, hipStream_t s) {
   GPTOSS_REQUIRE(p.K >= 1 && p.K <= SCAN_MAX_KEY && p.V >= 1 && p.key_heads >= 1 && p.heads % p.key_heads == 0,
                  GPTOSS_ERR_DIM, "scan: key dimension %d (at most %d), %d heads over %d", p.K, SCAN_MAX_KEY, p.heads,
                  p.key_heads);
-  GPTOSS_REQUIRE((long long)r.n_seg * (p.heads + 1) * cdiv(p.V, SCAN_COLS) < (1ll << 31), GPTOSS_ERR_DIM,
+  GPTOSS_REQUIRE((long long)r.n_seg * (p.heads + 1) * cdiv(p.V, 32) < (1ll << 31), GPTOSS_ERR_DIM,
                  "scan: too many workgroups");
   static const char *names[] = {"scan_delta", "scan_channel_delta", "scan_state_space"};
   TraceScope ts(names[p.kind], s);
-  const dim3 grid((unsigned)(r.n_seg * (p.heads + 1) * cdiv(p.V, SCAN_COLS)));
   switch (scan_key_pad(p.K) / 32) {
-    case 1: launch_scan<1>(p, r, grid, s); break;
-    case 2: launch_scan<2>(p, r, grid, s); break;
-    case 3: launch_scan<3>(p, r, grid, s); break;
-    case 4: launch_scan<4>(p, r, grid, s); break;
-    case 5: launch_scan<5>(p, r, grid, s); break;
-    case 6: launch_scan<6>(p, r, grid, s); break;
-    case 7: launch_scan<7>(p, r, grid, s); break;
-    default: launch_scan<8>(p, r, grid, s); break;
+    case 1: launch_scan<1>(p, r, s); break;
+    case 2: launch_scan<2>(p, r, s); break;
+    case 3: launch_scan<3>(p, r, s); break;
+    case 4: launch_scan<4>(p, r, s); break;
+    case 5: launch_scan<5>(p, r, s); break;
+    case 6: launch_scan<6>(p, r, s); break;
+    case 7: launch_scan<7>(p, r, s); break;
+    default: launch_scan<8>(p, r, s); break;
   }
   GPTOSS_LAUNCH_CHECK("scan_kernel");
   return GPTOSS_OK;

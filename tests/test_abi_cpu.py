@@ -53,7 +53,7 @@ def test_no_oracle_or_cpu_fallback_in_product(lib):
 
 def test_argument_validation_without_gpu(lib):
     L = lib.load()
-    assert L.gptoss_abi_version() == 101
+    assert L.gptoss_abi_version() == 102
     # null pointers and bad dimensions are rejected before anything touches a device
     assert L.gptoss_router_gemm(None, None, None, None, 4, 256, 8, None) == 1
     assert "null" in lib.last_error()
