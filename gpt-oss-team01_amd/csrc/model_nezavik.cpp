@@ -233,7 +233,7 @@ struct Loader {
       m.packed = b.upload_matrices(st ? full.data() : nullptr, 1, n_out, n_in, true, 0, next_seed(), 1.f / sqrtf((float)n_in));
     return m;
   }
-  // a norm with one number: the vector the norm kernels take, zero in the padding
+  // a norm whose gain is a scalar, as the vector the norm kernels take (zero in the padding)
   float *scalar_norm(const std::string &name) {
     std::vector<float> v(e->hidden, 0.f);
     const float g = st ? host(name, {})[0] : 1.f;

@@ -9,7 +9,7 @@ namespace gptoss {
 // projected rows; some of its heads are then made unit vectors.
 struct ShortConv {
   int col = 0, channels = 0, taps = 1;  // taps - 1 earlier inputs per channel are state
-  const float *weight = nullptr;        // [channels, taps], last column: the current token's
+  const float *weight = nullptr;        // [channels, taps], newest tap last
   const float *bias = nullptr;          // [channels] or nullptr
   // the first n_unit * 2 heads of unit_dim channels are unit vectors; the first n_unit of them are
   // also scaled by unit_scale (queries, then keys); the remaining channels are taken as they are

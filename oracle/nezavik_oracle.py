@@ -52,7 +52,7 @@ def linear(h, weight):
 
 # ---- short convolution -------------------------------------------------------------------------
 def short_conv(x, taps, bias=None):
-    """x [T, C]; taps [C, n], the last column weighs the current token; zeros before the start."""
+    """x [T, C]; taps [C, n], oldest first; nothing precedes token 0."""
     x, taps = f64(x), f64(taps)
     T, C = x.shape
     n = taps.shape[1]

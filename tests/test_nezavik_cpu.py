@@ -20,7 +20,7 @@ def test_short_conv_is_a_causal_convolution():
     y = nz.short_conv(x, taps, bias)
     for c in range(3):
         assert np.allclose(y[:, c], np.convolve(x[:, c], taps[c, ::-1])[:9] + bias[c])
-    assert np.allclose(nz.short_conv(x, taps[:, -1:]), x * taps[:, -1])     # one tap: the current token's
+    assert np.allclose(nz.short_conv(x, taps[:, -1:]), x * taps[:, -1])     # one tap: no memory
 
 
 def test_delta_rule_stores_and_overwrites():
@@ -31,7 +31,7 @@ def test_delta_rule_stores_and_overwrites():
     q = keys[[0, 0, 1, 2, 1, 0]][:, None, :]
     one = np.ones((6, 1))
     o, S = nz.delta_rule(q, k, vals, one, np.ones((6, 1, 4)))
-    for t, src in enumerate([0, 0, 1, 2, 3, 5]):                          # the read-out sees the token's own write
+    for t, src in enumerate([0, 0, 1, 2, 3, 5]):                          # a read includes what its own token wrote
         assert np.allclose(o[t, 0], vals[src, 0])
     # beta = 0 writes nothing; a decay of 0 forgets before it reads
     o2, S2 = nz.delta_rule(q, k, vals, 0 * one, np.ones((6, 1, 4)), S)

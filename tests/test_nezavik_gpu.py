@@ -96,8 +96,8 @@ def test_each_mechanism_alone(open_model, name, precise):
 
 @BOTH
 def test_first_tokens_of_a_sequence(open_model, precise):
-    """Zeros in front of the start: lengths below, at and above every number of taps, in one step and
-    token by token."""
+    """Convolutions that reach past token 0: lengths below, at and above every number of taps, in one step
+    and token by token."""
     cfg = nm.config([nm.delta(conv=5), nm.parallel(conv=4), nm.channel_delta(conv=2)])
     w = nm.weights(cfg, 5)
     e = open_model(cfg, w, precise)
