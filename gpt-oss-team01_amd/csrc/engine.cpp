@@ -123,7 +123,11 @@ int gptoss_engine::class_gemm(int row0, int count, float *out) {
   return dense_gemm(t + (size_t)row0 * hidden, unembedding, class_bias, out, EPI_F32, count, vocab_rows, hidden, stream);
 }
 
-// Final norm and next ids of sampled rows first .. first + count - 1 (count <= max_batch); with the
+int gptoss_engine::norm_sampled(int m) {
+  return run_rmsnorm(x, nullptr, final_norm, t, t_f32, m, hidden, stream, norm_eps, hidden_real);
+}
+
+// Next ids of normed sampled rows first .. first + count - 1 (count <= max_batch); with the
 // logits kept, those of a sequence's row stay in its slot's place.
 int gptoss_engine::sample_rows(const StepRows &r, const int *sample, const int *slot, int first, int count) {
   if (logits) {
@@ -135,6 +139,7 @@ int gptoss_engine::sample_rows(const StepRows &r, const int *sample, const int *
       float *lg = logits + (size_t)slot[sample[first + j]] * vocab_rows;
       GPTOSS_STEP(class_gemm(j, m, lg));
       GPTOSS_STEP(run_argmax(lg, d_next + j, m, vocab_rows, stream));
+      if (logit_softcap > 0.f) GPTOSS_STEP(run_softcap(lg, (size_t)m * vocab_rows, logit_softcap, stream));
     }
     return GPTOSS_OK;
   }
@@ -158,9 +163,10 @@ int gptoss_engine::run_rows(int n, const int *tok, const int *slot, const int *p
   for (int first = 0; first < n_sample; first += max_batch) {
     const int m = std::min(max_batch, n_sample - first);
     GPTOSS_STEP(run_gather_rows_idx(rows_x, x, r.sample + first, m, hidden, stream));
-    GPTOSS_STEP(run_rmsnorm(x, nullptr, final_norm, t, t_f32, m, hidden, stream, norm_eps, hidden_real));
+    GPTOSS_STEP(norm_sampled(m));
     if (host_logits) {
       GPTOSS_STEP(class_gemm(0, m, logits));
+      if (logit_softcap > 0.f) GPTOSS_STEP(run_softcap(logits, (size_t)m * vocab_rows, logit_softcap, stream));
       GPTOSS_HIP(hipMemcpy2DAsync(host_logits + (size_t)first * vocab, sizeof(float) * vocab, logits,
                                   sizeof(float) * vocab_rows, sizeof(float) * vocab, m, hipMemcpyDeviceToHost, stream));
       GPTOSS_HIP(hipStreamSynchronize(stream));   // the buffer is reused by the next portion
@@ -171,6 +177,14 @@ int gptoss_engine::run_rows(int n, const int *tok, const int *slot, const int *p
   }
   GPTOSS_HIP(hipStreamSynchronize(stream));
   if (host_next && !host_logits) memcpy(host_next, h_next, sizeof(int) * n_sample);
+  return GPTOSS_OK;
+}
+
+int gptoss_engine::continue_slots(const std::vector<RowSeg> &segs) {
+  for (const RowSeg &s : segs)
+    GPTOSS_REQUIRE(s.pos0 == 0 || s.pos0 == lengths[s.slot], GPTOSS_ERR_STATE,
+                   "step: slot %d holds %d positions and cannot continue at position %d", s.slot, lengths[s.slot], s.pos0);
+  for (const RowSeg &s : segs) lengths[s.slot] = s.pos0 + s.n;
   return GPTOSS_OK;
 }
 

@@ -56,6 +56,7 @@ struct gptoss_engine {
   gptoss::bf16_t *unembedding = nullptr;
   float *unembedding_f32 = nullptr;
   float *class_bias = nullptr;   // [vocab_rows]: 0, and a large negative value in the padding; or nullptr
+  float logit_softcap = 0.f;     // > 0: logits become softcap * tanh(logits / softcap) (their order stays)
   // run state
   int *d_next = nullptr;
   int *h_next = nullptr;         // pinned
@@ -74,6 +75,7 @@ struct gptoss_engine {
   std::vector<gptoss::RowSeg> seg_scratch;
   // cache slots handed out to callers that keep sequences of their own
   std::vector<char> slot_used;
+  std::vector<int> lengths;      // models with states: positions every slot's states hold (continue_slots)
 
   virtual ~gptoss_engine();
   bool precise() const { return (flags & GPTOSS_ENGINE_PRECISE) != 0; }
@@ -89,7 +91,13 @@ struct gptoss_engine {
   // Positions 0..T-1 of sequences 0..B-1.
   virtual int prefill(const int *host_tokens, int B, int T, int *host_next);
   virtual bool reference_schedule() const { return false; }
+  // x (m sampled rows) -> t (and t_f32): the norm in front of the classifier.
+  virtual int norm_sampled(int m);
   virtual int tensor_view(int tensor, int layer, void **ptr, size_t *bytes);
+
+  // check_segments of models with states: a state knows only its own position, so a sequence goes on where it
+  // stopped, or starts over.
+  int continue_slots(const std::vector<gptoss::RowSeg> &segs);
 
   // Validate, upload and run a row list; then next ids (host_next) or logits (host_logits) of the
   // sampled rows.  n <= rows; n_sample <= max_batch for ids.

@@ -1,6 +1,7 @@
 // Internal interface of the grouped (moe_gemm.hip) and dense (gemm_dense.cpp) GEMM kernels.
 #pragma once
 #include "common.hpp"
+#include "glue.hpp"
 
 namespace gptoss {
 
@@ -13,6 +14,13 @@ struct GemmBf16Range {
   bf16_t *out = nullptr;  // column `from` of row 0
   int ld = 0;             // elements per row, a multiple of 4
   int relu_squared = 0;   // the square of relu instead of the value itself
+};
+
+// The gated activation of an expert's first product (EPI_SWIGLU):
+//   g sigmoid(rate g) (u + shift),  g = min(gate, limit), u = up clamped to [-limit, limit].
+// GPT-OSS: rate 1.702, shift 1 and a limit; silu(gate) * up: rate 1, shift 0, no limit.
+struct GluForm {
+  float rate = 1.702f, shift = 1.f, limit = 7.f;
 };
 
 // Row tiles of ONE expert are grouped into blocks of up to MOE_TILE_BLOCK consecutive tiles by the
@@ -42,7 +50,7 @@ struct GemmParams {
   int dense_rows;      // rows of the dense problem when tiles == nullptr
   int N, K;
   int n_col_tiles;     // gemm_col_tiles(N)
-  float limit;         // SwiGLU clamp
+  GluForm glu;         // EPI_SWIGLU
   GemmBf16Range range[2];  // EPI_MIXED
   int k_splits;        // EPI_PARTIAL (dense only): the sum over K is cut into k_splits parts of split_slabs
   int split_slabs;     // 64-k slabs; part s is written to out + s * dense_rows * N (no bias)
@@ -66,11 +74,14 @@ inline bool gemm_tall_shape_ok(int N, int K, long long max_rows) {
 int check_gemm_tall(const GemmParams &p, bool gather, int epi, long long max_rows);
 int run_gemm_tall(const GemmParams &p, int epi, int max_tiles, long long max_rows, hipStream_t s);  // no gather
 int run_gemm_tall_gather(const GemmParams &p, int max_tiles, long long max_rows, hipStream_t s);    // gemm_tall_grouped.hip
+// MXFP4 weights: set by gemm_mxfp4.hip where that is linked
+extern int (*run_gemm_mxfp4)(const GemmParams &p, bool gather, int epi, int rows_per_tile, int max_tiles, hipStream_t s);
 // norm_w / norm_out (optional, accumulate only): also write RMSNorm(out) * norm_w as bf16.  Returns
 // with only the combine done when the fused form does not apply (H > 4096 or misaligned); the
-// caller checks with combine_norm_applies().
+// caller checks with combine_norm_applies().  With tanh_norm that norm instead, for any H.
 int run_combine(const float *y2, const float *topk_w, const int *inv_perm, float *out, int B, int H,
-                int k, int accumulate, const float *norm_w, bf16_t *norm_out, hipStream_t s);
+                int k, int accumulate, const float *norm_w, bf16_t *norm_out, hipStream_t s,
+                const TanhNorm *tanh_norm = nullptr);
 inline bool combine_norm_applies(int H, const float *norm_w, const bf16_t *norm_out) {
   return norm_w && norm_out && H % 4 == 0 && H <= 4096 && aligned(norm_w, 16) && aligned(norm_out, 8);
 }
@@ -88,6 +99,12 @@ struct MoePreNorm {
 int moe_forward_norm(const gptoss_moe_weights *w, const void *t, int B, float *out, void *workspace,
                      size_t workspace_bytes, hipStream_t s, int mxfp4, const float *norm_w, bf16_t *norm_out,
                      const MoePreNorm *pre = nullptr);
+// Most experts per token inside the framework (the C ABI's entry points take up to 8)
+constexpr int MOE_MAX_TOP = 32;
+// The MoE block of models with another activation: out += block(t), and with norm.weight also
+// norm_out = norm(out), in the same kernel as the combine.
+int moe_forward_glu(const gptoss_moe_weights *w, const GluForm &glu, const void *t, int B, float *out, void *workspace,
+                    size_t workspace_bytes, hipStream_t s, const TanhNorm &norm, bf16_t *norm_out);
 // moe_route.hip: residual add + RMSNorm + router GEMM + gating in one launch
 bool norm_router_applies(int B, int H, int E, const float *x, const float *residual, const float *weight,
                          const void *t_out);

@@ -23,7 +23,7 @@
 //     row and 16 channels: stores are 8/16 bytes wide, and since the packing order puts the gates
 //     of 16 (gate,up) pairs in channels 0-15 of a wave's block and their ups in channels 16-31,
 //     each pair sits in two registers of the same lane;
-//   * epilogues: +bias -> fp32, or +bias -> clamped SwiGLU -> bf16; for the dense form also the row arg-max,
+//   * epilogues: +bias -> fp32, or +bias -> gated activation (clamped SwiGLU, silu) -> bf16; for the dense form also the row arg-max,
 //     fp32 next to bf16 column ranges, and partial sums over parts of K.
 #pragma once
 
@@ -166,7 +166,7 @@ __device__ __forceinline__ void epilogue_store(const GemmParams &p, int mat, int
     // address = wave-uniform base (scalar registers) + a 32-bit per-lane element offset
     bf16_t *o = reinterpret_cast<bf16_t *>(p.out) + (size_t)row0 * half_n + (n0 >> 1);
     const uint32_t lane_off = (uint32_t)tok * (uint32_t)half_n + (uint32_t)h4;
-    const float L = p.limit;
+    const float L = p.glu.limit, shift = p.glu.shift, rate = -p.glu.rate * 1.4426950408889634f;
     const int row_lim = rows - tok;  // block i of this lane is a real row iff i*32 < row_lim
 #pragma unroll
     for (int i = 0; i < MB; i++) {
@@ -181,10 +181,10 @@ __device__ __forceinline__ void epilogue_store(const GemmParams &p, int mat, int
             float up = acc[i][(g + 2) * 4 + q] + bu[g * 4 + q];
             gate = fminf(gate, L);
             up = fminf(fmaxf(up, -L), L);
-            // gate * sigmoid(1.702 gate) * (up + 1); exp2 and the hardware reciprocal are accurate
+            // gate * sigmoid(rate gate) * (up + shift); exp2 and the hardware reciprocal are accurate
             // to a few ulp of fp32, far inside the bf16 rounding of the result
-            const float e = __builtin_amdgcn_exp2f(-1.702f * 1.4426950408889634f * gate);
-            v[q] = gate * __builtin_amdgcn_rcpf(1.0f + e) * (up + 1.0f);
+            const float e = __builtin_amdgcn_exp2f(rate * gate);
+            v[q] = gate * __builtin_amdgcn_rcpf(1.0f + e) * (up + shift);
           }
           const u32x2 pk = u32x2{pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
           if (hold) *reinterpret_cast<u32x2 *>(hold + (i * 32 + tok) * HOLD_ROW + hold_col + h4 + g * 8) = pk;

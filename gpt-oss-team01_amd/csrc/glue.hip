@@ -506,8 +506,8 @@ int run_synth_f32(float *dst, size_t n, uint64_t seed, float mean, float std, hi
   return GPTOSS_OK;
 }
 
-// x[b,:] = table[token[b],:] + positions[p,:], p = lens[b] - 1 (a learned position vector), fp32 rows of
-// stride ld whose columns from H on are zero; also the first entry of the depth average's history.
+// x[b,:] = table[token[b],:] + positions[p,:], p = lens[b] - 1 (a learned position vector, or nullptr), fp32 rows
+// of stride ld whose columns from H on are zero; x0 (or nullptr): the first entry of the depth average's history.
 template <typename T>
 __global__ __launch_bounds__(256) void embedding_position_kernel(const T *__restrict__ table,
                                                                  const T *__restrict__ positions,
@@ -522,9 +522,10 @@ __global__ __launch_bounds__(256) void embedding_position_kernel(const T *__rest
     else return v;
   };
   for (int h = threadIdx.x; h < ld; h += 256) {
-    const float v = h < H ? value(table[(size_t)tok * H + h]) + value(positions[(size_t)pos * H + h]) : 0.f;
+    float v = h < H ? value(table[(size_t)tok * H + h]) : 0.f;
+    if (positions && h < H) v += value(positions[(size_t)pos * H + h]);
     x[(size_t)b * ld + h] = v;
-    x0[(size_t)b * ld + h] = v;
+    if (x0) x0[(size_t)b * ld + h] = v;
   }
 }
 
@@ -599,6 +600,61 @@ __global__ __launch_bounds__(256) void depth_average_norm_kernel(float *__restri
       if (t_f32) *reinterpret_cast<f32x4 *>(t_f32 + row + h) = o;
     }
   }
+}
+
+// One thread per four elements of [rows, H].
+__global__ __launch_bounds__(256) void residual_tanh_norm_kernel(float *__restrict__ x, const float *__restrict__ y, int parts,
+                                                                 size_t part_stride, TanhNorm norm,
+                                                                 bf16_t *__restrict__ t_bf16, float *__restrict__ t_f32,
+                                                                 int H) {
+  const size_t at = ((size_t)blockIdx.x * 256 + threadIdx.x) * 4;
+  if (at >= part_stride) return;
+  f32x4 v = *reinterpret_cast<const f32x4 *>(x + at);
+  if (parts > 0) {
+    // sums in order of their index, four loads in flight at a time
+    f32x4 own = *reinterpret_cast<const f32x4 *>(y + at);
+    int k = 1;
+    for (; k + 4 <= parts; k += 4) {
+      f32x4 part[4];
+#pragma unroll
+      for (int q = 0; q < 4; q++) part[q] = *reinterpret_cast<const f32x4 *>(y + (k + q) * part_stride + at);
+#pragma unroll
+      for (int q = 0; q < 4; q++) own += part[q];
+    }
+    for (; k < parts; k++) own += *reinterpret_cast<const f32x4 *>(y + k * part_stride + at);
+    v += own;
+    *reinterpret_cast<f32x4 *>(x + at) = v;
+  }
+  if (!norm.weight) return;
+  const int h = (int)(at % (unsigned)H);
+  const f32x4 w = *reinterpret_cast<const f32x4 *>(norm.weight + h), b = *reinterpret_cast<const f32x4 *>(norm.bias + h);
+  f32x4 o;
+#pragma unroll
+  for (int q = 0; q < 4; q++) o[q] = fmaf(tanhf(norm.alpha * v[q]), w[q], b[q]);
+  *reinterpret_cast<u32x2 *>(t_bf16 + at) = u32x2{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
+  if (t_f32) *reinterpret_cast<f32x4 *>(t_f32 + at) = o;
+}
+
+__global__ __launch_bounds__(256) void softcap_kernel(float *__restrict__ z, size_t n, float cap) {
+  for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256)
+    z[i] = cap * tanhf(z[i] / cap);
+}
+
+int run_residual_tanh_norm(float *x, const float *y, int parts, const TanhNorm &norm, bf16_t *t_bf16, float *t_f32,
+                           int rows, int H, hipStream_t s) {
+  GPTOSS_REQUIRE(H % 4 == 0, GPTOSS_ERR_DIM, "tanh_norm: rows of %d elements (a multiple of 4)", H);
+  TraceScope ts("residual_tanh_norm", s);
+  const size_t n = (size_t)rows * H;
+  residual_tanh_norm_kernel<<<(unsigned)((n / 4 + 255) / 256), 256, 0, s>>>(x, y, parts, n, norm, t_bf16, t_f32, H);
+  GPTOSS_LAUNCH_CHECK("residual_tanh_norm_kernel");
+  return GPTOSS_OK;
+}
+
+int run_softcap(float *z, size_t n, float cap, hipStream_t s) {
+  TraceScope ts("softcap", s);
+  softcap_kernel<<<grid_for(n), 256, 0, s>>>(z, n, cap);
+  GPTOSS_LAUNCH_CHECK("softcap_kernel");
+  return GPTOSS_OK;
 }
 
 template <typename T>

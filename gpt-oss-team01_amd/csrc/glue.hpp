@@ -9,7 +9,17 @@ int run_embedding(const bf16_t *table, const int *tokens, float *x, int B, int H
 // is taken over (0: H)
 int run_rmsnorm(float *x, const float *residual, const float *weight, bf16_t *t_bf16, float *t_f32,
                 int B, int H, hipStream_t s, float eps = 1e-5f, int n_mean = 0);
-// x = x0 = table[token] + positions[lens - 1], rows of stride ld (zero from column H on)
+// x (+= the sum of `parts` partial sums y [parts][rows, H]; 0: nothing) and, with a norm,
+// t = tanh(alpha x) * weight + bias: a norm without a statistic over the row ("dynamic tanh")
+struct TanhNorm {
+  const float *weight = nullptr, *bias = nullptr;   // [H]; nullptr: no norm
+  float alpha = 1.f;
+};
+int run_residual_tanh_norm(float *x, const float *y, int parts, const TanhNorm &norm, bf16_t *t_bf16, float *t_f32,
+                           int rows, int H, hipStream_t s);
+// z = cap * tanh(z / cap)
+int run_softcap(float *z, size_t n, float cap, hipStream_t s);
+// x = x0 = table[token] + positions[lens - 1], rows of stride ld (zero from column H on); positions and x0 may be null
 int run_embedding_position(const bf16_t *table, const bf16_t *positions, const int *tokens, const int *lens, float *x,
                            float *x0, int rows, int H, int ld, int V, int n_pos, hipStream_t s);
 int run_embedding_position_f32(const float *table, const float *positions, const int *tokens, const int *lens,

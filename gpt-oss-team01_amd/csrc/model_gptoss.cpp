@@ -231,7 +231,7 @@ static int precise_step(GptOss *e, int pos, int B) {
     // one row per (token, slot): the slot's expert selects the matrix
     STEP(precise_matmul(pr.mlp1, pr.t, W + pr.w1 + (size_t)l * E * 2 * I * H, W + pr.b1 + (size_t)l * E * 2 * I,
                         pr.topk_i, B * k, H, 2 * I, k, s));
-    STEP(precise_swiglu(pr.mlp1, pr.act, B * k, I, c.swiglu_limit, s));
+    STEP(precise_swiglu(pr.mlp1, pr.act, B * k, I, GluForm{1.702f, 1.f, c.swiglu_limit}, s));
     STEP(precise_matmul(pr.mlp2, pr.act, W + pr.w2 + (size_t)l * E * H * I, W + pr.b2 + (size_t)l * E * H,
                         pr.topk_i, B * k, I, H, 1, s));
     STEP(precise_moe_agg(pr.mlp2, pr.topk_w, pr.topk_i, e->x, B, H, k, s));

@@ -10,10 +10,7 @@
 //   columns of one packed matrix), and the depth average with the next layer's norm.
 // Every size and constant comes from config.json or a tensor's shape.  With GPTOSS_ENGINE_PRECISE
 // weights, activations and the K/V ring are fp32 and so is every product.
-#include <math.h>
-
-#include "builder.hpp"
-#include "model_registry.hpp"
+#include "model_loader.hpp"
 #include "recurrent.hpp"
 #include "window_attn.hpp"
 
@@ -23,12 +20,6 @@ namespace {
 
 // rows of one sequence in a pass: the window rings hold the window in front of such a stretch as well
 constexpr int NEZAVIK_STRETCH = 2048;
-
-struct Matrix {   // bf16 packed, or fp32 row-major
-  bf16_t *packed = nullptr;
-  float *f32 = nullptr;
-  int n_out = 0, n_in = 0;
-};
 
 struct NezavikLayer {
   enum Type { DELTA, CHANNEL_DELTA, PARALLEL } type = DELTA;
@@ -55,7 +46,6 @@ struct Nezavik final : gptoss_engine {
   float *embedding_f32 = nullptr, *positions_f32 = nullptr;
   int n_positions = 0;
   std::vector<NezavikLayer> layers;
-  std::vector<int> lengths;   // positions every slot's states hold
   // activations of a pass
   Shapes wide;
   float *in_rows = nullptr, *conv_rows = nullptr, *y_rows = nullptr, *low_out_rows = nullptr, *q_rows = nullptr;
@@ -66,7 +56,7 @@ struct Nezavik final : gptoss_engine {
   void *act_rows = nullptr, *low_rows = nullptr;
 
   int max_stretch(int) const override { return NEZAVIK_STRETCH; }
-  int check_segments(const std::vector<RowSeg> &segs) override;
+  int check_segments(const std::vector<RowSeg> &segs) override { return continue_slots(segs); }
   int forward_rows(const StepRows &r) override;
 
   int project_in(const NezavikLayer &w, int n);
@@ -92,15 +82,6 @@ int Nezavik::project_in(const NezavikLayer &w, int n) {
   if (w.ff) ranges[k++] = {w.up_col, ld_in, (bf16_t *)act_rows, ld_act, 1};   // the last columns
   if (w.low_width) ranges[k++] = {w.low_col, w.low_col + (w.low_width + 31) / 32 * 32, (bf16_t *)low_rows, ld_low, 0};
   return dense_gemm_mixed(t_rows, w.in.packed, in_rows, ranges, k, n, ld_in, w.in.n_in, stream);
-}
-
-// A recurrent state knows only its own position: a sequence goes on where it stopped, or starts over.
-int Nezavik::check_segments(const std::vector<RowSeg> &segs) {
-  for (const RowSeg &s : segs)
-    GPTOSS_REQUIRE(s.pos0 == 0 || s.pos0 == lengths[s.slot], GPTOSS_ERR_STATE,
-                   "step: slot %d holds %d positions and cannot continue at position %d", s.slot, lengths[s.slot], s.pos0);
-  for (const RowSeg &s : segs) lengths[s.slot] = s.pos0 + s.n;
-  return GPTOSS_OK;
 }
 
 int Nezavik::forward_rows(const StepRows &r) {
@@ -165,123 +146,6 @@ int Nezavik::forward_rows(const StepRows &r) {
 
 namespace {
 
-// ---- config.json ---------------------------------------------------------------------------------
-struct ConfigError {
-  int rc;
-};
-
-const Json &field(const Json &j, const char *key, Json::Type type) {
-  const Json *v = j.find(key);
-  if (!v || !v->is(type)) throw ConfigError{fail(GPTOSS_ERR_IO, "config.json: \"%s\" is missing or of the wrong type", key)};
-  return *v;
-}
-double number(const Json &j, const char *key) { return field(j, key, Json::NUMBER).number; }
-int size_of(const Json &j, const char *key) {
-  const double v = number(j, key);
-  if (!(v >= 1 && v <= (1 << 30) && v == floor(v)))
-    throw ConfigError{fail(GPTOSS_ERR_DIM, "config.json: \"%s\" must be a positive integer", key)};
-  return (int)v;
-}
-void require(bool ok, const char *what, int layer) {
-  if (!ok) throw ConfigError{fail(GPTOSS_ERR_DIM, "config.json: layer %d: %s", layer, what)};
-}
-
-int up32(int n) { return (n + 31) / 32 * 32; }
-int up64(int n) { return (n + 63) / 64 * 64; }
-
-// ---- weights -------------------------------------------------------------------------------------
-// A matrix assembled on the host from several tensors, its unused rows and columns zero.
-struct Loader {
-  Nezavik *e;
-  Builder &b;
-  const SafeTensors *st;   // nullptr: random weights
-  uint64_t seed;
-  uint64_t next_seed() { return seed += 0x9E3779B97F4A7C15ull; }
-
-  std::vector<float> host(const std::string &name, const std::vector<long long> &shape) {
-    std::vector<float> v;
-    const int rc = st->read(name, shape, &v);
-    if (rc != GPTOSS_OK) throw ConfigError{rc};
-    return v;
-  }
-  // fp32 vector on the device; random: N(mean, std)
-  float *vec(const std::string &name, const std::vector<long long> &shape, float mean, float std) {
-    size_t n = 1;
-    for (long long d : shape) n *= d;
-    if (!st) return b.upload_f32(nullptr, n, next_seed(), mean, std);
-    return b.upload_f32(host(name, shape).data(), n, 0, 0, 0);
-  }
-  struct Part {
-    std::string name;
-    int rows, cols, row0, col0;
-  };
-  Matrix matrix(int n_out, int n_in, const std::vector<Part> &parts) {
-    Matrix m;
-    m.n_out = n_out;
-    m.n_in = n_in;
-    std::vector<float> full;
-    if (st) {
-      full.assign((size_t)n_out * n_in, 0.f);
-      for (const Part &p : parts) {
-        const std::vector<float> v = host(p.name, {p.rows, p.cols});
-        for (int i = 0; i < p.rows; i++)
-          memcpy(&full[(size_t)(p.row0 + i) * n_in + p.col0], &v[(size_t)i * p.cols], sizeof(float) * p.cols);
-      }
-    }
-    if (e->precise()) m.f32 = b.upload_f32(full.data(), (size_t)n_out * n_in, 0, 0, 0);
-    else
-      m.packed = b.upload_matrices(st ? full.data() : nullptr, 1, n_out, n_in, true, 0, next_seed(), 1.f / sqrtf((float)n_in));
-    return m;
-  }
-  // a norm whose gain is a scalar, as the vector the norm kernels take (zero in the padding)
-  float *scalar_norm(const std::string &name) {
-    std::vector<float> v(e->hidden, 0.f);
-    const float g = st ? host(name, {})[0] : 1.f;
-    for (int i = 0; i < e->hidden_real; i++) v[i] = g;
-    float *d = b.alloc<float>(e->hidden);
-    if (b.ok()) b.hip(hipMemcpy(d, v.data(), sizeof(float) * v.size(), hipMemcpyHostToDevice), "H2D");
-    return d;
-  }
-  // a table whose rows are gathered
-  void table(const std::string &name, int n_rows, int cols, bf16_t **t, float **t_f32) {
-    std::vector<float> v;
-    if (st) v = host(name, {n_rows, cols});
-    if (e->precise()) *t_f32 = b.upload_f32(v.data(), v.size(), 0, 0, 0);
-    else {
-      const size_t n = (size_t)n_rows * cols;
-      *t = b.alloc<bf16_t>(n);
-      if (!st) {
-        if (b.ok()) b.check(run_synth_bf16(*t, n, next_seed(), 0.f, 1.f, e->stream));
-        return;
-      }
-      for (size_t o = 0; o < n && b.ok(); o += b.st.elems) {
-        const size_t c = std::min(b.st.elems, n - o);
-        int slot;
-        const float *src = b.stage_in(v.data() + o, c, &slot);
-        if (!b.ok()) break;
-        b.check(run_f32_to_bf16(src, *t + o, c, e->stream));
-        b.release(slot);
-      }
-    }
-  }
-  float *zeros(size_t n) {
-    float *d = b.alloc<float>(n);
-    if (b.ok()) b.hip(hipMemsetAsync(d, 0, n * sizeof(float), e->stream), "memset");
-    return d;
-  }
-};
-
-// Columns of the projected rows are handed out in the order they are asked for.
-struct Columns {
-  int used = 0;
-  int take(int n) {
-    const int o = used;
-    used += n;
-    return o;
-  }
-  void align() { used = up32(used); }
-};
-
 using Part = Loader::Part;
 
 void check_scan(const Scan &s, const ShortConv &c, int i) {
@@ -291,7 +155,7 @@ void check_scan(const Scan &s, const ShortConv &c, int i) {
 }
 
 void scan_state(Loader &ld, NezavikLayer &w, const std::string &p) {
-  Nezavik *e = ld.e;
+  gptoss_engine *e = ld.e;
   Scan &s = w.scan;
   s.state = ld.zeros((size_t)e->max_batch * scan_state_elems(s.heads, s.K, s.V));
   s.conv_state = ld.zeros((size_t)e->max_batch * (w.conv.taps - 1) * w.conv.channels);
@@ -380,7 +244,7 @@ void load_state_space(Loader &ld, NezavikLayer &w, const Json &mix, const std::s
 
 void load_window(Loader &ld, NezavikLayer &w, const Json &mix, const std::string &p, int i, Columns &cols,
                  std::vector<Part> &parts) {
-  Nezavik *e = ld.e;
+  gptoss_engine *e = ld.e;
   WindowAttn &a = w.attn;
   a.heads = size_of(mix, "heads");
   a.kv_heads = size_of(mix, "kv_heads");
@@ -399,24 +263,11 @@ void load_window(Loader &ld, NezavikLayer &w, const Json &mix, const std::string
   parts.push_back({p + ".v", a.kv_heads * a.vdim, e->hidden_real, a.v_col, 0});
   a.q_norm = ld.vec(p + ".q.norm", {a.dim}, 1.f, 0.02f);
   a.k_norm = ld.vec(p + ".k.norm", {a.dim}, 1.f, 0.02f);
-  const long long stretch = std::min(e->max_seq, NEZAVIK_STRETCH);
-  a.cap = (int)std::min<long long>((e->max_seq + 63) / 64 * 64, (a.window - 1 + stretch + 63) / 64 * 64);
-  const size_t slots = (size_t)e->max_batch * a.cap * a.kv_heads;
-  if (e->precise()) {
-    a.k32 = ld.zeros(slots * a.dim);
-    a.v32 = ld.zeros(slots * a.vdim);
-  } else {
-    // slots that were never written are masked, but must hold finite values
-    a.kv = (bf16_t *)ld.zeros(slots / KV_BLOCK * a.block_elems() / 2);
-  }
-  const int tr = window_attn_tile_rows(a.heads, a.kv_heads);
-  auto at = std::find(e->tile_rows.begin(), e->tile_rows.end(), tr);
-  a.tiles = (int)(at - e->tile_rows.begin());
-  if (at == e->tile_rows.end()) e->tile_rows.push_back(tr);
+  window_attn_cache(ld, a, NEZAVIK_STRETCH);
 }
 
 void load_layer(Loader &ld, NezavikLayer &w, const Json &j, int i) {
-  Nezavik *e = ld.e;
+  Nezavik *e = static_cast<Nezavik *>(ld.e);
   const int W = e->hidden_real;
   const std::string l = "l" + std::to_string(i), p = l + ".mix";
   const std::string &type = field(j, "type", Json::STRING).text;
@@ -508,20 +359,15 @@ void load_model(Nezavik *e, Builder &b, const ModelSource &src, uint64_t seed) {
   Loader ld{e, b, src.weights, seed * 1000003ull + 29};
   const Json &list = field(cfg, "layers", Json::ARRAY);
   const int V = e->vocab, W = e->hidden_real;
-  ld.table("embed", V, W, &e->embedding, &e->embedding_f32);
-  ld.table("pos", e->n_positions, W, &e->positions, &e->positions_f32);
+  ld.table("embed", V, W, W, 1.f, &e->embedding, &e->embedding_f32);
+  ld.table("pos", e->n_positions, W, W, 1.f, &e->positions, &e->positions_f32);
   e->layers.resize(list.items.size());
   for (size_t i = 0; i < list.items.size() && b.ok(); i++) load_layer(ld, e->layers[i], list.items[i], (int)i);
   e->final_norm = ld.scalar_norm("final.norm");
   const Matrix head = ld.matrix(e->vocab_rows, e->hidden, {{"head", V, W, 0, 0}});
   e->unembedding = head.packed;
   e->unembedding_f32 = head.f32;
-  if (e->vocab_rows != V) {
-    std::vector<float> bias(e->vocab_rows, 0.f);
-    for (int v = V; v < e->vocab_rows; v++) bias[v] = -3.0e38f;   // never the arg-max
-    e->class_bias = b.alloc<float>(bias.size());
-    if (b.ok()) b.hip(hipMemcpy(e->class_bias, bias.data(), sizeof(float) * bias.size(), hipMemcpyHostToDevice), "H2D");
-  }
+  e->class_bias = ld.class_bias();
 }
 
 // largest matrix of the model in elements (the staging buffers hold one), from the configuration alone

@@ -9,42 +9,56 @@
 
 namespace gptoss {
 
+// A token's experts in ascending order: their rows of y2 and their weights.
+template <int KMAX>
+struct TokenExperts {
+  int rows[KMAX];
+  float w[KMAX];
+  __device__ __forceinline__ void load(const float *__restrict__ topk_w, const int *__restrict__ inv_perm, int b, int k) {
+#pragma unroll
+    for (int s = 0; s < KMAX; s++) {
+      rows[s] = (s < k) ? inv_perm[(size_t)b * k + s] : 0x7fffffff;
+      w[s] = (s < k) ? topk_w[(size_t)b * k + s] : 0.f;
+    }
+    // sorted position grows with expert id, so ordering by row orders by expert
+#pragma unroll
+    for (int i = 0; i < KMAX; i++)
+#pragma unroll
+      for (int j = 0; j + 1 < KMAX - i; j++)
+        if (rows[j] > rows[j + 1]) {
+          int tr = rows[j]; rows[j] = rows[j + 1]; rows[j + 1] = tr;
+          float tw = w[j]; w[j] = w[j + 1]; w[j + 1] = tw;
+        }
+  }
+  __device__ __forceinline__ f32x4 sum(const float *__restrict__ y2, int H, int h, int k) const {
+    f32x4 agg = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < KMAX; s++) {
+      if (s < k) {
+        const f32x4 v = *reinterpret_cast<const f32x4 *>(y2 + (size_t)rows[s] * H + h);
+#pragma unroll
+        for (int q = 0; q < 4; q++) agg[q] = __fadd_rn(agg[q], __fmul_rn(v[q], w[s]));
+      }
+    }
+    return agg;
+  }
+};
+
 // Weighted combine: out[b,:] (+)= sum over the token's k experts, in ascending expert order (the
 // order of the reference CPU loop, run.cpp:642-704), of w * y2[row of that pair].  Products and
 // sums are rounded separately, as that loop rounds them.
-template <int VPT>  // float4 chunks per thread: rows of at most 1024 * VPT floats (0: any length, a loop)
+// KMAX: room for a token's experts.
+template <int VPT, int KMAX = 8>  // float4 chunks per thread: rows of at most 1024 * VPT floats (0: any length, a loop)
 __global__ __launch_bounds__(256) void combine_kernel(const float *__restrict__ y2,
                                                       const float *__restrict__ topk_w,
                                                       const int *__restrict__ inv_perm,
                                                       float *__restrict__ out, int H, int k,
                                                       int accumulate) {
   const int b = blockIdx.x;
-  int rows[8];
-  float w[8];
-#pragma unroll
-  for (int s = 0; s < 8; s++) {
-    rows[s] = (s < k) ? inv_perm[(size_t)b * k + s] : 0x7fffffff;
-    w[s] = (s < k) ? topk_w[(size_t)b * k + s] : 0.f;
-  }
-  // sorted position grows with expert id, so ordering by row orders by expert
-#pragma unroll
-  for (int i = 0; i < 8; i++)
-#pragma unroll
-    for (int j = 0; j + 1 < 8 - i; j++)
-      if (rows[j] > rows[j + 1]) {
-        int tr = rows[j]; rows[j] = rows[j + 1]; rows[j + 1] = tr;
-        float tw = w[j]; w[j] = w[j + 1]; w[j + 1] = tw;
-      }
+  TokenExperts<KMAX> x;
+  x.load(topk_w, inv_perm, b, k);
   auto chunk = [&](int h) {
-    f32x4 agg = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int s = 0; s < 8; s++) {
-      if (s < k) {
-        f32x4 v = *reinterpret_cast<const f32x4 *>(y2 + (size_t)rows[s] * H + h);
-#pragma unroll
-        for (int q = 0; q < 4; q++) agg[q] = __fadd_rn(agg[q], __fmul_rn(v[q], w[s]));
-      }
-    }
+    f32x4 agg = x.sum(y2, H, h, k);
     f32x4 *op = reinterpret_cast<f32x4 *>(out + (size_t)b * H + h);
     if (accumulate) {
       f32x4 prev = *op;
@@ -79,21 +93,8 @@ __global__ __launch_bounds__(256) void combine_norm_kernel(const float *__restri
                                                            bf16_t *__restrict__ t_bf16) {
   __shared__ double red[4];
   const int b = blockIdx.x;
-  int rows[8];
-  float w[8];
-#pragma unroll
-  for (int s = 0; s < 8; s++) {
-    rows[s] = (s < k) ? inv_perm[(size_t)b * k + s] : 0x7fffffff;
-    w[s] = (s < k) ? topk_w[(size_t)b * k + s] : 0.f;
-  }
-#pragma unroll
-  for (int i = 0; i < 8; i++)
-#pragma unroll
-    for (int j = 0; j + 1 < 8 - i; j++)
-      if (rows[j] > rows[j + 1]) {
-        int tr = rows[j]; rows[j] = rows[j + 1]; rows[j + 1] = tr;
-        float tw = w[j]; w[j] = w[j + 1]; w[j + 1] = tw;
-      }
+  TokenExperts<8> x;
+  x.load(topk_w, inv_perm, b, k);
   f32x4 v[VPT];
   double ss = 0.0;
 #pragma unroll
@@ -101,15 +102,7 @@ __global__ __launch_bounds__(256) void combine_norm_kernel(const float *__restri
     const int h = (threadIdx.x + 256 * i) * 4;
     v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (h < H) {
-      f32x4 agg = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int s = 0; s < 8; s++) {
-        if (s < k) {
-          const f32x4 y = *reinterpret_cast<const f32x4 *>(y2 + (size_t)rows[s] * H + h);
-#pragma unroll
-          for (int q = 0; q < 4; q++) agg[q] = __fadd_rn(agg[q], __fmul_rn(y[q], w[s]));
-        }
-      }
+      const f32x4 agg = x.sum(y2, H, h, k);
       f32x4 *op = reinterpret_cast<f32x4 *>(out + (size_t)b * H + h);
       const f32x4 prev = *op;
 #pragma unroll
@@ -138,6 +131,31 @@ __global__ __launch_bounds__(256) void combine_norm_kernel(const float *__restri
           u32x2{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
     }
   }
+}
+
+// The combine into the residual stream followed by a dynamic tanh norm of the updated row, element by element.
+template <int KMAX>
+__global__ __launch_bounds__(256) void combine_tanh_norm_kernel(const float *__restrict__ y2,
+                                                                const float *__restrict__ topk_w,
+                                                                const int *__restrict__ inv_perm,
+                                                                float *__restrict__ out, int H, int k, TanhNorm norm,
+                                                                bf16_t *__restrict__ t_bf16) {
+  const int b = blockIdx.x, h = (blockIdx.y * 256 + threadIdx.x) * 4;
+  TokenExperts<KMAX> x;
+  x.load(topk_w, inv_perm, b, k);
+  if (h >= H) return;
+  const f32x4 agg = x.sum(y2, H, h, k);
+  f32x4 *op = reinterpret_cast<f32x4 *>(out + (size_t)b * H + h);
+  const f32x4 prev = *op, w = *reinterpret_cast<const f32x4 *>(norm.weight + h),
+              c = *reinterpret_cast<const f32x4 *>(norm.bias + h);
+  f32x4 v, o;
+#pragma unroll
+  for (int q = 0; q < 4; q++) {
+    v[q] = __fadd_rn(prev[q], agg[q]);
+    o[q] = fmaf(tanhf(norm.alpha * v[q]), w[q], c[q]);
+  }
+  *op = v;
+  *reinterpret_cast<u32x2 *>(t_bf16 + (size_t)b * H + h) = u32x2{pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3])};
 }
 
 // MXFP4 repack: blocks [n_out, n_in/2] (low nibble = even element) and e8m0 scales [n_out, n_in/32]
@@ -177,22 +195,23 @@ __global__ __launch_bounds__(256) void pack_mxfp4_kernel(const unsigned char *__
 
 // Host-side dispatcher used by the MoE layer.  rows_per_tile selects the kernel.
 template <int MBMAX, bool GATHER, int EPI, bool FP4>
-int launch_gemm(const GemmParams &p, int max_tiles, hipStream_t s);  // gemm_gather_bf16.hip, gemm_mxfp4.hip
+int launch_gemm(const GemmParams &p, int max_tiles, hipStream_t s);  // gemm_gather_bf16.hip
 
-template <bool GATHER, int EPI, bool FP4>
+int (*run_gemm_mxfp4)(const GemmParams &p, bool gather, int epi, int rows_per_tile, int max_tiles, hipStream_t s) = nullptr;
+
+template <bool GATHER, int EPI>
 static int dispatch_rows(const GemmParams &p, int rows_per_tile, int max_tiles, hipStream_t s) {
   switch (rows_per_tile) {
-    case 32: return launch_gemm<1, GATHER, EPI, FP4>(p, max_tiles, s);
-    case 64: return launch_gemm<2, GATHER, EPI, FP4>(p, max_tiles, s);
-    case 96: return launch_gemm<3, GATHER, EPI, FP4>(p, max_tiles, s);
-    case 128: return launch_gemm<4, GATHER, EPI, FP4>(p, max_tiles, s);
-    case 160: return launch_gemm<5, GATHER, EPI, FP4>(p, max_tiles, s);
+    case 32: return launch_gemm<1, GATHER, EPI, false>(p, max_tiles, s);
+    case 64: return launch_gemm<2, GATHER, EPI, false>(p, max_tiles, s);
+    case 96: return launch_gemm<3, GATHER, EPI, false>(p, max_tiles, s);
+    case 128: return launch_gemm<4, GATHER, EPI, false>(p, max_tiles, s);
+    case 160: return launch_gemm<5, GATHER, EPI, false>(p, max_tiles, s);
   }
   return fail(GPTOSS_ERR_DIM, "run_gemm: unsupported rows_per_tile %d", rows_per_tile);
 }
 
 hipError_t gemm_set_attrs_gather_bf16();  // gemm_gather_bf16.hip
-hipError_t gemm_set_attrs_mxfp4();        // gemm_mxfp4.hip
 
 // Raises the dynamic-LDS limit of every grouped GEMM kernel on the calling thread's current device, the
 // first time that device launches one.
@@ -206,7 +225,6 @@ static int gemm_prepare_device() {
   std::lock_guard<std::mutex> lock(mu);
   if (!done[dev]) {
     GPTOSS_HIP(gemm_set_attrs_gather_bf16());
-    GPTOSS_HIP(gemm_set_attrs_mxfp4());
     done[dev] = true;
   }
   return GPTOSS_OK;
@@ -223,20 +241,31 @@ int run_gemm(const GemmParams &p, bool gather, int epi, int rows_per_tile, int m
     GPTOSS_REQUIRE(gather && epi == EPI_SWIGLU, GPTOSS_ERR_DIM, "run_gemm: no 256-row tiles for this form (epi=%d)", epi);
     return run_gemm_tall_gather(p, max_tiles, max_rows, s);
   }
+  if (p.w_mxfp4) {
+    GPTOSS_REQUIRE(run_gemm_mxfp4, GPTOSS_ERR_STATE, "run_gemm: this library was linked without the MXFP4 kernels");
+    return run_gemm_mxfp4(p, gather, epi, rows_per_tile, max_tiles, s);
+  }
   int prc = gemm_prepare_device();
   if (prc != GPTOSS_OK) return prc;
-  if (gather && epi == EPI_SWIGLU)
-    return p.w_mxfp4 ? dispatch_rows<true, EPI_SWIGLU, true>(p, rows_per_tile, max_tiles, s)
-                     : dispatch_rows<true, EPI_SWIGLU, false>(p, rows_per_tile, max_tiles, s);
-  if (!gather && epi == EPI_F32) return dispatch_rows<false, EPI_F32, true>(p, rows_per_tile, max_tiles, s);
+  if (gather && epi == EPI_SWIGLU) return dispatch_rows<true, EPI_SWIGLU>(p, rows_per_tile, max_tiles, s);
   return fail(GPTOSS_ERR_DIM, "run_gemm: unsupported combination (gather=%d epi=%d)", (int)gather, epi);
 }
 
 int run_combine(const float *y2, const float *topk_w, const int *inv_perm, float *out, int B, int H,
-                int k, int accumulate, const float *norm_w, bf16_t *norm_out, hipStream_t s) {
+                int k, int accumulate, const float *norm_w, bf16_t *norm_out, hipStream_t s,
+                const TanhNorm *tanh_norm) {
   if (B == 0) return GPTOSS_OK;
+  if (tanh_norm && tanh_norm->weight) {
+    GPTOSS_REQUIRE(accumulate && norm_out && H % 4 == 0, GPTOSS_ERR_DIM, "combine: the tanh norm follows an accumulation");
+    TraceScope ts("combine_tanh_norm", s);
+    const dim3 grid(B, cdiv(H, 1024));
+    if (k <= 8) combine_tanh_norm_kernel<8><<<grid, 256, 0, s>>>(y2, topk_w, inv_perm, out, H, k, *tanh_norm, norm_out);
+    else combine_tanh_norm_kernel<MOE_MAX_TOP><<<grid, 256, 0, s>>>(y2, topk_w, inv_perm, out, H, k, *tanh_norm, norm_out);
+    GPTOSS_LAUNCH_CHECK("combine_tanh_norm_kernel");
+    return GPTOSS_OK;
+  }
   // out += combine, then norm_out = RMSNorm(out) * norm_w in the same kernel, when asked for
-  if (norm_w && norm_out && accumulate && H % 4 == 0 && H <= 4096 && aligned(norm_w, 16) && aligned(norm_out, 8)) {
+  if (norm_w && norm_out && accumulate && k <= 8 && H % 4 == 0 && H <= 4096 && aligned(norm_w, 16) && aligned(norm_out, 8)) {
     TraceScope ts("combine_rmsnorm", s);
     if (H <= 1024) combine_norm_kernel<1><<<B, 256, 0, s>>>(y2, topk_w, inv_perm, out, H, k, norm_w, norm_out);
     else if (H <= 2048) combine_norm_kernel<2><<<B, 256, 0, s>>>(y2, topk_w, inv_perm, out, H, k, norm_w, norm_out);
@@ -247,7 +276,8 @@ int run_combine(const float *y2, const float *topk_w, const int *inv_perm, float
   }
   {
     TraceScope ts("combine", s);
-    if (H <= 3072 && H > 2048) combine_kernel<3><<<B, 256, 0, s>>>(y2, topk_w, inv_perm, out, H, k, accumulate);
+    if (k > 8) combine_kernel<0, MOE_MAX_TOP><<<B, 256, 0, s>>>(y2, topk_w, inv_perm, out, H, k, accumulate);
+    else if (H <= 3072 && H > 2048) combine_kernel<3><<<B, 256, 0, s>>>(y2, topk_w, inv_perm, out, H, k, accumulate);
     else if (H <= 1024) combine_kernel<1><<<B, 256, 0, s>>>(y2, topk_w, inv_perm, out, H, k, accumulate);
     else combine_kernel<0><<<B, 256, 0, s>>>(y2, topk_w, inv_perm, out, H, k, accumulate);
   }

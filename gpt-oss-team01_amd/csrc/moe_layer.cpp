@@ -85,12 +85,12 @@ constexpr int MOE_TILE_COST0_X2_BF16 = 32;
 constexpr int MOE_TILE_COST0_X2_MXFP4 = 10;
 
 static int check_moe(const gptoss_moe_weights *w, const void *t, int B, float *out, void *ws,
-                     size_t ws_bytes) {
+                     size_t ws_bytes, int max_top) {
   GPTOSS_REQUIRE(w && t && out, GPTOSS_ERR_NULL, "moe_forward: null pointer");
   GPTOSS_REQUIRE(w->w_router && w->w1 && w->w2, GPTOSS_ERR_NULL, "moe_forward: null weight pointer");
   const int E = w->n_experts, k = w->top_k, H = w->hidden, I = w->intermediate;
-  GPTOSS_REQUIRE(B >= 0 && E >= 1 && E <= 256 && k >= 1 && k <= 8 && k <= E, GPTOSS_ERR_DIM,
-                 "moe_forward: need 1 <= k <= min(8,E), E <= 256 (B=%d E=%d k=%d)", B, E, k);
+  GPTOSS_REQUIRE(B >= 0 && E >= 1 && E <= 256 && k >= 1 && k <= max_top && k <= E, GPTOSS_ERR_DIM,
+                 "moe_forward: need 1 <= k <= min(%d,E), E <= 256 (B=%d E=%d k=%d)", max_top, B, E, k);
   GPTOSS_REQUIRE(aligned(t, 16), GPTOSS_ERR_ALIGN, "moe_forward: t must be 16-byte aligned");
   GPTOSS_REQUIRE(H > 0 && I > 0 && H % 64 == 0 && I % 64 == 0, GPTOSS_ERR_DIM,
                  "moe_forward: need hidden %% 64 == 0 and intermediate %% 64 == 0 (H=%d I=%d)", H, I);
@@ -136,8 +136,9 @@ extern "C" int gptoss_moe_workspace_views(void *workspace, int B, int E, int k, 
 static int moe_forward_impl(const gptoss_moe_weights *w, const void *t, int B, float *out,
                             int accumulate, void *workspace, size_t workspace_bytes, void *stream,
                             int mxfp4, const float *norm_w = nullptr, bf16_t *norm_out = nullptr,
-                            const MoePreNorm *pre = nullptr) {
-  int rc = check_moe(w, t, B, out, workspace, workspace_bytes);
+                            const MoePreNorm *pre = nullptr, const GluForm *glu = nullptr,
+                            const TanhNorm *tanh_norm = nullptr) {
+  int rc = check_moe(w, t, B, out, workspace, workspace_bytes, glu ? MOE_MAX_TOP : 8);
   if (rc != GPTOSS_OK) return rc;
   if (B == 0) return GPTOSS_OK;
   const int E = w->n_experts, k = w->top_k, H = w->hidden, I = w->intermediate;
@@ -191,7 +192,8 @@ static int moe_forward_impl(const gptoss_moe_weights *w, const void *t, int B, f
   g1.N = 2 * I;
   g1.K = H;
   g1.n_col_tiles = gemm_col_tiles(2 * I);
-  g1.limit = w->swiglu_limit;
+  if (glu) g1.glu = *glu;
+  else g1.glu.limit = w->swiglu_limit;
   rc = run_gemm(g1, true, EPI_SWIGLU, rpt, max_tiles, s);
   if (rc != GPTOSS_OK) return rc;
 
@@ -210,13 +212,18 @@ static int moe_forward_impl(const gptoss_moe_weights *w, const void *t, int B, f
   rc = run_gemm(g2, false, EPI_F32, rpt, max_tiles, s);
   if (rc != GPTOSS_OK) return rc;
 
-  return run_combine(ws.y2, ws.topk_w, ws.inv_perm, out, B, H, k, accumulate, norm_w, norm_out, s);
+  return run_combine(ws.y2, ws.topk_w, ws.inv_perm, out, B, H, k, accumulate, norm_w, norm_out, s, tanh_norm);
 }
 
 int gptoss::moe_forward_norm(const gptoss_moe_weights *w, const void *t, int B, float *out, void *workspace,
                              size_t workspace_bytes, hipStream_t s, int mxfp4, const float *norm_w,
                              bf16_t *norm_out, const MoePreNorm *pre) {
   return moe_forward_impl(w, t, B, out, 1, workspace, workspace_bytes, s, mxfp4, norm_w, norm_out, pre);
+}
+
+int gptoss::moe_forward_glu(const gptoss_moe_weights *w, const GluForm &glu, const void *t, int B, float *out,
+                            void *workspace, size_t workspace_bytes, hipStream_t s, const TanhNorm &norm, bf16_t *norm_out) {
+  return moe_forward_impl(w, t, B, out, 1, workspace, workspace_bytes, s, 0, nullptr, norm_out, nullptr, &glu, &norm);
 }
 
 extern "C" int gptoss_moe_forward(const gptoss_moe_weights *w, const void *t, int B, float *out,

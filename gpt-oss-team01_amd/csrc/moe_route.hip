@@ -15,16 +15,16 @@ namespace gptoss {
 // softmax over the k picked values with exp in float and the sum and division in double
 // (run.cpp:319-337).  Every lane of the group must call; lane 0 of the group writes.
 // ------------------------------------------------------------------------------------------------
-template <int NJ>
+template <int NJ, int KMAX = 8>
 __device__ __forceinline__ void topk_softmax_group(const float (&v)[NJ], int sub, int E, int k,
                                                    bool live, float *__restrict__ w_out,
                                                    int *__restrict__ i_out) {
   uint32_t used = 0;
-  float pick_v[8];
-  int pick_i[8];
+  float pick_v[KMAX];
+  int pick_i[KMAX];
   constexpr int NONE = 0x7fffffff;
 #pragma unroll
-  for (int s = 0; s < 8; s++) {
+  for (int s = 0; s < KMAX; s++) {
     pick_v[s] = -INFINITY;
     pick_i[s] = 0;
     if (s < k) {
@@ -54,15 +54,15 @@ __device__ __forceinline__ void topk_softmax_group(const float (&v)[NJ], int sub
     }
   }
   if (live && sub == 0) {
-    float ex[8];
+    float ex[KMAX];
     double sum = 0.0;
 #pragma unroll
-    for (int s = 0; s < 8; s++) {
+    for (int s = 0; s < KMAX; s++) {
       ex[s] = (s < k) ? expf(pick_v[s] - pick_v[0]) : 0.f;
       sum += ex[s];
     }
 #pragma unroll
-    for (int s = 0; s < 8; s++) {
+    for (int s = 0; s < KMAX; s++) {
       if (s < k) {
         w_out[s] = (float)((double)ex[s] / sum);
         i_out[s] = pick_i[s];
@@ -217,7 +217,7 @@ __global__ __launch_bounds__(ROUTER_WAVES * 64) void router_gemm_kernel(
 // ------------------------------------------------------------------------------------------------
 // Stand-alone gating from logits in memory: 32 lanes per token, two tokens per wave.
 // ------------------------------------------------------------------------------------------------
-template <int NJ>
+template <int NJ, int KMAX = 8>
 __global__ __launch_bounds__(256) void topk_softmax_kernel(const float *__restrict__ logits, int B,
                                                            int E, int k, float *__restrict__ topk_w,
                                                            int *__restrict__ topk_i) {
@@ -232,7 +232,7 @@ __global__ __launch_bounds__(256) void topk_softmax_kernel(const float *__restri
     v[j] = (live && e < E) ? row[e] : -INFINITY;
   }
   const size_t o = (size_t)(live ? token : 0) * k;
-  topk_softmax_group<NJ>(v, sub, E, k, live, topk_w + o, topk_i + o);
+  topk_softmax_group<NJ, KMAX>(v, sub, E, k, live, topk_w + o, topk_i + o);
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -534,7 +534,8 @@ int run_topk_softmax(const float *logits, int B, int E, int k, float *topk_w, in
   dim3 grid(cdiv(B * 32, 256)), block(256);
   int nj = cdiv(E, 32);
   TraceScope ts("topk_softmax", s);
-  if (nj <= 1) topk_softmax_kernel<1><<<grid, block, 0, s>>>(logits, B, E, k, topk_w, topk_i);
+  if (k > 8) topk_softmax_kernel<8, MOE_MAX_TOP><<<grid, block, 0, s>>>(logits, B, E, k, topk_w, topk_i);
+  else if (nj <= 1) topk_softmax_kernel<1><<<grid, block, 0, s>>>(logits, B, E, k, topk_w, topk_i);
   else if (nj <= 2) topk_softmax_kernel<2><<<grid, block, 0, s>>>(logits, B, E, k, topk_w, topk_i);
   else if (nj <= 4) topk_softmax_kernel<4><<<grid, block, 0, s>>>(logits, B, E, k, topk_w, topk_i);
   else topk_softmax_kernel<8><<<grid, block, 0, s>>>(logits, B, E, k, topk_w, topk_i);
@@ -560,6 +561,10 @@ int run_router(const void *t, const void *w_router, const float *b_router, float
   const bf16_t *tp = (const bf16_t *)t, *wp = (const bf16_t *)w_router;
   int nb = cdiv(E, 16);
   const RouterNorm none{nullptr, nullptr, nullptr, nullptr};
+  if (topk_w && k > 8) {   // more experts per token than the fused gating holds
+    const int rc = run_router(t, w_router, b_router, logits, B, H, E, k, nullptr, nullptr, s);
+    return rc != GPTOSS_OK ? rc : run_topk_softmax(logits, B, E, k, topk_w, topk_i, s);
+  }
   TraceScope ts(topk_w ? "router_gemm_topk" : "router_gemm", s);
   if (nb <= 1) router_gemm_kernel<1, false><<<grid, block, 0, s>>>(tp, wp, b_router, logits, B, H, E, k, topk_w, topk_i, rows_per_wg, none);
   else if (nb <= 2) router_gemm_kernel<2, false><<<grid, block, 0, s>>>(tp, wp, b_router, logits, B, H, E, k, topk_w, topk_i, rows_per_wg, none);
@@ -676,8 +681,9 @@ static int moe_route_impl(const float *logits, int B, int E, int k, float *topk_
   GPTOSS_REQUIRE(expert_offsets, GPTOSS_ERR_NULL, "moe_route: null pointer");
   GPTOSS_REQUIRE(B <= 0 || ((logits || !gate) && topk_w && topk_i && sorted_pair_ids && inv_perm),
                  GPTOSS_ERR_NULL, "moe_route: null pointer");
-  GPTOSS_REQUIRE(E >= 1 && E <= 256 && k >= 1 && k <= 8 && k <= E && B >= 0, GPTOSS_ERR_DIM,
-                 "moe_route: need 1 <= k <= min(8,E), E <= 256 (B=%d E=%d k=%d)", B, E, k);
+  const int max_top = gate ? 8 : MOE_MAX_TOP;
+  GPTOSS_REQUIRE(E >= 1 && E <= 256 && k >= 1 && k <= max_top && k <= E && B >= 0, GPTOSS_ERR_DIM,
+                 "moe_route: need 1 <= k <= min(%d,E), E <= 256 (B=%d E=%d k=%d)", max_top, B, E, k);
   GPTOSS_REQUIRE((long long)B * k < (1ll << 30), GPTOSS_ERR_DIM, "moe_route: B*k too large");
   bool tile_ok = rows_per_tile >= 0 && rows_per_tile <= 256 && rows_per_tile % 32 == 0;
   GPTOSS_REQUIRE(tile_ok, GPTOSS_ERR_DIM, "moe_route: rows_per_tile must be 0 or a multiple of 32 up to 256");

@@ -143,20 +143,20 @@ __global__ __launch_bounds__(256) void precise_attn_kernel(const float *__restri
   }
 }
 
-// clamped SwiGLU of interleaved (gate, up) rows (run.cpp:664-686)
+// gated activation of interleaved (gate, up) rows (GPT-OSS: clamped SwiGLU, run.cpp:664-686)
 __global__ __launch_bounds__(256) void precise_swiglu_kernel(const float *__restrict__ mlp1,
-                                                             float *__restrict__ act, int I, float limit,
+                                                             float *__restrict__ act, int I, GluForm glu,
                                                              size_t total) {
   const size_t idx = (size_t)blockIdx.x * 256 + threadIdx.x;
   if (idx >= total) return;
   const size_t r = idx / I;
   const int j = (int)(idx - r * I);
   float val = mlp1[r * 2 * I + 2 * j], up = mlp1[r * 2 * I + 2 * j + 1];
-  if (val > limit) val = limit;
-  if (up > limit) up = limit;
-  if (up < -limit) up = -limit;
-  val = __fmul_rn(val, 1.0f / __fadd_rn(1.0f, expf(__fmul_rn(-1.702f, val))));
-  val = __fmul_rn(val, __fadd_rn(up, 1.0f));
+  if (val > glu.limit) val = glu.limit;
+  if (up > glu.limit) up = glu.limit;
+  if (up < -glu.limit) up = -glu.limit;
+  val = __fmul_rn(val, 1.0f / __fadd_rn(1.0f, expf(__fmul_rn(-glu.rate, val))));
+  val = __fmul_rn(val, __fadd_rn(up, glu.shift));
   act[idx] = val;
 }
 
@@ -167,7 +167,7 @@ __global__ __launch_bounds__(256) void precise_moe_agg_kernel(const float *__res
                                                               const int *__restrict__ topk_i,
                                                               float *__restrict__ x, int H, int k) {
   const int b = blockIdx.x;
-  int order[8];
+  int order[MOE_MAX_TOP];
   for (int s = 0; s < k; s++) order[s] = s;
   for (int a = 0; a < k; a++)
     for (int c = a + 1; c < k; c++)
@@ -194,10 +194,14 @@ __global__ __launch_bounds__(256) void precise_add_kernel(float *__restrict__ x,
 
 int precise_matmul(float *out, const float *x, const float *w, const float *bias, const int *mat_ids,
                    int rows, int n_in, int n_out, int x_row_div, hipStream_t s) {
-  if (rows == 0) return GPTOSS_OK;
-  dim3 grid(cdiv(n_out, 4), rows);
-  precise_matmul_kernel<<<grid, 256, 0, s>>>(out, x, w, bias, mat_ids, n_in, n_out, x_row_div);
-  GPTOSS_LAUNCH_CHECK("precise_matmul_kernel");
+  // rows in grid dimension y: at most 65535 at a time
+  const int most = 65535 / x_row_div * x_row_div;
+  for (int r0 = 0; r0 < rows; r0 += most) {
+    dim3 grid(cdiv(n_out, 4), rows - r0 < most ? rows - r0 : most);
+    precise_matmul_kernel<<<grid, 256, 0, s>>>(out + (size_t)r0 * n_out, x + (size_t)(r0 / x_row_div) * n_in, w, bias,
+                                               mat_ids ? mat_ids + r0 : nullptr, n_in, n_out, x_row_div);
+    GPTOSS_LAUNCH_CHECK("precise_matmul_kernel");
+  }
   return GPTOSS_OK;
 }
 
@@ -222,16 +226,17 @@ int precise_attn(const float *q, const float *kc, const float *vc, const float *
   return GPTOSS_OK;
 }
 
-int precise_swiglu(const float *mlp1, float *act, int rows, int I, float limit, hipStream_t s) {
+int precise_swiglu(const float *mlp1, float *act, int rows, int I, const GluForm &glu, hipStream_t s) {
   const size_t total = (size_t)rows * I;
   if (total == 0) return GPTOSS_OK;
-  precise_swiglu_kernel<<<(unsigned)((total + 255) / 256), 256, 0, s>>>(mlp1, act, I, limit, total);
+  precise_swiglu_kernel<<<(unsigned)((total + 255) / 256), 256, 0, s>>>(mlp1, act, I, glu, total);
   GPTOSS_LAUNCH_CHECK("precise_swiglu_kernel");
   return GPTOSS_OK;
 }
 
 int precise_moe_agg(const float *mlp2, const float *topk_w, const int *topk_i, float *x, int B, int H,
                     int k, hipStream_t s) {
+  GPTOSS_REQUIRE(k >= 1 && k <= MOE_MAX_TOP, GPTOSS_ERR_DIM, "moe: at most %d experts per token (%d)", MOE_MAX_TOP, k);
   precise_moe_agg_kernel<<<B, 256, 0, s>>>(mlp2, topk_w, topk_i, x, H, k);
   GPTOSS_LAUNCH_CHECK("precise_moe_agg_kernel");
   return GPTOSS_OK;

@@ -1,5 +1,6 @@
-// Recurrent mixers for gfx950: gated delta rules (one decay per head, or one per key channel) and the
-// state-space recurrence, with the short convolutions in front of them and the gated norms behind.
+// Recurrent mixers for gfx950: gated delta rules (one decay per head, or one per key channel), the
+// state-space recurrence and retention (a fixed decay per head, plain writes), with the short
+// convolutions in front of them and the gated norms behind.
 //
 // The recurrence of a head acts on a K x V state whose V columns are independent of each other, so a
 // column lives in 8 lanes of a wave (K / 8 rows each, in registers) and a wave owns 16 columns (8 where
@@ -174,7 +175,7 @@ struct ScanToken {
 template <int NI, int KIND, bool ONE, int CPL>
 __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restrict__ segs, int n_seg) {
   constexpr int KP = 32 * NI, TC = ONE ? 1 : SCAN_TOKENS;
-  constexpr bool CHANNEL = KIND == SCAN_CHANNEL_DELTA, SSM = KIND == SCAN_STATE_SPACE;
+  constexpr bool CHANNEL = KIND == SCAN_CHANNEL_DELTA, SSM = KIND == SCAN_STATE_SPACE, RET = KIND == SCAN_RETENTION;
   constexpr int COLS = 32 * CPL;
   constexpr int PIECES = (TC * KP / 4 + 255) / 256, VPIECES = (TC * COLS / 4 + 255) / 256;
   // one token more than is staged: the loop reads a token ahead
@@ -195,8 +196,9 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
   const int c0 = (unit - h * blocks) * COLS, cw = (wave * 8 + (lane >> 3)) * CPL;   // this lane's first column is c0 + cw
   const bool busy = c0 + wave * 8 * CPL < p.V;   // wave-uniform
   const int kh = h / (p.heads / p.key_heads);
-  const float rate = expf(p.a_log[h]);
-  const float bias = CHANNEL ? 0.f : p.dt_bias[h];
+  const float rate = RET ? 0.f : expf(p.a_log[h]);
+  const float bias = CHANNEL || RET ? 0.f : p.dt_bias[h];
+  const float fixed = RET ? p.head_decay[h] : 0.f;
   const float skip = SSM ? p.d_skip[h] : 0.f;
 
   f32x4 S[CPL][NI];
@@ -243,6 +245,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
       const int idx = tid + 256 * x, t = min(idx / (COLS / 4), T - 1), c = c0 + idx % (COLS / 4) * 4;
       rv[x] = load4(v_src + (first + t) * p.ld_conv, c, p.V);
     }
+    if (RET) return;
     const float *ir = p.in + (first + min(tid, T - 1)) * p.ld_in + h;
     if (!SSM) r_beta = ir[p.beta_col];
     if (!CHANNEL) r_decay = ir[p.decay_col];
@@ -269,7 +272,7 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
       if (TC * COLS / 4 % 256 == 0 || idx < TC * COLS / 4)
         *reinterpret_cast<f32x4 *>(&sv[0][0] + idx * 4) = rv[x];
     }
-    if (tid < TC) {
+    if (!RET && tid < TC) {
       if (SSM) {
         const float dt = softplus_f(r_decay + bias);
         s_decay[tid] = exp_f(-rate * dt);
@@ -290,8 +293,8 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
     }
 #pragma unroll
     for (int c = 0; c < CPL; c++) x.v[c] = sv[t][cw + c];
-    x.beta = s_beta[t];
-    if (!CHANNEL) x.decay = s_decay[t];
+    if (!RET) x.beta = s_beta[t];
+    if (!CHANNEL && !RET) x.decay = s_decay[t];
   };
   auto advance = [&](const Token &x, float (&o)[CPL]) {
 #pragma unroll
@@ -299,11 +302,13 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
 #pragma unroll
       for (int i = 0; i < NI; i++)
 #pragma unroll
-        for (int e = 0; e < 4; e++) S[c][i][e] *= CHANNEL ? x.g[CHANNEL ? i : 0][e] : x.decay;
+        for (int e = 0; e < 4; e++) S[c][i][e] *= CHANNEL ? x.g[CHANNEL ? i : 0][e] : RET ? fixed : x.decay;
     float u[CPL];
 #pragma unroll
     for (int c = 0; c < CPL; c++) {
-      if constexpr (SSM) {
+      if constexpr (RET) {
+        u[c] = p.value_scale * x.v[c];
+      } else if constexpr (SSM) {
         u[c] = x.beta * x.v[c];
       } else {
         float d0 = 0.f, d1 = 0.f;
@@ -412,7 +417,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNorm g) {
   if (group >= g.groups) return;
   const float *y = g.y + (size_t)row * g.ld_y + group * g.size;
   const float *gate = g.gate + (size_t)row * g.ld_gate + group * g.size;
-  const float *w = g.weight + (g.weight_per_group ? group * g.size : 0);
+  const float *w = g.weight ? g.weight + (g.weight_per_group ? group * g.size : 0) : nullptr;
   float ss = 0.f;
   for (int d = lane; d < g.size; d += 64) {
     const float v = gated_value(g, y[d], gate[d]);
@@ -421,7 +426,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(GatedNorm g) {
   const float inv = 1.f / sqrtf(wave_sum_f(ss) / g.size + g.eps);
   OUT *out = (OUT *)g.out + (size_t)row * g.ld_out + g.out_col + group * g.size;
   for (int d = lane; d < g.size; d += 64) {
-    float v = gated_value(g, y[d], gate[d]) * inv * w[d];
+    float v = gated_value(g, y[d], gate[d]) * inv * (w ? w[d] : 1.f);
     if (!g.gate_first) v *= g.sigmoid_gate ? sigmoid_f(gate[d]) : silu_f(gate[d]);
     v *= g.scale;
     if constexpr (sizeof(OUT) == 2) out[d] = f32_to_bf16(v);
@@ -438,7 +443,7 @@ __global__ __launch_bounds__(256) void gated_norm_vec_kernel(GatedNorm g) {
   const bool live = group < g.groups;
   const int at = (live ? group : 0) * g.size;
   const float *y = g.y + (size_t)row * g.ld_y + at, *gate = g.gate + (size_t)row * g.ld_gate + at;
-  const float *w = g.weight + (g.weight_per_group ? at : 0);
+  const float *w = g.weight ? g.weight + (g.weight_per_group ? at : 0) : nullptr;
   f32x4 v[VPT], z[VPT];
   float ss = 0.f;
 #pragma unroll
@@ -466,7 +471,7 @@ __global__ __launch_bounds__(256) void gated_norm_vec_kernel(GatedNorm g) {
   for (int i = 0; i < VPT; i++) {
     const int d = (l + LANES * i) * 4;
     if (d < g.size) {
-      const f32x4 wv = *reinterpret_cast<const f32x4 *>(w + d);
+      const f32x4 wv = w ? *reinterpret_cast<const f32x4 *>(w + d) : f32x4{1.f, 1.f, 1.f, 1.f};
       f32x4 o;
 #pragma unroll
       for (int e = 0; e < 4; e++) {
@@ -517,7 +522,7 @@ int run_short_conv(const ShortConv &c, const StepRows &r, const float *in, int l
 
 template <int NI, int KIND>
 static void launch_scan_kind(const Scan &p, const StepRows &r, hipStream_t s) {
-  auto grid = [&](int cols) { return dim3((unsigned)(r.n_seg * (p.heads + 1) * cdiv(p.V, cols))); };
+  auto grid = [&](int cols) { return dim3((unsigned)(r.n_seg * (p.heads + (KIND == SCAN_RETENTION ? 0 : 1)) * cdiv(p.V, cols))); };
   // stretches of few heads and sequences: with two columns per lane half of the chip would be idle
   const bool few = (long long)r.n_seg * p.heads * cdiv(p.V, 64) <= 128;
   if (r.longest == 1) scan_kernel<NI, KIND, true, 2><<<grid(64), 256, 0, s>>>(p, r.segs, r.n_seg);
@@ -531,6 +536,7 @@ static void launch_scan(const Scan &p, const StepRows &r, hipStream_t s) {
     case SCAN_DELTA: launch_scan_kind<NI, SCAN_DELTA>(p, r, s); break;
     case SCAN_CHANNEL_DELTA: launch_scan_kind<NI, SCAN_CHANNEL_DELTA>(p, r, s); break;
     case SCAN_STATE_SPACE: launch_scan_kind<NI, SCAN_STATE_SPACE>(p, r, s); break;
+    case SCAN_RETENTION: launch_scan_kind<NI, SCAN_RETENTION>(p, r, s); break;
   }
 }
 
@@ -544,7 +550,7 @@ int run_scan(const Scan &scan, const StepRows &r, hipStream_t s) {
                  p.key_heads);
   GPTOSS_REQUIRE((long long)r.n_seg * (p.heads + 1) * cdiv(p.V, 32) < (1ll << 31), GPTOSS_ERR_DIM,
                  "scan: too many workgroups");
-  static const char *names[] = {"scan_delta", "scan_channel_delta", "scan_state_space"};
+  static const char *names[] = {"scan_delta", "scan_channel_delta", "scan_state_space", "scan_retention"};
   TraceScope ts(names[p.kind], s);
   switch (scan_key_pad(p.K) / 32) {
     case 1: launch_scan<1>(p, r, s); break;

@@ -1,5 +1,5 @@
 // Internal interface of the recurrent mixers (recurrent.hip): short causal convolution, the gated
-// delta rules and the state-space recurrence, and their gated output norms.
+// delta rules, the state-space recurrence and retention, and their gated output norms.
 #pragma once
 #include "engine.hpp"
 
@@ -20,7 +20,7 @@ struct ShortConv {
 int run_short_conv(const ShortConv &c, const StepRows &r, const float *in, int ld_in, const float *state,
                    float *out, int ld_out, hipStream_t s);
 
-enum ScanKind { SCAN_DELTA = 0, SCAN_CHANNEL_DELTA = 1, SCAN_STATE_SPACE = 2 };
+enum ScanKind { SCAN_DELTA = 0, SCAN_CHANNEL_DELTA = 1, SCAN_STATE_SPACE = 2, SCAN_RETENTION = 3 };
 constexpr int SCAN_MAX_KEY = 256;   // largest key (state) dimension
 
 // One recurrence over the rows of a step, per sequence and head.  The state of a head is K x V
@@ -28,7 +28,7 @@ constexpr int SCAN_MAX_KEY = 256;   // largest key (state) dimension
 struct Scan {
   ScanKind kind = SCAN_DELTA;
   int heads = 0, key_heads = 0, K = 0, V = 0;
-  // columns of the convolved rows: queries and keys (C and B) per key head, values (x) per head
+  // columns of the convolved rows (retention: of rows that no convolution precedes): queries and keys (C and B) per key head, values (x) per head
   const float *conv = nullptr;
   int ld_conv = 0, q_col = 0, k_col = 0, v_col = 0;
   // columns of the projected rows: write strength (delta rules) and decay (step size)
@@ -37,6 +37,8 @@ struct Scan {
   const float *channel_decay = nullptr;  // [n, ld_decay]: heads x K (SCAN_CHANNEL_DELTA)
   int ld_decay = 0;
   const float *a_log = nullptr, *dt_bias = nullptr, *d_skip = nullptr;
+  const float *head_decay = nullptr;     // [heads] (SCAN_RETENTION): the decay itself
+  float value_scale = 1.f;               // of what is written (SCAN_RETENTION)
   float *state = nullptr;
   float *out = nullptr;   // [n, ld_out]: heads x V
   int ld_out = 0;
@@ -57,7 +59,7 @@ struct GatedNorm {
   int ld_gate = 0;
   int gate_first = 0;            // 1: y * silu(gate), then the norm; 0: the norm, then the gate
   int sigmoid_gate = 0;          // gate behind the norm: sigmoid instead of silu
-  const float *weight = nullptr; // [size], or [groups * size] with weight_per_group
+  const float *weight = nullptr; // [size], or [groups * size] with weight_per_group; nullptr: ones
   int weight_per_group = 0;
   float scale = 1.f, eps = 1e-5f;
   void *out = nullptr;           // bf16 (or fp32 with out_f32) [n, ld_out], from column out_col

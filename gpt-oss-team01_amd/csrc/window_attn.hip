@@ -1,5 +1,5 @@
-// Sliding-window attention over the rows of a step for gfx950: decoding rows and stretches of prompts,
-// any head sizes up to 256 (padded to multiples of 32 in the cache), grouped queries.
+// Attention over a sliding window or a chunk of the sequence, for the rows of a step on gfx950: decoding rows
+// and stretches of prompts, any head sizes up to 256 (padded to multiples of 32 in the cache), grouped queries.
 //
 // The arithmetic is that of the decode attention (attn_decode.hip): scores and outputs on the matrix
 // cores in transposed form, S^T = K Q^T and O^T += V^T P^T (16x16x32), K rows and V operands in 64-slot
@@ -16,6 +16,19 @@ namespace gptoss {
 constexpr float WNEG = -1.0e30f;
 
 // ---- norms and K/V store -------------------------------------------------------------------------
+// Places of one position's key and value elements in the cache: the block of its slot, then kv_k_elem /
+// kv_v_elem with rows of DK and DV.
+struct StorePlace {
+  bf16_t *blk;
+  int slot, DK, DV;
+  __device__ bf16_t *key(int d) const { return blk + (slot & 63) * DK + d; }
+  __device__ bf16_t *value(int d) const {
+    const int tt = slot & 31, within = tt & 15;
+    return blk + KV_BLOCK * DK + (((slot & 63) >> 5) * (DV >> 4) + (d >> 4)) * 512 +
+           ((within >> 2) * 16 + (d & 15)) * 8 + (tt >> 4) * 4 + (within & 3);
+  }
+};
+
 // One wave per (RT rows, head): query heads, key heads, value heads.
 template <bool F32, int RT>
 __global__ __launch_bounds__(256) void window_store_kernel(WindowAttn a, const int *__restrict__ slots,
@@ -78,22 +91,74 @@ __global__ __launch_bounds__(256) void window_store_kernel(WindowAttn a, const i
       for (int i = 0; i < PIECES; i++)
         if (lane + 64 * i < width) dst[lane + 64 * i] = v[i][r];
     } else {
-      bf16_t *blk = a.kv + ((size_t)(seq * G + head) * (a.cap >> 6) + (cslot >> 6)) * a.block_elems();
+      const StorePlace at{a.kv + ((size_t)(seq * G + head) * (a.cap >> 6) + (cslot >> 6)) * a.block_elems(), cslot, DK, DV};
 #pragma unroll
       for (int i = 0; i < PIECES; i++) {
         const int d = lane + 64 * i;
         if (is_v) {
-          // operand order of V^T behind the block's 64 key rows (kv_v_elem, value rows of vdim_pad)
-          if (d < DV) {
-            const int tt = cslot & 31, within = tt & 15;
-            const int e = (((cslot & 63) >> 5) * (DV >> 4) + (d >> 4)) * 512 + ((within >> 2) * 16 + (d & 15)) * 8 +
-                          (tt >> 4) * 4 + (within & 3);
-            blk[KV_BLOCK * DK + e] = f32_to_bf16(v[i][r]);
-          }
+          // operand order of V^T behind the block's 64 key rows
+          if (d < DV) *at.value(d) = f32_to_bf16(v[i][r]);
         } else if (d < DK) {
-          blk[(cslot & 63) * DK + d] = f32_to_bf16(v[i][r]);
+          *at.key(d) = f32_to_bf16(v[i][r]);
         }
       }
+    }
+  }
+}
+
+// Norm over all heads at once, rotation, K/V store: one workgroup per row.
+template <bool F32>
+__global__ __launch_bounds__(256) void window_store_row_kernel(WindowAttn a, const int *__restrict__ slots,
+                                                               const int *__restrict__ lens) {
+  __shared__ float red[2][4];
+  const int row = blockIdx.x, tid = threadIdx.x, H = a.heads, G = a.kv_heads, D = a.dim;
+  const float *q = a.in + (size_t)row * a.ld_in + a.q_col, *k = a.in + (size_t)row * a.ld_in + a.k_col;
+  float ss[2] = {0.f, 0.f};
+  for (int i = tid; i < H * D; i += 256) ss[0] = fmaf(q[i], q[i], ss[0]);
+  for (int i = tid; i < G * D; i += 256) ss[1] = fmaf(k[i], k[i], ss[1]);
+#pragma unroll
+  for (int x = 0; x < 2; x++) {
+#pragma unroll
+    for (int m = 32; m >= 1; m >>= 1) ss[x] += __shfl_xor(ss[x], m, 64);
+    if ((tid & 63) == 0) red[x][tid >> 6] = ss[x];
+  }
+  __syncthreads();
+  const float qi = 1.f / sqrtf((red[0][0] + red[0][1] + red[0][2] + red[0][3]) / (H * D) + a.eps);
+  const float ki = 1.f / sqrtf((red[1][0] + red[1][1] + red[1][2] + red[1][3]) / (G * D) + a.eps);
+  const int DK = F32 ? D : a.dim_pad(), DV = a.vdim_pad();
+  const int pos = lens[row] - 1, half = a.rot.table ? a.rot.dims >> 1 : 0, seq = slots[row], cslot = pos % a.cap;
+  const float2 *cs = reinterpret_cast<const float2 *>(a.rot.table) + (size_t)pos * half;
+  // element d of a head: normed, and turned with its partner
+  auto value = [&](const float *x, const float *w, float inv, int head, int d) {
+    const int at = head * D + d;
+    const float own = x[at] * inv * w[at];
+    if (d >= 2 * half) return own;
+    const bool second = a.rot.interleaved ? (d & 1) != 0 : d >= half;
+    const int i = a.rot.interleaved ? d >> 1 : second ? d - half : d;
+    const int pt = head * D + (a.rot.interleaved ? d ^ 1 : second ? i : i + half);
+    const float other = x[pt] * inv * w[pt];
+    const float2 c = cs[i];
+    return second ? own * c.x + other * c.y : own * c.x - other * c.y;
+  };
+  for (int i = tid; i < H * DK; i += 256) {
+    const int head = i / DK, d = i - head * DK;
+    a.q[(size_t)row * H * DK + i] = d < D ? value(q, a.q_norm, qi, head, d) : 0.f;
+  }
+  const float *v = a.in + (size_t)row * a.ld_in + a.v_col;
+  if constexpr (F32) {
+    float *kd = a.k32 + ((size_t)seq * a.cap + cslot) * G * D, *vd = a.v32 + ((size_t)seq * a.cap + cslot) * G * a.vdim;
+    for (int i = tid; i < G * D; i += 256) kd[i] = value(k, a.k_norm, ki, i / D, i % D);
+    for (int i = tid; i < G * a.vdim; i += 256) vd[i] = v[i];
+  } else {
+    for (int i = tid; i < G * DK; i += 256) {
+      const int g = i / DK, d = i - g * DK;
+      const StorePlace at{a.kv + ((size_t)(seq * G + g) * (a.cap >> 6) + (cslot >> 6)) * a.block_elems(), cslot, DK, DV};
+      *at.key(d) = f32_to_bf16(d < D ? value(k, a.k_norm, ki, g, d) : 0.f);
+    }
+    for (int i = tid; i < G * DV; i += 256) {
+      const int g = i / DV, d = i - g * DV;
+      const StorePlace at{a.kv + ((size_t)(seq * G + g) * (a.cap >> 6) + (cslot >> 6)) * a.block_elems(), cslot, DK, DV};
+      *at.value(d) = f32_to_bf16(d < a.vdim ? v[g * a.vdim + d] : 0.f);
     }
   }
 }
@@ -256,7 +321,7 @@ __global__ __launch_bounds__(256) void window_decode_kernel(WindowAttn a, const 
   const int hh = blockIdx.z * 16 + n;             // head within the group
   const bool live = hh < per;
   const int head = g * per + min(hh, per - 1);
-  const int hi = seg.pos0, lo = max(0, hi - a.window + 1);
+  const int hi = seg.pos0, lo = a.first(hi);
   float m = WNEG, l = 0.f;
   f32x4 o[DB];
 #pragma unroll
@@ -381,14 +446,14 @@ __global__ __launch_bounds__(256, DMAX > 128 ? 1 : 2) void window_tile_kernel(Wi
       qi[i] = q0 + wave * 32 + i * 16 + n;
       const int use = min(qi[i], queries - 1), r = use / per;
       hi[i] = seg.pos0 + r;
-      lo[i] = max(0, hi[i] - a.window + 1);
+      lo[i] = a.first(hi[i]);
       load_q<KS>(q[i], a.q + ((size_t)(seg.row0 + r) * a.heads + g * per + (use - r * per)) * DK, ks_n, c,
                  a.scale * 1.4426950408889634f);
 #pragma unroll
       for (int db = 0; db < DB; db++) o[i][db] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
     const int r_first = q0 / per, r_last = min(q0 + 127, queries - 1) / per;
-    const int b_lo = max(0, seg.pos0 + r_first - a.window + 1) >> 6, b_hi = (seg.pos0 + r_last) >> 6;
+    const int b_lo = a.first(seg.pos0 + r_first) >> 6, b_hi = (seg.pos0 + r_last) >> 6;
     const bool busy0 = q0 + wave * 32 < queries, busy1 = q0 + wave * 32 + 16 < queries;   // wave-uniform
     fetch(b_lo);
     for (int b = b_lo; b <= b_hi; b++) {
@@ -422,7 +487,7 @@ __global__ __launch_bounds__(256) void window_f32_kernel(WindowAttn a, const int
   __shared__ float sq[WINDOW_ATTN_MAX_DIM], sp[256], red[8];
   const int h = blockIdx.x, row = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int g = h / (a.heads / a.kv_heads);
-  const int hi = lens[row] - 1, lo = max(0, hi - a.window + 1);
+  const int hi = lens[row] - 1, lo = a.first(hi);
   const size_t base = (size_t)slots[row] * a.cap;
   if (tid < a.dim) sq[tid] = a.q[((size_t)row * a.heads + h) * a.dim + tid];
   __syncthreads();
@@ -470,11 +535,15 @@ int run_window_attn(const WindowAttn &a, const StepRows &r, hipStream_t s) {
                  WINDOW_ATTN_MAX_DIM, a.dim, a.vdim, a.heads, a.kv_heads, a.window);
   GPTOSS_REQUIRE(r.max_len <= a.cap || a.window - 1 + r.longest <= a.cap, GPTOSS_ERR_DIM,
                  "window_attn: a ring of %d slots cannot hold a window of %d and %d rows", a.cap, a.window, r.longest);
+  GPTOSS_REQUIRE(a.whole_norm || !a.rot.table, GPTOSS_ERR_DIM, "window_attn: rotation needs a norm over the whole projection");
+  GPTOSS_REQUIRE(!a.rot.table || (a.rot.dims >= 2 && a.rot.dims % 2 == 0 && a.rot.dims <= a.dim), GPTOSS_ERR_DIM,
+                 "window_attn: %d of %d dimensions rotated (an even number)", a.rot.dims, a.dim);
   const int units = a.heads + 2 * a.kv_heads;
   if (a.k32) {
     {
       TraceScope ts("window_store", s);
-      window_store_kernel<true, 1><<<dim3(cdiv(units, 4), r.n), 256, 0, s>>>(a, r.slots, r.lens, r.n);
+      if (a.whole_norm) window_store_row_kernel<true><<<r.n, 256, 0, s>>>(a, r.slots, r.lens);
+      else window_store_kernel<true, 1><<<dim3(cdiv(units, 4), r.n), 256, 0, s>>>(a, r.slots, r.lens, r.n);
     }
     GPTOSS_LAUNCH_CHECK("window_store_kernel");
     TraceScope ts("window_attn_f32", s);
@@ -484,7 +553,8 @@ int run_window_attn(const WindowAttn &a, const StepRows &r, hipStream_t s) {
   }
   {
     TraceScope ts("window_store", s);
-    if (r.n >= 1024) window_store_kernel<false, 4><<<dim3(cdiv(units, 4), cdiv(r.n, 4)), 256, 0, s>>>(a, r.slots, r.lens, r.n);
+    if (a.whole_norm) window_store_row_kernel<false><<<r.n, 256, 0, s>>>(a, r.slots, r.lens);
+    else if (r.n >= 1024) window_store_kernel<false, 4><<<dim3(cdiv(units, 4), cdiv(r.n, 4)), 256, 0, s>>>(a, r.slots, r.lens, r.n);
     else window_store_kernel<false, 1><<<dim3(cdiv(units, 4), r.n), 256, 0, s>>>(a, r.slots, r.lens, r.n);
   }
   GPTOSS_LAUNCH_CHECK("window_store_kernel");

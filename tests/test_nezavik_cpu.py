@@ -124,7 +124,7 @@ def test_registry_lists_the_model_classes(lib):
     while (n := lib.load().gptoss_model_name(i)) is not None:
         names.append(n.decode())
         i += 1
-    assert sorted(names) == ["Nezavik", "gpt-oss"]
+    assert sorted(names) == ["Netinex", "Nezavik", "gpt-oss"]
 
 
 def test_open_reports_what_is_wrong(lib, tmp_path):
