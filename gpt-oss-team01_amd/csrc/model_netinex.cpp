@@ -395,8 +395,9 @@ int open_netinex(const ModelSource &src, const OpenOptions &o, gptoss_engine **o
     e->hidden_real = size_of(cfg, "width");
     e->hidden = up64(e->hidden_real);
     e->norm_eps = (float)number(field(cfg, "norm", Json::OBJECT), "eps");
-    e->logit_softcap = (float)number(cfg, "logit_softcap");
-    if (!(e->logit_softcap > 0.f)) throw ConfigError{fail(GPTOSS_ERR_DIM, "config.json: \"logit_softcap\" must be positive")};
+    const Json *cap = cfg.find("logit_softcap");
+    if (cap && !cap->is(Json::NUL)) e->logit_softcap = (float)number(cfg, "logit_softcap");
+    if (!(e->logit_softcap >= 0.f)) throw ConfigError{fail(GPTOSS_ERR_DIM, "config.json: \"logit_softcap\" must not be negative")};
     e->n_layers = (int)field(cfg, "layers", Json::ARRAY).items.size();
     if (e->n_layers < 1) throw ConfigError{fail(GPTOSS_ERR_DIM, "config.json: no layers")};
     if (e->hidden > 16384) throw ConfigError{fail(GPTOSS_ERR_DIM, "config.json: widths above 16384 are not supported")};

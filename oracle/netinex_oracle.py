@@ -64,13 +64,13 @@ def frequencies(rot):
 def rotate(x, positions, rot, interleaved):
     """x [T, heads, dim]: the first rot.dims of every head; pairs (2i, 2i + 1), or (i, i + dims / 2)."""
     f, gain = frequencies(rot)
-    out, half = f64(x).copy(), rot["dims"] // 2
-    for t, p in enumerate(positions):
-        for i in range(half):
-            a, b = (2 * i, 2 * i + 1) if interleaved else (i, i + half)
-            c, s = gain * math.cos(p * f[i]), gain * math.sin(p * f[i])
-            u, v = f64(x)[t, :, a], f64(x)[t, :, b]
-            out[t, :, a], out[t, :, b] = u * c - v * s, v * c + u * s
+    x, half = f64(x), rot["dims"] // 2
+    out = x.copy()
+    for i in range(half):
+        a, b = (2 * i, 2 * i + 1) if interleaved else (i, i + half)
+        angle = np.asarray(positions)[:, None] * f[i]
+        c, s = gain * np.cos(angle), gain * np.sin(angle)
+        out[:, :, a], out[:, :, b] = x[:, :, a] * c - x[:, :, b] * s, x[:, :, b] * c + x[:, :, a] * s
     return out
 
 
@@ -136,8 +136,17 @@ def route(z, top):
     return ids, e / e.sum(axis=1, keepdims=True)
 
 
-def feed_forward(h, w, p, mlp, rnd=exact):
-    ids, share = route(linear(h, w[f"{p}.router"], rnd) + f64(w[f"{p}.router.b"]), mlp["router"]["top"])
+def margin(z, top):
+    """Distance of the last chosen logit from the first one that is not, per token."""
+    order = -np.sort(-z, axis=1)
+    return order[:, top - 1] - order[:, top] if top < z.shape[1] else np.full(len(z), np.inf)
+
+
+def feed_forward(h, w, p, mlp, rnd=exact, margins=None):
+    z = linear(h, w[f"{p}.router"], rnd) + f64(w[f"{p}.router.b"])
+    ids, share = route(z, mlp["router"]["top"])
+    if margins is not None:
+        margins.append(margin(z, mlp["router"]["top"]))
     y = np.zeros(h.shape)
     for t in range(len(h)):
         x = h[t:t + 1]
@@ -152,8 +161,9 @@ def _norm(x, w, name):
     return tanh_norm(x, w[name], w[name + ".b"], w[name + ".alpha"])
 
 
-def forward(cfg, w, tokens, want_layers=False, rnd=None):
-    """Logits [T, vocab] of one sequence from position 0 (and the residual stream after every layer)."""
+def forward(cfg, w, tokens, want_layers=False, rnd=None, margins=None):
+    """Logits [T, vocab] of one sequence from position 0 (and the residual stream after every layer).
+    margins: a list that receives every router's margins."""
     eps = cfg["norm"]["eps"]
     rounding = exact if rnd is None else rnd
     rnd = lambda x: f64(rounding(x)).reshape(np.shape(x))
@@ -161,7 +171,9 @@ def forward(cfg, w, tokens, want_layers=False, rnd=None):
     for i, layer in enumerate(cfg["layers"]):
         x = x + MIXERS[layer["type"]](_norm(x, w, f"l{i}.norm1"), w, f"l{i}.mix", layer["mixer"], eps, rnd)
         if layer.get("mlp") is not None:
-            x = x + feed_forward(_norm(x, w, f"l{i}.norm2"), w, f"l{i}.mlp", layer["mlp"], rnd)
+            x = x + feed_forward(_norm(x, w, f"l{i}.norm2"), w, f"l{i}.mlp", layer["mlp"], rnd, margins)
         after.append(x)
-    logits = softcap(linear(_norm(x, w, "final.norm"), w["embed"], rnd), cfg["logit_softcap"])
+    logits = linear(_norm(x, w, "final.norm"), w["embed"], rnd)
+    if cfg.get("logit_softcap"):
+        logits = softcap(logits, cfg["logit_softcap"])
     return (logits, after) if want_layers else logits

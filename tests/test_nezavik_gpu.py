@@ -16,6 +16,7 @@ import pytest
 
 from conftest import ROOT, load_pkg
 import nezavik_models as nm
+from engine_harness import feed, greedy, open_model, requests  # noqa: F401
 from oracle import nezavik_oracle as nz
 
 pytestmark = pytest.mark.gpu
@@ -23,32 +24,6 @@ pytestmark = pytest.mark.gpu
 TOL = {True: 2e-5, False: 3e-2}      # keyed by `precise`
 STAGED_TOL = 1e-2                    # bf16 against the restatement with bf16 inputs
 BOTH = pytest.mark.parametrize("precise", [True, False], ids=["fp32", "bf16"])
-
-
-@pytest.fixture
-def open_model(ops, tmp_path):
-    engines = []
-
-    def make(cfg, w, precise=True, max_batch=4, max_seq=0, **kw):
-        path = nm.save(str(tmp_path / f"m{len(engines)}"), cfg, w)
-        e = load_pkg("engine").Engine.open(path, max_batch=max_batch, max_seq=max_seq, precise=precise, **kw)
-        e.path = path
-        engines.append(e)
-        return e
-    yield make
-    for e in engines:
-        e.close()
-
-
-def feed(e, slot, tok, cuts=None, start=0):
-    """Logits of every position of one sequence, fed in portions of the sizes `cuts` (the last repeats)."""
-    out, at, i = [], 0, 0
-    cuts = cuts or [len(tok)]
-    while at < len(tok):
-        n = min(cuts[min(i, len(cuts) - 1)], len(tok) - at)
-        out.append(e.step_logits(tok[at:at + n], [slot] * n, np.arange(at, at + n) + start, np.arange(n)))
-        at, i = at + n, i + 1
-    return np.concatenate(out)
 
 
 def check(got, want, precise, factor=1.0):
@@ -359,23 +334,7 @@ def test_missing_and_misshapen_tensors_are_named(open_model, tmp_path):
 
 # ---- generation ----------------------------------------------------------------------------------
 def _greedy(cfg, w, prompt, total):
-    """Greedy ids and the smallest margin between the best two logits on the way."""
-    seq, margin = list(prompt), np.inf
-    while len(seq) < total:
-        lg = nz.forward(cfg, w, np.array(seq))[-1]
-        top = np.sort(lg)[-2:]
-        margin = min(margin, (top[1] - top[0]) / lg.std())
-        seq.append(int(lg.argmax()))
-    return seq[len(prompt):], margin
-
-
-def _requests(cfg):
-    prompts = [nm.tokens(cfg, n, 80 + n) for n in (5, 1, 23, 9, 40, 2, 17)]
-    n_prompt = np.array([len(p) for p in prompts], np.int32)
-    ids = np.zeros((len(prompts), n_prompt.max()), np.int32)
-    for i, p in enumerate(prompts):
-        ids[i, :len(p)] = p
-    return prompts, n_prompt, ids
+    return greedy(lambda seq: nz.forward(cfg, w, seq), prompt, total)
 
 
 def test_greedy_generation_through_the_scheduler(open_model):
@@ -383,7 +342,7 @@ def test_greedy_generation_through_the_scheduler(open_model):
     the ids it would get alone."""
     cfg = nm.config([nm.delta(heads=2), nm.parallel(window=7), nm.channel_delta()])
     w = nm.weights(cfg, 91)
-    prompts, n_prompt, ids = _requests(cfg)
+    prompts, n_prompt, ids = requests(cfg)
     limit = n_prompt + 13
     e = open_model(cfg, w, True, max_batch=3, max_seq=64)
     out, n = e.generate(ids, int(limit.max()), n_prompt=n_prompt, max_len=limit)
@@ -414,7 +373,7 @@ def test_bf16_generation_matches_its_own_logits(open_model):
     a second engine computes for the same sequences (vocabularies that are padded included)."""
     cfg = nm.config(MIXED, vocab=101)
     w = nm.weights(cfg, 92)
-    prompts, n_prompt, ids = _requests(cfg)
+    prompts, n_prompt, ids = requests(cfg)
     e = open_model(cfg, w, False, max_batch=3, max_seq=80, keep_logits=False)
     out, _ = e.generate(ids, 60, n_prompt=n_prompt)
     ref = open_model(cfg, w, False, max_batch=3, max_seq=80)
@@ -434,7 +393,7 @@ def test_command_line_generates_and_replays(open_model, tmp_path):
     cfg = nm.config([nm.delta(), nm.parallel(window=6)])
     w = nm.weights(cfg, 93)
     e = open_model(cfg, w, True, max_batch=2, max_seq=40)
-    prompts, n_prompt, ids = _requests(cfg)
+    prompts, n_prompt, ids = requests(cfg)
     out, _ = e.generate(ids[:3, :23], 23 + 9, n_prompt=n_prompt[:3], max_len=n_prompt[:3] + 8)
     cmd = [sys.executable, os.path.join(ROOT, "bin", "gptoss"), "generate", "--model", e.path, "--dtype", "float32",
            "--max-new", "8", "--batch", "2"]
