@@ -71,10 +71,10 @@ def parse():
     ap.add_argument("--mfma-rates", action="store_true",
                     help="only measure the register-fed issue rate of the bf16 and the scaled f8f6f4 MFMA "
                          "(gptoss_diag_mfma_rate) and print one JSON line of its own")
-    ap.add_argument("--model", choices=("gpt-oss", "nezavik"), default="gpt-oss",
-                    help="nezavik: only measure prefill and decode of the Nezavik model class at a few sizes, "
+    ap.add_argument("--model", choices=("gpt-oss", "nezavik", "netinex"), default="gpt-oss",
+                    help="nezavik, netinex: only measure prefill and decode of that model class at a few sizes, "
                          "beside GPT-OSS engines of the same width, and print one JSON line of its own")
-    ap.add_argument("--only", default="", help="with --model nezavik: sizes to run, with commas between them")
+    ap.add_argument("--only", default="", help="with --model nezavik or netinex: sizes to run, with commas between them")
     ap.add_argument("--no-sched", action="store_true", help="skip the scheduler leg of the end-to-end figure")
     return ap.parse_args()
 
@@ -634,7 +634,7 @@ def _gptoss_work(cfg, rows, seqs, contexts):
     D, nq, nkv, L = cfg.head_dim, cfg.n_attn_heads, cfg.n_kv_heads, cfg.n_layers
     qkv = (nq + 2 * nkv) * D
     work = {"gemm_f32": [0.0, 0.0], "gemm1_gather_swiglu": [0.0, 0.0], "attn": [0.0, 0.0], "rope_store": [0.0, 0.0],
-            "combine_rmsnorm": [0.0, 0.0]}
+            "combine_rmsnorm": [0.0, 0.0], "residual_rmsnorm": [0.0, 0.0]}
 
     def add(label, nbytes, flop=0.0):
         work[label][0] += nbytes
@@ -649,6 +649,7 @@ def _gptoss_work(cfg, rows, seqs, contexts):
         add("attn", seqs * ctx * nkv * D * 4 + rows * nq * D * 6, 4.0 * rows * ctx * nq * D)
         add("rope_store", rows * (qkv * 4 + nq * D * 4 + 2 * nkv * D * 2))
         add("combine_rmsnorm", rows * H * (k * 4 + 8 + 2))
+        add("residual_rmsnorm", rows * H * (4 + 8 + 2))
     work = {n: (b, f, MFMA_BF16_PEAK_TFLOPS) for n, (b, f) in work.items()}
     for n in ("attn_decode", "attn_prefill_tiles"):
         work[n] = work["attn"]
@@ -696,47 +697,143 @@ def _time_engine(ops, torch, eng, vocab, decode, prompt, steps):
     return res
 
 
-def bench_nezavik(ops, torch, steps, only):
+def netinex_config(width, heads, ff, experts, top, layers, attn_heads, kv_heads, chunk, vocab=65536):
+    """Layers in the proportions of a real model: retention with heads of 128 x 128 and attention with heads of 64
+    in turn, a mixture of experts behind each."""
+    decay = [1 - 2.0 ** -(5 + 7 * h / max(1, heads - 1)) for h in range(heads)]
+    ret = {"heads": heads, "dim": 128, "vdim": 128, "decay": decay, "rot": {"base": 10000.0, "dims": 128}}
+    att = {"heads": attn_heads, "kv_heads": kv_heads, "dim": 64, "vdim": 64, "scale": 0.125, "mask": {"size": chunk},
+           "rot": {"base": 150000.0, "dims": 64, "scaling": {"factor": 32.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    return {"architecture": "Netinex", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "layers": [{"type": t, "mixer": m, "mlp": mlp}
+                       for t, m in ((("retention", ret), ("attention", att))[i % 2] for i in range(layers))]}
+
+
+def _netinex_work(cfg, rows, seqs, context):
+    """As for Nezavik; the context is what a row sees of its chunk."""
+    W = cfg["width"]
+    work = {}
+
+    def add(label, nbytes, flop=0.0, peak=MFMA_BF16_PEAK_TFLOPS):
+        b, f, _ = work.get(label, (0.0, 0.0, peak))
+        work[label] = (b + nbytes, f + flop, peak)
+
+    def gemm(n_out, n_in):
+        add("gemm_f32", n_out * n_in * 2 + rows * (n_in * 2 + n_out * 4), 2.0 * rows * n_out * n_in)
+
+    add("residual_tanh_norm", rows * W * 6)
+    for layer in cfg["layers"]:
+        m, r, ff = layer["mixer"], layer["mlp"]["router"], layer["mlp"]["expert"]["ff"]
+        H = m["heads"]
+        if layer["type"] == "retention":
+            nk, nv = H * m["dim"], H * m["vdim"]
+            gemm(2 * nk + 2 * nv, W)
+            add("rotary", rows * 2 * H * m["rot"]["dims"] * 8)
+            # per state element and token: decay, update, read-out
+            add("scan_retention", seqs * nk * m["vdim"] * 8 + rows * (2 * nk + 2 * nv) * 4, 5.0 * rows * nk * m["vdim"],
+                VALU_FP32_PEAK_TFLOPS)
+            add("gated_norm", rows * nv * 10)
+        else:
+            nq, nk, nv = H * m["dim"], m["kv_heads"] * m["dim"], H * m["vdim"]
+            gemm(nq + nk, W)
+            add("window_store", rows * ((nq + nk) * 4 + nq * 4 + nk * 4))
+            add("window_decode" if rows == seqs else "window_tiles",
+                seqs * context * nk * 4 + rows * H * (m["dim"] * 4 + m["vdim"] * 2),
+                2.0 * rows * context * H * (m["dim"] + m["vdim"]))
+        gemm(W, nv)
+        add("residual_tanh_norm", rows * W * 14)
+        E, k = r["experts"], r["top"]
+        used = min(E, rows * k)
+        add("gemm1_gather_swiglu", used * 2 * ff * W * 2 + rows * W * 2 + rows * k * ff * 2, 4.0 * rows * k * W * ff)
+        add("gemm_f32", used * W * ff * 2 + rows * k * (ff * 2 + W * 4), 2.0 * rows * k * W * ff)
+        add("combine_tanh_norm", rows * W * (k * 4 + 8 + 2))
+    add("gemm_argmax", cfg["vocab"] * W * 2 + seqs * W * 2, 2.0 * seqs * cfg["vocab"] * W)
+    return work
+
+
+#: as NEZAVIK_SIZES; a decoding row sees about three quarters of its chunk
+NETINEX_SIZES = {
+    "width2048": (dict(width=2048, heads=16, ff=1024, experts=32, top=4, layers=8, attn_heads=32, kv_heads=8, chunk=512),
+                  (256, 1400), (8, 1024)),
+    "width4096": (dict(width=4096, heads=32, ff=2048, experts=32, top=4, layers=8, attn_heads=64, kv_heads=8, chunk=1024),
+                  (256, 1800), (4, 2048)),
+    "width4096_small_batch": (dict(width=4096, heads=32, ff=2048, experts=32, top=4, layers=8, attn_heads=64, kv_heads=8,
+                                   chunk=1024), (16, 1800), (1, 2048)),
+}
+
+
+def _bench_beside_gptoss(ops, torch, steps, who, cfg, works, other, shape, decode, prompt, window):
+    """One size of a model class and a GPT-OSS engine `other` in turn: throughput and kernels against rooflines.
+    works: of a decode step and of a prefill pass of the class."""
     import tempfile
+    (B, ctx), (Bp, T) = decode, prompt
+    positions = max(ctx + steps + 8, T)
+    seen = (window * (T - window) + window * (window + 1) / 2) / T if T > window else (T + 1) / 2
+    other_works = (_gptoss_work(other, B, B, (ctx, min(window, ctx))), _gptoss_work(other, Bp * T, Bp, ((T + 1) / 2, seen)))
+    with tempfile.TemporaryDirectory() as d:
+        with open(os.path.join(d, "config.json"), "w") as f:
+            json.dump(cfg, f)
+        eng = ops.Engine.open(d, max_batch=max(B, Bp), max_seq=positions, synthetic=True, keep_logits=False)
+    row = {}
+    for name, e, w in ((who, eng, works), ("gpt_oss", None, other_works)):
+        if e is None:
+            e = ops.Engine(other, None, max_batch=max(B, Bp), max_seq=positions, synthetic=True, keep_logits=False)
+        r = _time_engine(ops, torch, e, cfg["vocab"], decode, prompt, steps)
+        row[name] = {"decode_ms": round(r["decode"][0], 3), "decode_tok_s": round(B / r["decode"][0] * 1e3, 1),
+                     "prefill_ms": round(r["prefill"][0], 2), "prefill_tok_s": round(Bp * T / r["prefill"][0] * 1e3, 1),
+                     "device_gb": round(e.device_bytes() / 1e9, 2),
+                     "decode_kernels": _against_roofline(r["decode"][1], w[0]),
+                     "prefill_kernels": _against_roofline(r["prefill"][1], w[1])}
+        e.close()
+        del e, eng
+        eng = None
+    row["config"] = dict(shape, decode=f"{B} sequences at position {ctx}", prefill=f"{Bp} prompts of {T}")
+    return row
+
+
+def _gptoss_beside(shape, vocab, positions, window, **moe):
+    """GPT-OSS of the same width and depth, its 64-wide attention heads in the same numbers."""
     binfmt = importlib.import_module("gpt-oss-team01_amd.binfmt")
+    return binfmt.Config(vocab_size=vocab, hidden_dim=shape["width"], n_layers=shape["layers"], head_dim=64,
+                         n_attn_heads=shape["attn_heads"], n_kv_heads=shape["kv_heads"], seq_len=positions,
+                         initial_context_length=4096, rope_theta=150000.0, rope_scaling_factor=32.0,
+                         sliding_window=window, swiglu_limit=7.0, **moe)
+
+
+def bench_nezavik(ops, torch, steps, only):
     out = {}
     for name, (shape, decode, prompt) in NEZAVIK_SIZES.items():
         if only and name not in only:
             continue
         (B, ctx), (Bp, T) = decode, prompt
-        positions = max(ctx + steps + 8, T)
+        positions, window = max(ctx + steps + 8, T), shape["window"]
         cfg = nezavik_config(positions=positions, **shape)
-        W, L, window = shape["width"], shape["layers"], shape["window"]
-        # GPT-OSS of the same width and depth: 64-wide heads in the same numbers, its experts all active and
-        # together as wide as the feed-forward
-        other = binfmt.Config(vocab_size=cfg["vocab"], hidden_dim=W, n_experts=4, experts_per_token=4,
-                              intermediate_dim=shape["ff"] // 4, n_layers=L, head_dim=64,
-                              n_attn_heads=shape["attn_heads"], n_kv_heads=shape["kv_heads"], seq_len=positions,
-                              initial_context_length=4096, rope_theta=150000.0, rope_scaling_factor=32.0,
-                              sliding_window=window, swiglu_limit=7.0)
-        with tempfile.TemporaryDirectory() as d:
-            with open(os.path.join(d, "config.json"), "w") as f:
-                json.dump(cfg, f)
-            eng = ops.Engine.open(d, max_batch=max(B, Bp), max_seq=positions, synthetic=True, keep_logits=False)
+        # experts that are all active and together as wide as the feed-forward
+        other = _gptoss_beside(shape, cfg["vocab"], positions, window, n_experts=4, experts_per_token=4,
+                               intermediate_dim=shape["ff"] // 4)
         mean_prompt = (window * (T - window) + window * (window + 1) / 2) / T if T > window else (T + 1) / 2
-        row = {}
-        for who, e, works in (
-                ("nezavik", eng, (_nezavik_work(cfg, B, B, min(window, ctx)),
-                                  _nezavik_work(cfg, Bp * T, Bp, mean_prompt))),
-                ("gpt_oss", None, (_gptoss_work(other, B, B, (ctx, min(window, ctx))),
-                                   _gptoss_work(other, Bp * T, Bp, ((T + 1) / 2, mean_prompt))))):
-            if e is None:
-                e = ops.Engine(other, None, max_batch=max(B, Bp), max_seq=positions, synthetic=True, keep_logits=False)
-            r = _time_engine(ops, torch, e, cfg["vocab"], decode, prompt, steps)
-            row[who] = {"decode_ms": round(r["decode"][0], 3), "decode_tok_s": round(B / r["decode"][0] * 1e3, 1),
-                        "prefill_ms": round(r["prefill"][0], 2), "prefill_tok_s": round(Bp * T / r["prefill"][0] * 1e3, 1),
-                        "device_gb": round(e.device_bytes() / 1e9, 2),
-                        "decode_kernels": _against_roofline(r["decode"][1], works[0]),
-                        "prefill_kernels": _against_roofline(r["prefill"][1], works[1])}
-            e.close()
-            del e
-        row["config"] = dict(shape, decode=f"{B} sequences at position {ctx}", prefill=f"{Bp} prompts of {T}")
-        out[name] = row
+        works = (_nezavik_work(cfg, B, B, min(window, ctx)), _nezavik_work(cfg, Bp * T, Bp, mean_prompt))
+        out[name] = _bench_beside_gptoss(ops, torch, steps, "nezavik", cfg, works, other, shape, decode, prompt, window)
+        print(f"{name}: done", file=sys.stderr, flush=True)
+    return out
+
+
+def bench_netinex(ops, torch, steps, only):
+    out = {}
+    for name, (shape, decode, prompt) in NETINEX_SIZES.items():
+        if only and name not in only:
+            continue
+        (B, ctx), (Bp, T) = decode, prompt
+        chunk = shape["chunk"]
+        cfg = netinex_config(**shape)
+        # the same experts
+        other = _gptoss_beside(shape, cfg["vocab"], max(ctx + steps + 8, T), chunk, n_experts=shape["experts"],
+                               experts_per_token=shape["top"], intermediate_dim=shape["ff"])
+        seen = (ctx + 3 + steps) % chunk + 1            # by the traced decode step
+        mean_prompt = sum(i % chunk + 1 for i in range(T)) / T
+        works = (_netinex_work(cfg, B, B, seen), _netinex_work(cfg, Bp * T, Bp, mean_prompt))
+        out[name] = _bench_beside_gptoss(ops, torch, steps, "netinex", cfg, works, other, shape, decode, prompt, chunk)
         print(f"{name}: done", file=sys.stderr, flush=True)
     return out
 
@@ -780,11 +877,12 @@ def main():
                           "rates": bench_mfma_rates(torch)}))
         return
 
-    if args.model == "nezavik":
+    if args.model != "gpt-oss":
         only = [x for x in args.only.split(",") if x]
-        print(json.dumps({"what": "Nezavik beside GPT-OSS of the same width (random weights, bf16): ms per step, kernel "
+        title, bench = {"nezavik": ("Nezavik", bench_nezavik), "netinex": ("Netinex", bench_netinex)}[args.model]
+        print(json.dumps({"what": f"{title} beside GPT-OSS of the same width (random weights, bf16): ms per step, kernel "
                                   "times and fraction of roofline (8 TB/s HBM, 2.5 PFLOP/s bf16, 78.6 TFLOP/s fp32)",
-                          "sizes": bench_nezavik(ops, torch, max(10, args.steps), only)}))
+                          "sizes": bench(ops, torch, max(10, args.steps), only)}))
         return
 
     # a plain device copy of known size (2 x 1 GiB moved), so counter runs of this same command can
