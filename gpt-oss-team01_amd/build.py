@@ -29,7 +29,7 @@ CORE = ("common.cpp", "engine.cpp", "model_registry.cpp", "glue.hip", "precise.h
         "gemm_bf16.hip", "gemm_mixed_bf16.hip", "gemm_tall.hip")
 #: architecture -> sources of its class beside CORE (None: all of them)
 MODELS = {"gpt-oss": None, "Nezavik": ("model_nezavik.cpp", "recurrent.hip", "window_attn.hip"),
-          "Netinex": ("model_netinex.cpp", "recurrent.hip", "window_attn.hip", "rotary.hip", "moe_layer.cpp",
+          "Netinex": ("model_netinex.cpp", "retention.hip", "recurrent.hip", "window_attn.hip", "rotary.hip", "moe_layer.cpp",
                       "moe_route.hip", "moe_gemm.hip", "gemm_gather_bf16.hip", "gemm_tall_grouped.hip")}
 
 

@@ -3,7 +3,7 @@
 // dynamic tanh, positions rotary, the classifier is the embedding table and its logits are soft-capped.
 //
 // Per layer the step runs
-//   one GEMM for the mixer's projections (rows of one packed matrix), the mixer's kernels (rotary.hip,
+//   one GEMM for the mixer's projections (rows of one packed matrix), the mixer's kernels (retention.hip,
 //   recurrent.hip / window_attn.hip), the output GEMM, the residual sum with the feed-forward's norm, the
 //   MoE block (moe_layer.cpp), whose combine adds into the residual stream and norms it for the next layer.
 // Every size and constant comes from config.json.  With GPTOSS_ENGINE_PRECISE weights, activations and the
@@ -27,7 +27,6 @@ struct NetinexLayer {
   TanhNorm norm1, norm2;
   Matrix in, out;
   // retention; pointers to activations are filled in per step
-  Rotary rot;
   Scan scan;
   GatedNorm gated;
   int gate_col = 0;
@@ -84,13 +83,11 @@ int Netinex::mix(NetinexLayer &w, const StepRows &r) {
     return run_window_attn(a, r, stream);
   }
   Scan sc = w.scan;
-  // queries and keys are neighbours
-  GPTOSS_STEP(run_rotary(w.rot, in_rows, ld_in, sc.q_col, 2 * sc.heads, sc.K, r.lens, r.n, stream));
   sc.conv = sc.in = in_rows;
   sc.ld_conv = sc.ld_in = ld_in;
   sc.out = y_rows;
   sc.ld_out = sc.heads * sc.V;
-  GPTOSS_STEP(run_scan(sc, r, stream));
+  GPTOSS_STEP(run_retention(sc, r, precise(), in_rows, stream));
   GatedNorm g = w.gated;
   g.y = y_rows;
   g.ld_y = sc.ld_out;
@@ -194,7 +191,7 @@ void load_retention(Loader &ld, NetinexLayer &w, const Json &mix, const std::str
   s.K = size_of(mix, "dim");
   s.V = size_of(mix, "vdim");
   require(s.K <= SCAN_MAX_KEY, "key dimensions above 256 are not supported", i);
-  w.rot = load_rotary(ld, mix, s.K, false, i);
+  s.rot = load_rotary(ld, mix, s.K, false, i);
   s.value_scale = 1.f / sqrtf((float)s.K);   // of the keys; what is written is linear in both
   const int nk = s.heads * s.K, nv = s.heads * s.V;
   const Json &decay = field(mix, "decay", Json::ARRAY);
@@ -205,6 +202,12 @@ void load_retention(Loader &ld, NetinexLayer &w, const Json &mix, const std::str
     d.push_back((float)x.number);
   }
   s.head_decay = ld.put(d);
+  std::vector<float> powers;
+  for (float x : d) {
+    double power = 1.0;
+    for (int t = 0; t <= RETENTION_CHUNK; t++, power *= x) powers.push_back((float)power);
+  }
+  s.decay_powers = ld.put(powers);
   Columns cols;
   s.q_col = cols.take(nk);
   s.k_col = cols.take(nk);

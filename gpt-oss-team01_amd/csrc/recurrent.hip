@@ -236,8 +236,25 @@ __global__ __launch_bounds__(256) void scan_kernel(Scan p, const RowSeg *__restr
 #pragma unroll
     for (int x = 0; x < PIECES; x++) {
       const int idx = tid + 256 * x, t = min(idx / (KP / 4), T - 1), d = idx % (KP / 4) * 4;
-      rk[x] = load4(k_src + (first + t) * p.ld_conv, d, p.K);
-      rq[x] = load4(q_src + (first + t) * p.ld_conv, d, p.K);
+      const float *kr = k_src + (first + t) * p.ld_conv, *qr = q_src + (first + t) * p.ld_conv;
+      rk[x] = load4(kr, d, p.K);
+      rq[x] = load4(qr, d, p.K);
+      if constexpr (RET && ONE) {
+        const int half = p.rot.table ? p.rot.dims >> 1 : 0;
+        if (d < 2 * half) {   // pairs (i, i + half)
+          const bool second = d >= half;
+          const int i = second ? d - half : d, partner = second ? i : i + half;
+          const f32x4 ko = load4(kr, partner, p.K), qo = load4(qr, partner, p.K);
+          const f32x4 *at = reinterpret_cast<const f32x4 *>(p.rot.table + ((size_t)seg.pos0 * half + i) * 2);
+          const f32x4 cs[2] = {at[0], at[1]};
+#pragma unroll
+          for (int e = 0; e < 4; e++) {
+            const float c = cs[e >> 1][2 * (e & 1)], s = (second ? 1.f : -1.f) * cs[e >> 1][2 * (e & 1) + 1];
+            rk[x][e] = rk[x][e] * c + ko[e] * s;
+            rq[x][e] = rq[x][e] * c + qo[e] * s;
+          }
+        }
+      }
       if (CHANNEL) rg[x] = load4(g_src + (first + t) * p.ld_decay, d, p.K);
     }
 #pragma unroll
@@ -542,9 +559,10 @@ static void launch_scan(const Scan &p, const StepRows &r, hipStream_t s) {
 
 int run_scan(const Scan &scan, const StepRows &r, hipStream_t s) {
   Scan p = scan;
-  p.vec = p.K % 4 == 0 && p.V % 4 == 0 && p.ld_conv % 4 == 0 && p.k_col % 4 == 0 && p.q_col % 4 == 0 && p.v_col % 4 == 0 &&
-          aligned(p.conv, 16) &&
-          (p.kind != SCAN_CHANNEL_DELTA || (p.ld_decay % 4 == 0 && aligned(p.channel_decay, 16)));
+  p.vec = scan_reads_wide(p);
+  GPTOSS_REQUIRE(!p.rot.table || (p.kind == SCAN_RETENTION && r.longest == 1 && p.vec && !p.rot.interleaved &&
+                                  p.rot.dims % 8 == 0 && p.rot.dims <= p.K),
+                 GPTOSS_ERR_DIM, "scan: only steps of one row per sequence rotate queries and keys, in groups of four dimensions");
   GPTOSS_REQUIRE(p.K >= 1 && p.K <= SCAN_MAX_KEY && p.V >= 1 && p.key_heads >= 1 && p.heads % p.key_heads == 0,
                  GPTOSS_ERR_DIM, "scan: key dimension %d (at most %d), %d heads over %d", p.K, SCAN_MAX_KEY, p.heads,
                  p.key_heads);

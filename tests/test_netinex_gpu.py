@@ -45,6 +45,9 @@ MIXED = [xm.retention(mlp=xm.moe()), xm.attention(mlp=xm.moe(experts=9, top=3), 
 MECHANISMS = {
     "retention": [xm.retention()],
     "retention_part_rotated": [xm.retention(heads=5, dim=33, vdim=65, dims=6, base=30.0)],
+    "retention_rotated_in_fours": [xm.retention(heads=3, dim=36, vdim=68, dims=24, base=30.0)],
+    "retention_rotated_in_twos": [xm.retention(heads=2, dim=28, vdim=20, dims=12)],
+    "retention_fast_decay": [xm.retention(heads=4, decay=[0.0, 0.01, 0.25, 1.0])],
     "attention": [xm.attention()],
     "attention_scaled_part_rotated": [xm.attention(heads=6, kv=2, dim=48, dims=40, size=70, scaling=xm.YARN)],
     "attention_one_group": [xm.attention(heads=20, kv=1, dim=24, dims=24, size=50)],
@@ -90,7 +93,8 @@ def test_first_tokens_of_a_sequence(open_model, precise):
 
 
 @BOTH
-@pytest.mark.parametrize("cuts", [[1], [2], [3, 2], [5, 1, 1, 7], [64], [63, 1, 2], [130, 2, 1], [16], [17, 2, 31], [47, 46, 1]])
+@pytest.mark.parametrize("cuts", [[1], [2], [3, 2], [5, 1, 1, 7], [64], [63, 1, 2], [130, 2, 1], [16], [17, 2, 31], [47, 46, 1],
+                                  [8, 9], [65, 15], [10, 1, 1, 33]])
 def test_portions_and_decoding_equal_the_whole_prompt(open_model, cuts, precise):
     cfg = xm.config(MIXED)
     w = xm.weights(cfg, 20)
@@ -261,6 +265,9 @@ SIZES = {
                               xm.attention(heads=2, kv=1, dim=256, dims=128, size=70, scale=0.06),
                               xm.retention(heads=1, dim=160, vdim=128, dims=32, mlp=xm.moe(ff=256, experts=4, top=2))],
                              vocab=64, width=128),
+    "keys_of_every_width": xm.config([xm.retention(heads=2, dim=d, vdim=v, dims=r)
+                                      for d, v, r in ((64, 64, 64), (96, 32, 48), (128, 132, 128), (192, 48, 64), (224, 16, 224))],
+                                     width=160),
     "many_heads": xm.config([xm.attention(heads=40, kv=2, dim=16, dims=16, size=24),
                              xm.retention(heads=24, dim=8, vdim=16, dims=4, mlp=xm.moe(experts=33, top=8))],
                             vocab=128, width=192, eps=1e-2, softcap=4.0),
