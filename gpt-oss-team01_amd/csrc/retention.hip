@@ -52,220 +52,245 @@ template <int NI, int C>
 struct RetentionTile {
   static constexpr int KP = 32 * NI, TT = C / 16, SG = C / 32;
   static constexpr int ROW = KP + 8, COL = C + 8;   // rows of an operand matrix, 16 bytes apart in their banks
-  static constexpr int Q = 0, K = Q + 2 * C * ROW, KT = K + 2 * C * ROW, P = KT + 2 * KP * COL;   // hi parts, then lo parts
-  static constexpr int ELEMS = P + 2 * TT * SG * 512;
+  // hi parts, then lo parts
+  static constexpr int Q = 0, K = Q + 2 * C * ROW, KT = K + 2 * C * ROW, P = KT + 2 * KP * COL, X = P + 2 * TT * SG * 512;
+  static constexpr int ELEMS = X + 8 * (TT / 2) * 64 * 8;   // X: fp32
 };
 
+// Waves w and w + 4 share 16 columns: the first has the lower half of their state (by key dimension) and, in the end,
+// of the chunk's rows.  The first four waves stage keys, the others queries.
 template <int NI, int C>
-__global__ __launch_bounds__(256) void retention_chunk_kernel(Scan p, const RowSeg *__restrict__ segs, int n_seg) {
+__global__ __launch_bounds__(512) void retention_chunk_kernel(Scan p, const RowSeg *__restrict__ segs, int n_seg) {
   using L = RetentionTile<NI, C>;
   constexpr int KP = L::KP, TT = L::TT, SG = L::SG, UPT = KP / 8;   // units of 8 dimensions x 4 tokens
-  constexpr int OWN = TT * TT / 4;                                  // tiles of the token products per wave
+  constexpr int OWN = TT * TT > 8 ? TT * TT / 8 : 1;                // tiles of the token products per wave
+  constexpr int NK = (NI + 1) / 2, HT = TT / 2;                     // of a wave: 32-key steps (at most), row tiles
   extern __shared__ __attribute__((aligned(16))) bf16_t lds[];
   const int seg_id = blockIdx.x % n_seg, unit = blockIdx.x / n_seg, blocks = (p.V + 63) / 64;
   const RowSeg seg = segs[seg_id];
   const int h = unit / blocks, kh = h / (p.heads / p.key_heads);
-  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int tid = threadIdx.x & 255, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int half = wave >> 2, k0 = half * NK, n_k = half ? NI - NK : NK;
   const int n = lane & 15, c = lane >> 4;
-  const int c0 = (unit - h * blocks) * 64 + wave * 16, col = min(c0 + n, p.V - 1);   // columns c0 .. + 15 of the wave
+  const int c0 = (unit - h * blocks) * 64 + (wave & 3) * 16, col = min(c0 + n, p.V - 1);   // columns c0 .. + 15 of the wave
   const bool live = c0 + n < p.V;
   const float *power = p.decay_powers + h * (RETENTION_CHUNK + 1);
 
-  f32x4 S[2 * NI];   // d = 16 b + 4 c + e of column c0 + n
-  float *st = p.state + (((size_t)seg.slot * p.heads + h) * p.V + col) * KP + 4 * c;
+  f32x4 S[2 * NK];   // d = 32 k0 + 16 b + 4 c + e of column c0 + n
+  float *st = p.state + (((size_t)seg.slot * p.heads + h) * p.V + col) * KP + 32 * k0 + 4 * c;
 #pragma unroll
-  for (int b = 0; b < 2 * NI; b++) {
+  for (int b = 0; b < 2 * NK; b++) {
     S[b] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (seg.pos0 > 0 && live) S[b] = __builtin_nontemporal_load(reinterpret_cast<const f32x4 *>(st + 16 * b));
+    if (seg.pos0 > 0 && live && b < 2 * n_k) S[b] = __builtin_nontemporal_load(reinterpret_cast<const f32x4 *>(st + 16 * b));
   }
 
   // powers that do not change from chunk to chunk: of this wave's tiles of token products, and of the rows of the output
-  const int p_t = wave % TT, p_s = wave / TT;   // token tile of the queries; tiles p_s, p_s + 4 / TT, .. of the keys
+  const int p_t = wave % TT, p_s = wave / TT;   // token tile of the queries; tiles p_s, p_s + 8 / TT, .. of the keys
   float tri[OWN][4], from[TT];
 #pragma unroll
   for (int i = 0; i < OWN; i++)
 #pragma unroll
     for (int e = 0; e < 4; e++) {
-      const int back = p_t * 16 + n - ((p_s + i * (4 / TT)) * 16 + 4 * c + e);
-      tri[i][e] = back >= 0 ? power[max(back, 0)] : 0.f;
+      const int back = p_t * 16 + n - ((p_s + i * (8 / TT)) * 16 + 4 * c + e);
+      tri[i][e] = back >= 0 ? p.value_scale * power[max(back, 0)] : 0.f;
     }
 #pragma unroll
   for (int t = 0; t < TT; t++) from[t] = power[t * 16 + n + 1];
 
-  // one staging unit per thread: dimensions d0 .. + 3 and d1 .. + 3 (partners where they are rotated) of tokens 4 a .. 4 a + 3
-  const int y = tid % UPT, a = tid / UPT, half = p.rot.table ? p.rot.dims >> 1 : 0;
-  const bool stages = a < C / 4, turned = 4 * y < half;
-  const int d0 = turned ? 4 * y : 2 * half + 8 * (y - half / 4), d1 = turned ? 4 * y + half : d0 + 4;
-  const float *k_src = p.conv + p.k_col + kh * p.K, *q_src = p.conv + p.q_col + kh * p.K, *v_src = p.conv + p.v_col + h * p.V + col;
-  f32x4 rq[4][2], rk[4][2], cs[4][2];
-  float rv[SG * 8];
+  // One staging unit per thread: dimensions d0 .. + 3 and d1 .. + 3 (partners where they are rotated) of tokens
+  // 4 a .. 4 a + 3.  Addresses are a base per workgroup and a 32-bit offset per lane.
+  const int y = tid % UPT, a = tid / UPT, pairs = p.rot.table ? p.rot.dims >> 1 : 0;
+  const bool stages = UPT * (C / 4) == 256 || a < C / 4, turned = 4 * y < pairs, keys = half == 0;
+  const int d0 = turned ? 4 * y : 2 * pairs + 8 * (y - pairs / 4), d1 = turned ? 4 * y + pairs : d0 + 4;
+  const unsigned x0 = 4 * min(d0, p.K - 4), x1 = 4 * min(d1, p.K - 4), x_cs = 8 * min(4 * y, max(pairs - 4, 0));
+  const unsigned ld = 4 * p.ld_conv, ld_cs = 8 * pairs;   // in bytes
+  const int src_col = (keys ? p.k_col : p.q_col) + kh * p.K;
+  auto at4 = [](const void *base, unsigned offset) {
+    return *reinterpret_cast<const f32x4 *>(static_cast<const char *>(base) + offset);
+  };
+  f32x4 rx[4][2], cs[4][2];
+  float rv[SG * 8], rw[4], fade;
+#pragma unroll
+  for (int i = 0; i < 4; i++)
+#pragma unroll
+    for (int x = 0; x < 2; x++) rx[i][x] = cs[i][x] = f32x4{0.f, 0.f, 0.f, 0.f};
   auto fetch = [&](int t0) {
     const int T = min(C, seg.n - t0);
-    const size_t first = seg.row0 + t0;
+    const float *rows = p.conv + (size_t)(seg.row0 + t0) * p.ld_conv;
+    const float *src = rows + src_col, *v = rows + p.v_col + h * p.V;
+    const float *angles = p.rot.table + (size_t)(seg.pos0 + t0) * pairs * 2;
+    fade = power[T];
     if (stages) {
+      unsigned t[4];
+#pragma unroll
+      for (int i = 0; i < 4; i++) t[i] = min(4 * a + i, T - 1);
 #pragma unroll
       for (int i = 0; i < 4; i++) {
-        const int t = min(4 * a + i, T - 1);
-        const float *q = q_src + (first + t) * p.ld_conv, *k = k_src + (first + t) * p.ld_conv;
-        const int x0 = min(d0, p.K - 4), x1 = min(d1, p.K - 4);
-        rq[i][0] = *reinterpret_cast<const f32x4 *>(q + x0);
-        rq[i][1] = *reinterpret_cast<const f32x4 *>(q + x1);
-        rk[i][0] = *reinterpret_cast<const f32x4 *>(k + x0);
-        rk[i][1] = *reinterpret_cast<const f32x4 *>(k + x1);
-        if (turned) {
-          const f32x4 *at = reinterpret_cast<const f32x4 *>(p.rot.table + ((size_t)(seg.pos0 + t0 + t) * half + 4 * y) * 2);
-          cs[i][0] = at[0];
-          cs[i][1] = at[1];
-        }
+        rx[i][0] = at4(src, t[i] * ld + x0);
+        rx[i][1] = at4(src, t[i] * ld + x1);
+        rw[i] = power[max(T - 1 - (4 * a + i), 0)];
       }
+      if (pairs)
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+          cs[i][0] = at4(angles, t[i] * ld_cs + x_cs);
+          cs[i][1] = at4(angles, t[i] * ld_cs + x_cs + 16);
+        }
     }
 #pragma unroll
     for (int x = 0; x < SG * 8; x++) {
       const int t = (x >> 3) * 32 + ((x >> 2) & 1) * 16 + 4 * c + (x & 3);
-      rv[x] = v_src[(first + min(t, T - 1)) * p.ld_conv];
+      rv[x] = *reinterpret_cast<const float *>(reinterpret_cast<const char *>(v) + (min(t, T - 1) * ld + 4 * col));
     }
   };
   auto put = [&](int T) {
     if (!stages) return;
-    f32x4 kw[4][2];
+    if (T < C || p.K < KP) {   // rows and columns outside the problem
+#pragma unroll
+      for (int i = 0; i < 4; i++)
+#pragma unroll
+        for (int x = 0; x < 2; x++) {
+          const bool out = (x ? d1 : d0) >= p.K || 4 * a + i >= T;
+#pragma unroll
+          for (int e = 0; e < 4; e++) rx[i][x][e] = out ? 0.f : rx[i][x][e];
+        }
+    }
+    bf16_t *rows = lds + (keys ? L::K : L::Q);
 #pragma unroll
     for (int i = 0; i < 4; i++) {
-      const int t = 4 * a + i;
-      f32x4 q[2] = {rq[i][0], rq[i][1]}, k[2] = {rk[i][0], rk[i][1]};
-      if (turned) {
+      f32x4 z[2];
 #pragma unroll
-        for (int e = 0; e < 4; e++) {
-          const float cosine = cs[i][e >> 1][2 * (e & 1)], sine = cs[i][e >> 1][2 * (e & 1) + 1];
-          q[0][e] = rq[i][0][e] * cosine - rq[i][1][e] * sine;
-          q[1][e] = rq[i][1][e] * cosine + rq[i][0][e] * sine;
-          k[0][e] = rk[i][0][e] * cosine - rk[i][1][e] * sine;
-          k[1][e] = rk[i][1][e] * cosine + rk[i][0][e] * sine;
-        }
+      for (int e = 0; e < 4; e++) {
+        const float cosine = turned ? cs[i][e >> 1][2 * (e & 1)] : 1.f, sine = turned ? cs[i][e >> 1][2 * (e & 1) + 1] : 0.f;
+        z[0][e] = rx[i][0][e] * cosine - rx[i][1][e] * sine;
+        z[1][e] = rx[i][1][e] * cosine + rx[i][0][e] * sine;
       }
-      const float w = t < T ? power[max(T - 1 - t, 0)] : 0.f;
 #pragma unroll
       for (int x = 0; x < 2; x++) {
-        const int d = x ? d1 : d0;
-        if (d >= p.K) q[x] = k[x] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (t >= T) k[x] = f32x4{0.f, 0.f, 0.f, 0.f};
-        kw[i][x] = k[x] * w;
-        const int at = t * L::ROW + operand_place(d);
-        const Split4 sq = split4(q[x]), sk = split4(k[x]);
-        *reinterpret_cast<u32x2 *>(lds + L::Q + at) = sq.hi;
-        *reinterpret_cast<u32x2 *>(lds + L::Q + C * L::ROW + at) = sq.lo;
-        *reinterpret_cast<u32x2 *>(lds + L::K + at) = sk.hi;
-        *reinterpret_cast<u32x2 *>(lds + L::K + C * L::ROW + at) = sk.lo;
+        const int at = (4 * a + i) * L::ROW + operand_place(x ? d1 : d0);
+        const Split4 s = split4(z[x]);
+        *reinterpret_cast<u32x2 *>(rows + at) = s.hi;
+        *reinterpret_cast<u32x2 *>(rows + C * L::ROW + at) = s.lo;
+        rx[i][x] = z[x] * (p.value_scale * rw[i]);
       }
     }
+    if (!keys) return;
 #pragma unroll
     for (int x = 0; x < 2; x++)
 #pragma unroll
       for (int e = 0; e < 4; e++) {
-        const Split4 s = split4(f32x4{kw[0][x][e], kw[1][x][e], kw[2][x][e], kw[3][x][e]});
+        const Split4 s = split4(f32x4{rx[0][x][e], rx[1][x][e], rx[2][x][e], rx[3][x][e]});
         const int at = ((x ? d1 : d0) + e) * L::COL + operand_place(4 * a);
         *reinterpret_cast<u32x2 *>(lds + L::KT + at) = s.hi;
         *reinterpret_cast<u32x2 *>(lds + L::KT + KP * L::COL + at) = s.lo;
       }
   };
 
+  // Every tile is multiplied, also where a chunk has fewer tokens or a tile lies behind its queries: the operands or
+  // the powers are zero there.
   fetch(0);
   for (int t0 = 0; t0 < seg.n; t0 += C) {
-    const int T = min(C, seg.n - t0), nt = (T + 15) / 16;
+    const int T = min(C, seg.n - t0);
     put(T);   // the last reads of Q, K and KT lie before the barrier in front of the previous chunk's last products
+    if (T < C || c0 + 16 > p.V) {
+#pragma unroll
+      for (int x = 0; x < SG * 8; x++) {
+        const int t = (x >> 3) * 32 + ((x >> 2) & 1) * 16 + 4 * c + (x & 3);
+        rv[x] = t < T && live ? rv[x] : 0.f;
+      }
+    }
     Operand v[SG];
 #pragma unroll
-    for (int x = 0; x < SG; x++) {
-      f32x4 part[2];
-#pragma unroll
-      for (int e = 0; e < 8; e++) {
-        const int t = x * 32 + (e >> 2) * 16 + 4 * c + (e & 3);
-        part[e >> 2][e & 3] = t < T && live ? p.value_scale * rv[x * 8 + e] : 0.f;
-      }
-      v[x] = make_operand(part[0], part[1]);
-    }
+    for (int x = 0; x < SG; x++)
+      v[x] = make_operand(f32x4{rv[8 * x], rv[8 * x + 1], rv[8 * x + 2], rv[8 * x + 3]},
+                          f32x4{rv[8 * x + 4], rv[8 * x + 5], rv[8 * x + 6], rv[8 * x + 7]});
+    const float faded = fade;
     __syncthreads();
     if (t0 + C < seg.n) fetch(t0 + C);
 
     // products of keys and queries, [key][query], masked and decayed, in operand order
-    f32x4 prod[OWN];
+    if (TT * TT >= 8 || wave < TT * TT) {
+      f32x4 prod[OWN];
 #pragma unroll
-    for (int i = 0; i < OWN; i++) prod[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (p_t < nt) {
+      for (int i = 0; i < OWN; i++) prod[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < NI; ks++) {
         const Operand q = read_operand(lds + L::Q + (p_t * 16 + n) * L::ROW + ks * 32 + c * 8, C * L::ROW);
 #pragma unroll
-        for (int i = 0; i < OWN; i++) {
-          const int s = p_s + i * (4 / TT);
-          if (s <= p_t)
-            multiply_add(prod[i], read_operand(lds + L::K + (s * 16 + n) * L::ROW + ks * 32 + c * 8, C * L::ROW), q);
-        }
+        for (int i = 0; i < OWN; i++)
+          multiply_add(prod[i], read_operand(lds + L::K + ((p_s + i * (8 / TT)) * 16 + n) * L::ROW + ks * 32 + c * 8, C * L::ROW), q);
       }
 #pragma unroll
       for (int i = 0; i < OWN; i++) {
-        const int s = p_s + i * (4 / TT);
-        if (s / 2 <= p_t / 2) {
-          f32x4 w;
+        const int s = p_s + i * (8 / TT);
+        f32x4 w;
 #pragma unroll
-          for (int e = 0; e < 4; e++) w[e] = prod[i][e] * tri[i][e];
-          const Split4 x = split4(w);
-          bf16_t *at = lds + L::P + ((p_t * SG + s / 2) * 64 + lane) * 8 + (s & 1) * 4;
-          *reinterpret_cast<u32x2 *>(at) = x.hi;
-          *reinterpret_cast<u32x2 *>(at + TT * SG * 512) = x.lo;
-        }
+        for (int e = 0; e < 4; e++) w[e] = prod[i][e] * tri[i][e];
+        const Split4 x = split4(w);
+        bf16_t *at = lds + L::P + ((p_t * SG + s / 2) * 64 + lane) * 8 + (s & 1) * 4;
+        *reinterpret_cast<u32x2 *>(at) = x.hi;
+        *reinterpret_cast<u32x2 *>(at + TT * SG * 512) = x.lo;
       }
     }
 
-    // what the state in front of the chunk gives: [column][query]
+    // what this half of the state in front of the chunk gives: [column][query]
     f32x4 o[TT];
 #pragma unroll
     for (int t = 0; t < TT; t++) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (seg.pos0 + t0 > 0) {
 #pragma unroll
-      for (int ks = 0; ks < NI; ks++) {
-        const Operand s = make_operand(S[2 * ks], S[2 * ks + 1]);
+    for (int ks = 0; ks < NK; ks++) {
+      if (NI % 2 && ks >= n_k) break;
+      const Operand s = make_operand(S[2 * ks], S[2 * ks + 1]);
 #pragma unroll
-        for (int t = 0; t < TT; t++)
-          if (t < nt) multiply_add(o[t], s, read_operand(lds + L::Q + (t * 16 + n) * L::ROW + ks * 32 + c * 8, C * L::ROW));
-      }
+      for (int t = 0; t < TT; t++)
+        multiply_add(o[t], s, read_operand(lds + L::Q + (t * 16 + n) * L::ROW + (k0 + ks) * 32 + c * 8, C * L::ROW));
+    }
+    // the other wave's rows go to it
+    f32x4 mine[HT];
+    f32x4 *exchange = reinterpret_cast<f32x4 *>(lds + L::X) + lane;
 #pragma unroll
-      for (int t = 0; t < TT; t++) o[t] *= from[t];
+    for (int i = 0; i < HT; i++) {
+      mine[i] = half ? o[HT + i] * from[HT + i] : o[i] * from[i];
+      exchange[(wave * HT + i) * 64] = half ? o[i] * from[i] : o[HT + i] * from[HT + i];
     }
 
     // the state behind it
-    const float fade = power[T];
 #pragma unroll
-    for (int b = 0; b < 2 * NI; b++) {
-      S[b] *= fade;
+    for (int b = 0; b < 2 * NK; b++) {
+      if (NI % 2 && b >= 2 * n_k) break;
+      S[b] *= faded;
 #pragma unroll
       for (int x = 0; x < SG; x++)
-        if (32 * x < T)
-          multiply_add(S[b], read_operand(lds + L::KT + (b * 16 + n) * L::COL + x * 32 + c * 8, KP * L::COL), v[x]);
+        multiply_add(S[b], read_operand(lds + L::KT + (k0 * 32 + b * 16 + n) * L::COL + x * 32 + c * 8, KP * L::COL), v[x]);
     }
     __syncthreads();
 
 #pragma unroll
-    for (int t = 0; t < TT; t++) {
-      if (t >= nt) break;
+    for (int i = 0; i < HT; i++) mine[i] += exchange[((wave ^ 4) * HT + i) * 64];
 #pragma unroll
-      for (int x = 0; x <= t / 2; x++)
-        multiply_add(o[t], v[x], read_operand(lds + L::P + ((t * SG + x) * 64 + lane) * 8, TT * SG * 512));
-      const int row = t * 16 + n, first = c0 + 4 * c;
-      if (row < T) {
-        float *dst = p.out + (size_t)(seg.row0 + t0 + row) * p.ld_out + h * p.V + first;
-        if (p.vec && first + 4 <= p.V) {
-          *reinterpret_cast<f32x4 *>(dst) = o[t];
-        } else {
+    for (int x = 0; x < SG; x++) {
+      if (x > (half * HT + HT - 1) / 2) break;   // behind the queries
 #pragma unroll
-          for (int e = 0; e < 4; e++)
-            if (first + e < p.V) dst[e] = o[t][e];
-        }
-      }
+      for (int i = 0; i < HT; i++)
+        multiply_add(mine[i], v[x], read_operand(lds + L::P + (((half * HT + i) * SG + x) * 64 + lane) * 8, TT * SG * 512));
+    }
+    const int first = c0 + 4 * c, row = half * HT * 16 + n;
+    float *out = p.out + (size_t)(seg.row0 + t0) * p.ld_out + h * p.V;
+    if (p.vec && T == C && c0 + 16 <= p.V) {
+#pragma unroll
+      for (int i = 0; i < HT; i++) *reinterpret_cast<f32x4 *>(out + (unsigned)((row + i * 16) * p.ld_out + first)) = mine[i];
+    } else {
+#pragma unroll
+      for (int i = 0; i < HT; i++)
+#pragma unroll
+        for (int e = 0; e < 4; e++)
+          if (row + i * 16 < T && first + e < p.V) out[(row + i * 16) * p.ld_out + first + e] = mine[i][e];
     }
   }
   if (live) {
 #pragma unroll
-    for (int b = 0; b < 2 * NI; b++) __builtin_nontemporal_store(S[b], reinterpret_cast<f32x4 *>(st + 16 * b));
+    for (int b = 0; b < 2 * NK; b++)
+      if (b < 2 * n_k) __builtin_nontemporal_store(S[b], reinterpret_cast<f32x4 *>(st + 16 * b));
   }
 }
 
@@ -280,7 +305,7 @@ static int launch_chunks(const Scan &p, const StepRows &r, hipStream_t s) {
     ready = true;
   }
   TraceScope ts("retention_chunks", s);
-  kern<<<(unsigned)((size_t)r.n_seg * p.heads * cdiv(p.V, 64)), 256, bytes, s>>>(p, r.segs, r.n_seg);
+  kern<<<(unsigned)((size_t)r.n_seg * p.heads * cdiv(p.V, 64)), 512, bytes, s>>>(p, r.segs, r.n_seg);
   GPTOSS_LAUNCH_CHECK("retention_chunk_kernel");
   return GPTOSS_OK;
 }
