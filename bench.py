@@ -729,10 +729,10 @@ def _netinex_work(cfg, rows, seqs, context):
         if layer["type"] == "retention":
             nk, nv = H * m["dim"], H * m["vdim"]
             gemm(2 * nk + 2 * nv, W)
-            add("rotary", rows * 2 * H * m["rot"]["dims"] * 8)
-            # per state element and token: decay, update, read-out
-            add("scan_retention", seqs * nk * m["vdim"] * 8 + rows * (2 * nk + 2 * nv) * 4, 5.0 * rows * nk * m["vdim"],
-                VALU_FP32_PEAK_TFLOPS)
+            # per state element and token: decay, update, read-out; in chunks the last two are matrix products
+            nbytes = seqs * nk * m["vdim"] * 8 + rows * (2 * nk + 2 * nv) * 4
+            add("scan_retention", nbytes, 5.0 * rows * nk * m["vdim"], VALU_FP32_PEAK_TFLOPS)
+            add("retention_chunks", nbytes, 4.0 * rows * nk * m["vdim"])
             add("gated_norm", rows * nv * 10)
         else:
             nq, nk, nv = H * m["dim"], m["kv_heads"] * m["dim"], H * m["vdim"]

@@ -106,7 +106,103 @@ __global__ __launch_bounds__(256) void window_store_kernel(WindowAttn a, const i
   }
 }
 
-// Norm over all heads at once, rotation, K/V store: one workgroup per row.
+// Norm over all heads at once, rotation, K/V store: one workgroup per RT rows, whose heads (of a multiple of four
+// dimensions, rotated in neighbouring pairs, values the keys as projected) lie in its registers, four values a piece.
+template <bool F32, int NV, int RT>
+__global__ __launch_bounds__(256) void window_store_rows_kernel(WindowAttn a, const int *__restrict__ slots,
+                                                                const int *__restrict__ lens, int n) {
+  __shared__ float red[RT][2][4];
+  const int row0 = blockIdx.x * RT, tid = threadIdx.x, H = a.heads, G = a.kv_heads, D = a.dim, live = min(RT, n - row0);
+  const int DK = F32 ? D : a.dim_pad(), dims = a.rot.table ? a.rot.dims : 0;
+  constexpr bool EARLY = RT == 1;   // angles are requested with the rows
+  f32x4 x[NV][RT], w[NV], cs[EARLY ? NV : 1];
+  int head[NV], d[NV], pos[RT], seq[RT];
+#pragma unroll
+  for (int r = 0; r < RT; r++) {
+    const int row = row0 + min(r, live - 1);
+    pos[r] = lens[row] - 1;
+    seq[r] = slots[row];
+  }
+  auto angles = [&](int i, int r) {
+    return head[i] < H + G && d[i] < dims ? *reinterpret_cast<const f32x4 *>(a.rot.table + (size_t)pos[r] * dims + d[i])
+                                          : f32x4{1.f, 0.f, 1.f, 0.f};
+  };
+#pragma unroll
+  for (int i = 0; i < NV; i++) {
+    const int u = tid + 256 * i;
+    head[i] = u / (DK >> 2);
+    d[i] = (u - head[i] * (DK >> 2)) * 4;
+    const bool in = head[i] < H + G && d[i] < D, is_q = head[i] < H;
+    const int at = (is_q ? head[i] : head[i] - H) * D + d[i];
+    w[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (in) w[i] = *reinterpret_cast<const f32x4 *>((is_q ? a.q_norm : a.k_norm) + at);
+#pragma unroll
+    for (int r = 0; r < RT; r++) {
+      x[i][r] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (in) x[i][r] = *reinterpret_cast<const f32x4 *>(a.in + (size_t)(row0 + min(r, live - 1)) * a.ld_in + (is_q ? a.q_col : a.k_col) + at);
+      if (EARLY) cs[i] = angles(i, r);
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < RT; r++) {
+    float ss[2] = {0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NV; i++) {
+      float own = 0.f;
+#pragma unroll
+      for (int e = 0; e < 4; e++) own = fmaf(x[i][r][e], x[i][r][e], own);
+      ss[0] += head[i] < H ? own : 0.f;
+      ss[1] += head[i] < H ? 0.f : own;
+    }
+#pragma unroll
+    for (int k = 0; k < 2; k++) {
+#pragma unroll
+      for (int m = 32; m >= 1; m >>= 1) ss[k] += __shfl_xor(ss[k], m, 64);
+      if ((tid & 63) == 0) red[r][k][tid >> 6] = ss[k];
+    }
+  }
+  __syncthreads();
+  // four positions from a multiple of four on: a value's places are neighbours
+  const bool four = RT == 4 && live == 4 && pos[0] % 4 == 0 && pos[RT - 1] == pos[0] + 3 && seq[RT - 1] == seq[0];
+#pragma unroll
+  for (int r = 0; r < RT; r++) {
+    if (r >= live) break;
+    const float inv[2] = {1.f / sqrtf((red[r][0][0] + red[r][0][1] + red[r][0][2] + red[r][0][3]) / (H * D) + a.eps),
+                          1.f / sqrtf((red[r][1][0] + red[r][1][1] + red[r][1][2] + red[r][1][3]) / (G * D) + a.eps)};
+    const int cslot = pos[r] % a.cap;
+#pragma unroll
+    for (int i = 0; i < NV; i++) {
+      if (head[i] >= H + G) continue;
+      const bool is_q = head[i] < H;
+      const f32x4 own = x[i][r] * (is_q ? inv[0] : inv[1]) * w[i], c = EARLY ? cs[EARLY ? i : 0] : angles(i, r);
+      const f32x4 y = {own[0] * c[0] - own[1] * c[1], own[1] * c[0] + own[0] * c[1],
+                       own[2] * c[2] - own[3] * c[3], own[3] * c[2] + own[2] * c[3]};
+      const int g = head[i] - H;
+      if (is_q) {
+        *reinterpret_cast<f32x4 *>(a.q + ((size_t)(row0 + r) * H + head[i]) * DK + d[i]) = y;
+      } else if constexpr (F32) {
+        const size_t at = (((size_t)seq[r] * a.cap + cslot) * G + g) * D + d[i];
+        *reinterpret_cast<f32x4 *>(a.k32 + at) = y;
+        *reinterpret_cast<f32x4 *>(a.v32 + at) = x[i][r];
+      } else {
+        const StorePlace at{a.kv + ((size_t)(seq[r] * G + g) * (a.cap >> 6) + (cslot >> 6)) * a.block_elems(), cslot, DK, DK};
+        *reinterpret_cast<u32x2 *>(at.key(d[i])) = u32x2{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
+        bf16_t *v = at.value(d[i]);   // dimensions of a group of 16 lie 8 elements apart
+        if (!four) {
+#pragma unroll
+          for (int e = 0; e < 4; e++) v[8 * e] = f32_to_bf16(x[i][r][e]);
+        } else if (r == 0) {
+#pragma unroll
+          for (int e = 0; e < 4; e++)
+            *reinterpret_cast<u32x2 *>(v + 8 * e) = u32x2{pack_bf16x2(x[i][0][e], x[i][RT > 1 ? 1 : 0][e]),
+                                                          pack_bf16x2(x[i][RT > 2 ? 2 : 0][e], x[i][RT > 3 ? 3 : 0][e])};
+        }
+      }
+    }
+  }
+}
+
+// The same for any sizes and either layout of the rotated pairs, one workgroup per row.
 template <bool F32>
 __global__ __launch_bounds__(256) void window_store_row_kernel(WindowAttn a, const int *__restrict__ slots,
                                                                const int *__restrict__ lens) {
@@ -528,6 +624,33 @@ __global__ __launch_bounds__(256) void window_f32_kernel(WindowAttn a, const int
 }
 
 // ---- launches ------------------------------------------------------------------------------------
+template <bool F32>
+static void launch_store_rows(const WindowAttn &a, const StepRows &r, hipStream_t s) {
+  const bool pieces = a.dim % 4 == 0 && a.v_col == a.k_col && a.vdim == a.dim && a.ld_in % 4 == 0 && a.q_col % 4 == 0 &&
+                      a.k_col % 4 == 0 && aligned(a.in, 16) && aligned(a.q_norm, 16) && aligned(a.k_norm, 16) &&
+                      (!a.rot.table || (a.rot.interleaved && a.rot.dims % 4 == 0));
+  const int per_thread = cdiv((a.heads + a.kv_heads) * ((F32 ? a.dim : a.dim_pad()) / 4), 256);
+  auto go = [&](auto kern, int rt) { kern<<<cdiv(r.n, rt), 256, 0, s>>>(a, r.slots, r.lens, r.n); };
+  if (!pieces || per_thread > 8) {
+    window_store_row_kernel<F32><<<r.n, 256, 0, s>>>(a, r.slots, r.lens);
+  } else if (!F32 && r.n >= 1024 && per_thread <= 5) {
+    if constexpr (!F32) {
+      if (per_thread <= 1) go(window_store_rows_kernel<F32, 1, 4>, 4);
+      else if (per_thread <= 2) go(window_store_rows_kernel<F32, 2, 4>, 4);
+      else if (per_thread <= 3) go(window_store_rows_kernel<F32, 3, 4>, 4);
+      else go(window_store_rows_kernel<F32, 5, 4>, 4);
+    }
+  } else if (per_thread <= 1) {
+    go(window_store_rows_kernel<F32, 1, 1>, 1);
+  } else if (per_thread <= 3) {
+    go(window_store_rows_kernel<F32, 3, 1>, 1);
+  } else if (per_thread <= 5) {
+    go(window_store_rows_kernel<F32, 5, 1>, 1);
+  } else {
+    go(window_store_rows_kernel<F32, 8, 1>, 1);
+  }
+}
+
 int run_window_attn(const WindowAttn &a, const StepRows &r, hipStream_t s) {
   GPTOSS_REQUIRE(a.dim >= 1 && a.dim <= WINDOW_ATTN_MAX_DIM && a.vdim >= 1 && a.vdim <= WINDOW_ATTN_MAX_DIM &&
                      a.kv_heads >= 1 && a.heads % a.kv_heads == 0 && a.window >= 1 && a.cap % 64 == 0,
@@ -542,7 +665,7 @@ int run_window_attn(const WindowAttn &a, const StepRows &r, hipStream_t s) {
   if (a.k32) {
     {
       TraceScope ts("window_store", s);
-      if (a.whole_norm) window_store_row_kernel<true><<<r.n, 256, 0, s>>>(a, r.slots, r.lens);
+      if (a.whole_norm) launch_store_rows<true>(a, r, s);
       else window_store_kernel<true, 1><<<dim3(cdiv(units, 4), r.n), 256, 0, s>>>(a, r.slots, r.lens, r.n);
     }
     GPTOSS_LAUNCH_CHECK("window_store_kernel");
@@ -553,7 +676,7 @@ int run_window_attn(const WindowAttn &a, const StepRows &r, hipStream_t s) {
   }
   {
     TraceScope ts("window_store", s);
-    if (a.whole_norm) window_store_row_kernel<false><<<r.n, 256, 0, s>>>(a, r.slots, r.lens);
+    if (a.whole_norm) launch_store_rows<false>(a, r, s);
     else if (r.n >= 1024) window_store_kernel<false, 4><<<dim3(cdiv(units, 4), cdiv(r.n, 4)), 256, 0, s>>>(a, r.slots, r.lens, r.n);
     else window_store_kernel<false, 1><<<dim3(cdiv(units, 4), r.n), 256, 0, s>>>(a, r.slots, r.lens, r.n);
   }

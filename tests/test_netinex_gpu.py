@@ -252,6 +252,7 @@ def test_long_decoding_past_the_ring(open_model, precise):
     factor = 4.0
     check(feed(e, 0, tok, [2300, 1]), want, precise, factor)
     check(feed(e, 1, tok, [700, 1, 2, 900, 64]), want, precise, factor)
+    check(feed(e, 1, tok, [3, 1100, 1, 1030, 64]), want, precise, factor)
 
 
 SIZES = {
@@ -271,6 +272,8 @@ SIZES = {
     "many_heads": xm.config([xm.attention(heads=40, kv=2, dim=16, dims=16, size=24),
                              xm.retention(heads=24, dim=8, vdim=16, dims=4, mlp=xm.moe(experts=33, top=8))],
                             vocab=128, width=192, eps=1e-2, softcap=4.0),
+    "attention_of_many_heads": xm.config([xm.attention(heads=h, kv=g, dim=64, dims=d, size=50, scale=0.1)
+                                          for h, g, d in ((48, 16, 64), (64, 32, 32), (96, 48, 60))], width=40),
     "wide_heads": xm.config([xm.attention(heads=4, kv=4, dim=96, dims=96, size=60, scale=0.1),
                              xm.attention(heads=8, kv=1, dim=128, dims=64, size=90, scale=0.09, scaling=xm.YARN)],
                             width=256),
