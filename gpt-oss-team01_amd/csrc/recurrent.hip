@@ -4,11 +4,11 @@
 //
 // The recurrence of a head acts on a K x V state whose V columns are independent of each other, so a
 // column lives in 8 lanes of a wave (K / 8 rows each, in registers) and a wave owns 16 columns (8 where
-// there is little to share out): for a step of one token the launch streams every state once through the chip, 16 bytes per lane and
-// request; for a stretch of a prompt the state stays in registers while the tokens go by, their keys,
-// queries and gates staged in LDS and shared by the workgroup's columns.  Everything is fp32, and
-// the tokens are taken one after the other, so a sequence's results are bit for bit the same however
-// it is cut into steps.
+// there is little to share out): for a step of one token the launch streams every state once through
+// the chip, 16 bytes per lane and request; for a stretch of a prompt the state stays in registers while
+// the tokens go by, their keys, queries and gates staged in LDS and shared by the workgroup's columns.
+// Everything is fp32, and the tokens are taken one after the other, so a sequence's results are bit for
+// bit the same however it is cut into steps.  Long stretches of retention run in retention.hip instead.
 #include <type_traits>
 
 #include "recurrent.hpp"
